@@ -72,6 +72,7 @@ extern "C" {
 
 #define TEAL_F16 0
 #define TEAL_BF16 1
+#define TEAL_F32 2 /* the layered designs' entry points only (teal_layer_*, teal_gated_act, teal_logit_softcap, teal_latent_*) */
 
 int teal_version(void);
 const char* teal_strerror(int code);
@@ -376,6 +377,58 @@ int teal_prefill_resid_norm(const void* emb, const int32_t* tokens, int T, const
  * cache rows 0 .. T-1 written, causal softmax(q K^T / sqrt(d)) V -> yt [n_head * head_dim][8].  head_dim 64 or 128. */
 int teal_prefill_attention(const float* qkv_slabs, int split, const void* rope, void* k_cache, void* v_cache, void* yt, int T, int n_head,
                            int n_kv_head, int head_dim, int max_seq, int dtype, void* stream);
+
+/* ---- layered decoder designs: row kernels around their matrix products, teal_amd/csrc/teal_layered.hip ----------------
+ * dtype 0 / 1 / 2 (fp16, bf16, fp32) = activations and weights; the residual stream is always fp32. */
+
+/* Per row r (= rows[i], or i): x[r] = embed[tokens[r]] | x[r], plus y[r] (+ y_bias) — RMS-normed with post_w first when post_w is
+ * given — and then h[i] = x[r] / sqrt(mean(x[r]^2) + eps) * pre_w (rounded once).  tokens / y / post_w / pre_w are optional; h is
+ * packed [n_rows][dim].  Token ids are clamped to the table.  dim <= 15360. */
+int teal_layer_resid_norm(float* x, int n_rows, int dim, const int32_t* tokens, const void* embed, int vocab, const void* y, int ldy,
+                          const void* y_bias, const void* post_w, const void* pre_w, float eps, void* h, const int32_t* rows, int dtype,
+                          void* stream);
+#define TEAL_ACT_SILU 0
+#define TEAL_ACT_GELU_TANH 1
+/* h[t][n] = act(gu[t][n] + bias_gate[n]) * (gu[t][up0 + n] + bias_up[n]), n < n_cols; the biases are optional */
+int teal_gated_act(const void* gu, int ldg, int up0, const void* bias_gate, const void* bias_up, void* h, int ldh, int n_rows, int n_cols,
+                   int act, int dtype, void* stream);
+/* out (fp32 [n_rows][vocab]) = cap * tanh(logits / cap); cap <= 0: the conversion alone */
+int teal_logit_softcap(const void* logits, int ld, float* out, int n_rows, int vocab, float cap, int dtype, void* stream);
+
+/* ---- latent attention, teal_amd/csrc/teal_latent.hip -------------------------------------------------------------------
+ * Sizes: heads; per head dim unrotated + rot rotated query / key dimensions and vdim value dimensions; rank = size of the latent.
+ * proj rows: [q (heads x (dim + rot)) | ... | latent (rank), shared key part (rot) at column kv0]; kv0 < 0: the layer reads another
+ * layer's cache and writes none.  Cache: rows of ldc elements [latent | rotated key part | padding], pages of 2^page_shift rows;
+ * table [slots][max_pages] holds a sequence slot's page ids.  inv_freq [rot / 2]: angle of pair i at position p = p * inv_freq[i].
+ * window: a query at p sees p - window < j <= p.  sink [heads], gate [..][heads * vdim] optional.  dtype 0 / 1 / 2. */
+
+/* prompt pass: rotate the queries in place; write the cache row row[t] of every token (RMS-normed latent, rotated key part) */
+int teal_latent_prompt_rows(void* proj, int ldp, int kv0, int n_tokens, const int32_t* pos, const int32_t* row, const float* inv_freq, const void* norm_w,
+                            float eps, int heads, int dim, int rot, int rank, void* cache, int ldc, int dtype, void* stream);
+/* packed copies c [n_rows][rank], kr [n_rows][rot] of cache rows row[i] (row[i] < 0: zeros) */
+int teal_latent_gather(const void* cache, int ldc, const int32_t* row, int n_rows, int rank, int rot, void* c, void* kr, int dtype, void* stream);
+/* queries per workgroup of the attention launch over prompts whose longest portion is n_queries (1: the scalar kernel) */
+int teal_latent_prompt_tile(int dim, int rot, int vdim, int n_queries, int dtype);
+/* attention over expanded keys k [n_keys][heads * dim], kr [n_keys][rot] and values vt [heads * vdim][n_keys] (n_keys % 8 == 0).
+ * seqs: int32 [..][5] = first query row, queries, position of the first query, packed key row of position klo (a multiple of 64,
+ * every sequence's span padded to a multiple of 64), klo; tiles: int32 [n_tiles][2] = sequence, first query (a multiple of tile).
+ * out [..][ldo] = attention output * sigmoid(gate). */
+int teal_latent_prompt_attention(const void* q, int ldq, const void* k, const void* kr, const void* vt, int n_keys, const void* sink, const void* gate,
+                                 int ldg, void* out, int ldo, const int32_t* seqs, const int32_t* tiles, int n_tiles, int tile, int heads, int dim, int rot,
+                                 int vdim, int window, float scale, int dtype, void* stream);
+/* one token per sequence: the absorbed, rotated query -> qcat [batch][heads][ldq] (fp32) or [batch][heads][2][ldq] (16-bit: high and
+ * low halves), ldq % 32 == 0; the token's cache row at position pos[b] of slot[b].  uk [heads * dim][rank]. */
+int teal_latent_step_query(const void* proj, int ldp, int kv0, int batch, const int32_t* pos, const int32_t* slot, const int32_t* table, int max_pages, int page_shift,
+                           const float* inv_freq, const void* norm_w, float eps, const void* uk, int heads, int dim, int rot, int rank, void* cache, int ldc, void* qcat,
+                           int ldq, int dtype, void* stream);
+/* ... partial attention over the cached rows of the window, split over `splits` workgroups per 16 heads:
+ * part fp32 [batch][heads][splits][rank + 2] = {max of the scaled scores in log2 units, sum, weighted latent} */
+int teal_latent_step_attention(const void* qcat, int ldq, const void* cache, int ldc, const int32_t* pos, const int32_t* slot, const int32_t* table, int max_pages,
+                               int page_shift, int batch, int heads, int rank, int rot, int window, float scale, int splits, float* part, size_t part_bytes, int dtype,
+                               void* stream);
+/* ... and y [batch][ldy] = (W_uv,head (merged latent)) * sigmoid(gate); uv [heads * vdim][rank] */
+int teal_latent_step_merge(const float* part, int splits, const void* uv, const void* sink, const void* gate, int ldg, void* y, int ldy, int batch, int heads, int rank,
+                           int vdim, int dtype, void* stream);
 
 /* ---- benchmark comparator (scripts/benchmark_gemv.py only; not on the decode path) ----------- */
 

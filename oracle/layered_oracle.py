@@ -1,0 +1,104 @@
+"""Plain, slow restatement of the layered decoder designs (CPU, one function per mechanism, float64 unless told otherwise).
+
+TEST INFRASTRUCTURE ONLY: shares no code with teal_amd/.  A model is (config dict, tensor dict): the parsed config.json and
+the checkpoint's tensors by name.  Everything is computed for ONE sequence, all positions at once, with explicit loops over
+queries and heads and no cache; a test compares the framework's cached / batched / fused steps with it.
+
+Notation: h row vectors [T, width]; p, j positions; W [out, in].
+"""
+from __future__ import annotations
+
+import math
+
+import torch
+
+
+def rms_norm(x, w, eps):
+    """x / sqrt(mean(x^2) + eps) * w along the last axis."""
+    return x / torch.sqrt((x * x).mean(dim=-1, keepdim=True) + eps) * w
+
+
+def gelu_tanh(z):
+    return 0.5 * z * (1.0 + torch.tanh(math.sqrt(2.0 / math.pi) * (z + 0.044715 * z ** 3)))
+
+
+def rotate_pairs(x, positions, dims, base):
+    """Adjacent pairs (2i, 2i+1) of the first `dims` entries of x [T, ..., n] turn by position * base^(-2i/dims)."""
+    out = x.clone()
+    for i in range(dims // 2):
+        ang = positions.to(x.dtype) * (float(base) ** (-2.0 * i / dims))
+        shape = [-1] + [1] * (x.dim() - 2)
+        c, s = torch.cos(ang).view(shape), torch.sin(ang).view(shape)
+        u, v = x[..., 2 * i], x[..., 2 * i + 1]
+        out[..., 2 * i] = u * c - v * s
+        out[..., 2 * i + 1] = v * c + u * s
+    return out
+
+
+def window_keys(p, size):
+    """Positions a query at p sees: itself and the size - 1 before it (size None: all before it)."""
+    lo = 0 if size is None else max(0, p - int(size) + 1)
+    return range(lo, p + 1)
+
+
+def softmax_with_sink(scores, sink):
+    """Weights of the given scores when the denominator also holds exp(sink)."""
+    m = max(float(scores.max()), float(sink))
+    e = torch.exp(scores - m)
+    return e / (e.sum() + math.exp(float(sink) - m))
+
+
+def latents(h, W, name, a, eps, start=0):
+    """(latent c [T, kv_rank], rotated shared key part [T, rot_dim]) a layer that owns its latents leaves for its keys."""
+    kv = h @ W[name + ".dkv"].T
+    c = rms_norm(kv[:, : a["kv_rank"]], W[name + ".dkv.norm"], eps)
+    pos = torch.arange(start, start + h.shape[0])
+    return c, rotate_pairs(kv[:, a["kv_rank"]:], pos, a["rot"]["dims"], a["rot"]["base"])
+
+
+def latent_attention(h, c, kr, W, name, a):
+    """Mixer output [T, width] for inputs h [T, width] and the latents (c, kr) of the same positions."""
+    T, H, D, R, V = h.shape[0], a["heads"], a["dim"], a["rot_dim"], a["vdim"]
+    q = (h @ W[name + ".q"].T).view(T, H, D + R)
+    qr = rotate_pairs(q[..., D:], torch.arange(T), a["rot"]["dims"], a["rot"]["base"])
+    k = (c @ W[name + ".uk"].T).view(T, H, D)
+    v = (c @ W[name + ".uv"].T).view(T, H, V)
+    size = (a.get("mask") or {}).get("size")
+    o = torch.zeros(T, H, V, dtype=h.dtype)
+    for p in range(T):
+        keys = window_keys(p, size)
+        sl = slice(keys.start, keys.stop)
+        for n in range(H):
+            s = (k[sl, n] @ q[p, n, :D] + kr[sl] @ qr[p, n]) * a["scale"]
+            o[p, n] = softmax_with_sink(s, W[name + ".sink"][n]) @ v[sl, n]
+    gate = torch.sigmoid(h @ W[name + ".g"].T)
+    return (o.reshape(T, H * V) * gate) @ W[name + ".o"].T
+
+
+def dense_mlp(h, W, name):
+    g = gelu_tanh(h @ W[name + ".gate"].T + W[name + ".gate.b"])
+    return (g * (h @ W[name + ".up"].T + W[name + ".up.b"])) @ W[name + ".down"].T + W[name + ".down.b"]
+
+
+def forward(cfg, tensors, tokens, dtype=torch.float64, layers_out=None):
+    """Logits [T, vocab] of one sequence; `layers_out`: a list that receives the residual stream after every layer."""
+    W = {k: t.to(dtype) for k, t in tensors.items()}
+    eps = cfg["norm"]["eps"]
+    x = W["embed"][torch.as_tensor(tokens, dtype=torch.long)]
+    kept = {}
+    for i, layer in enumerate(cfg["layers"]):
+        n, a = f"l{i}", layer["mixer"]
+        assert layer["type"] == "latent_attention"
+        h = rms_norm(x, W[n + ".norm1"], eps)
+        if a.get("kv_from") is None:
+            kept[i] = latents(h, W, n + ".mix", a, eps)
+        c, kr = kept[i if a.get("kv_from") is None else a["kv_from"]]
+        x = x + rms_norm(latent_attention(h, c, kr, W, n + ".mix", a), W[n + ".norm1b"], eps)
+        if layer.get("mlp"):
+            assert layer["mlp"]["kind"] == "dense"
+            x = x + rms_norm(dense_mlp(rms_norm(x, W[n + ".norm2"], eps), W, n + ".mlp"), W[n + ".norm2b"], eps)
+        if layers_out is not None:
+            layers_out.append(x.clone())
+    logits = rms_norm(x, W["final.norm"], eps) @ W["embed"].T
+    cap = cfg.get("logit_softcap")
+    return logits if cap is None else cap * torch.tanh(logits / cap)

@@ -154,6 +154,7 @@ DeviceCtx* device_ctx() {
         return nullptr;
     }
     c->gqa_lds_ok = attention_device_init();
+    c->latent_lds_ok = latent_device_init();
     c->num_cu = cu;
     return c;
 }
@@ -571,7 +572,7 @@ const char* teal_strerror(int code) {
     switch (code) {
         case TEAL_OK: return "ok";
         case TEAL_ERR_ARG: return "bad argument (null pointer or non-positive size)";
-        case TEAL_ERR_DTYPE: return "unsupported dtype (0 = fp16, 1 = bf16)";
+        case TEAL_ERR_DTYPE: return "unsupported dtype (0 = fp16, 1 = bf16; 2 = fp32 where an entry point says so)";
         case TEAL_ERR_SHAPE: return "unsupported shape (need N % 8 == 0, Z <= 65536, segment sizes % 8 == 0)";
         case TEAL_ERR_ALIGN: return "pointer not sufficiently aligned (weights/workspace 16 B)";
         case TEAL_ERR_WORKSPACE: return "split-K workspace missing or too small (teal_workspace_bytes)";

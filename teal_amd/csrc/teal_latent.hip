@@ -1,0 +1,869 @@
+// teal_latent.hip — latent attention (one low-rank latent per token shared by all heads, plus one rotated key part) for
+// gfx950 / CDNA4, wave64.  Per token and layer the cache holds ONE row [c (rank) | rotated key part (rot)], padded to a multiple
+// of 32 elements; pages of 2^shift rows, a page table per sequence slot.
+//
+//   score(p, j, head) = (q_head . k_head(j) + rotate(qr_head, p) . kr(j)) * scale,   k_head = W_uk,head c,  v_head = W_uv,head c
+//   weights: softmax over the keys p - window < j <= p, optionally with exp(sink_head) in the denominator
+//   y_head = (sum_j weight_j v_head(j)) [* sigmoid(gate_head)]
+//
+// Prompts run in the EXPANDED form (keys and values of every head from two matrix products over the packed latents, then a flash
+// attention over matrix-core tiles); single tokens run in the ABSORBED form: W_uk moves to the query side (q_abs = W_uk^T q, one
+// vector of the latent's size per head), the attention works on the cached rows themselves — each row is read once for sixteen
+// heads — and W_uv is applied to the weighted latent.
+//
+// Precision: scores, softmax weights and sums are fp32.  Where fp32 values meet the 16-bit matrix cores (the absorbed query, the
+// softmax weights) they are carried as a high and a low 16-bit half and multiplied twice: the products see ~16 bits of mantissa.
+// With 32-bit elements the scalar kernels run instead: plain fp32 multiply-adds.
+#include "teal_layered.h"
+
+namespace teal {
+
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef _Float16 f16x8 __attribute__((ext_vector_type(8)));
+constexpr float kLog2e = 1.4426950408889634f;
+
+template <bool BF16>
+__device__ __forceinline__ f32x4 mfma16(const u32x4 a, const u32x4 b, const f32x4 c) {
+    if constexpr (BF16) return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
+    else return __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(f16x8, a), __builtin_bit_cast(f16x8, b), c, 0, 0, 0);
+}
+
+// v as a high and a low 16-bit half
+template <bool BF16>
+__device__ __forceinline__ void split16(const float v, uint32_t& hi, uint32_t& lo) {
+    hi = float_to_bits<BF16>(v);
+    lo = float_to_bits<BF16>(v - bits_to_float(hi, BF16));
+}
+
+// ------------------------------------------------------------------------------------------------
+// Prompt pass, part 1: one workgroup per token.  Rotates the queries' rotated parts in place and, for a layer that owns its
+// latents, writes the token's cache row: RMSNorm(latent) * w and the rotated shared key part.
+// ------------------------------------------------------------------------------------------------
+struct LatentRowArgs {
+    void* proj;            // [T][ldp]: q at column 0 (heads x (dim + rot)), the latent and the shared key part at column kv0
+    const int32_t* pos;    // [T]
+    const int32_t* row;    // [T] cache row (or null with kv0 < 0)
+    const float* inv_freq; // [rot / 2]
+    const void* norm_w;    // [rank]
+    void* cache;           // [rows][ldc]
+    int ldp, kv0, heads, dim, rot, rank, ldc;
+    float eps;
+};
+
+template <int DT>
+__device__ __forceinline__ void latent_row(const LatentRowArgs& a, const typename Num<DT>::S* __restrict__ kv, const int p,
+                                           typename Num<DT>::S* __restrict__ out, float* red, const int tid) {
+    using N = Num<DT>;
+    float ss = 0.0f;
+    for (int i = tid; i < a.rank; i += 256) {
+        const float v = N::ld(kv + i);
+        ss = fmaf(v, v, ss);
+    }
+    const float rstd = 1.0f / sqrtf(block_sum<256>(ss, red, tid) / (float)a.rank + a.eps);
+    const typename N::S* w = reinterpret_cast<const typename N::S*>(a.norm_w);
+    for (int i = tid; i < a.rank; i += 256) out[i] = N::cvt(N::ld(kv + i) * rstd * N::ld(w + i));
+    for (int i = tid; i < a.rot / 2; i += 256) {
+        float x, y;
+        rotate_pair(N::ld(kv + a.rank + 2 * i), N::ld(kv + a.rank + 2 * i + 1), p, a.inv_freq[i], x, y);
+        out[a.rank + 2 * i] = N::cvt(x);
+        out[a.rank + 2 * i + 1] = N::cvt(y);
+    }
+}
+
+template <int DT>
+__global__ __launch_bounds__(256) void latent_prompt_rows_kernel(const LatentRowArgs a) {
+    using N = Num<DT>;
+    using S = typename N::S;
+    __shared__ float red[4];
+    const int tid = threadIdx.x, p = a.pos[blockIdx.x], half = a.rot / 2;
+    S* proj = reinterpret_cast<S*>(a.proj) + (size_t)blockIdx.x * a.ldp;
+    for (int i = tid; i < a.heads * half; i += 256) {
+        const int h = i / half, j = i - h * half;
+        S* q = proj + h * (a.dim + a.rot) + a.dim + 2 * j;
+        float x, y;
+        rotate_pair(N::ld(q), N::ld(q + 1), p, a.inv_freq[j], x, y);
+        q[0] = N::cvt(x);
+        q[1] = N::cvt(y);
+    }
+    if (a.kv0 >= 0) latent_row<DT>(a, proj + a.kv0, p, reinterpret_cast<S*>(a.cache) + (size_t)a.row[blockIdx.x] * a.ldc, red, tid);
+}
+
+// Prompt pass, part 2: the cache rows the prompt's queries can see, packed (row < 0: zeros) for the matrix products that expand them
+template <int DT>
+__global__ __launch_bounds__(64) void latent_gather_kernel(const typename Num<DT>::S* __restrict__ cache, const int ldc, const int32_t* __restrict__ row,
+                                                           const int rank, const int rot, typename Num<DT>::S* __restrict__ c, typename Num<DT>::S* __restrict__ kr) {
+    const int r = row[blockIdx.x];
+    const typename Num<DT>::S* src = cache + (size_t)max(r, 0) * ldc;
+    for (int i = threadIdx.x; i < rank + rot; i += 64) {
+        const typename Num<DT>::S v = r >= 0 ? src[i] : (typename Num<DT>::S)0;
+        if (i < rank) c[(size_t)blockIdx.x * rank + i] = v;
+        else kr[(size_t)blockIdx.x * rot + i - rank] = v;
+    }
+}
+
+// ------------------------------------------------------------------------------------------------
+// Prompt pass, part 3: flash attention over the expanded keys.
+// ------------------------------------------------------------------------------------------------
+struct SeqSpan {      // one sequence of the pass (five int32)
+    int q0, nq;       // its rows among the packed tokens
+    int start;        // position of its first row
+    int k0, klo;      // packed key row of position klo (a multiple of 8), the first position packed
+};
+
+struct LatentPromptArgs {
+    const void* q;      // [T][ldq], heads x (dim + rot), rotated
+    const void* k;      // [S][heads * dim]
+    const void* kr;     // [S][rot]
+    const void* vt;     // [heads * vdim][S]
+    const void* sink;   // or null: [heads]
+    const void* gate;   // or null: [T][ldg], heads x vdim
+    void* out;          // [T][ldo]
+    const SeqSpan* seqs;
+    const int32_t* tiles;  // [ntiles][2]: sequence, first query of the tile
+    int ldq, ldg, ldo, heads, dim, rot, vdim, S, window;
+    float scale;
+};
+
+// S^T = K Q^T per tile: a lane then holds four consecutive keys of ONE query, which is the layout the second product's operand
+// needs when the keys of two 16-key tiles are interleaved per lane group — the weights never cross lanes.  O^T = V^T P^T.
+template <bool BF16, int DQP, int DVP, int NQ, int BN>
+__global__ __launch_bounds__(256) void latent_prompt_attention_kernel(const LatentPromptArgs a) {
+    constexpr int KS = DQP / 32, KT = BN / 16, VT = DVP / 16, LK = DQP + 8, LV = BN + 8, BM = 64 * NQ;
+    __shared__ __align__(16) uint16_t ks[BN * LK];
+    __shared__ __align__(16) uint16_t vs[DVP * LV];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, g = lane >> 4;
+    const int head = blockIdx.y;
+    const SeqSpan sq = a.seqs[a.tiles[2 * blockIdx.x]];
+    const int q_first = a.tiles[2 * blockIdx.x + 1];
+    const int dq = a.dim + a.rot;
+    const uint16_t* kp = reinterpret_cast<const uint16_t*>(a.k);
+    const uint16_t* krp = reinterpret_cast<const uint16_t*>(a.kr);
+    const uint16_t* vp = reinterpret_cast<const uint16_t*>(a.vt) + (size_t)head * a.vdim * a.S;
+    const bool qvec = !(a.dim & 7) && !(a.rot & 7) && !(a.ldq & 7);
+    const bool kvec = !(a.dim & 7) && !(a.rot & 7);
+
+    u32x4 qf[NQ][KS];
+    int qpos[NQ];
+#pragma unroll
+    for (int n = 0; n < NQ; ++n) {
+        const int qi = q_first + (wave * NQ + n) * 16 + l16;
+        qpos[n] = qi < sq.nq ? sq.start + qi : -1;
+        const uint16_t* src = reinterpret_cast<const uint16_t*>(a.q) + (size_t)(sq.q0 + min(qi, sq.nq - 1)) * a.ldq + head * dq;
+#pragma unroll
+        for (int s = 0; s < KS; ++s) {
+            const int d0 = s * 32 + g * 8;
+            u32x4 w = {0u, 0u, 0u, 0u};
+            if (qvec) {
+                if (d0 < dq) w = *reinterpret_cast<const u32x4*>(src + d0);
+            } else {
+#pragma unroll
+                for (int j = 0; j < 8; ++j)
+                    if (d0 + j < dq) w[j >> 1] |= (uint32_t)src[d0 + j] << (16 * (j & 1));
+            }
+            qf[n][s] = w;
+        }
+    }
+    float m[NQ], l[NQ];
+    f32x4 o[NQ][VT];
+    const float sink2 = a.sink ? bits_to_float(reinterpret_cast<const uint16_t*>(a.sink)[head], BF16) * kLog2e : -INFINITY;
+#pragma unroll
+    for (int n = 0; n < NQ; ++n) {
+        m[n] = sink2;
+        l[n] = 0.0f;
+#pragma unroll
+        for (int v = 0; v < VT; ++v) o[n][v] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    const int last = sq.start + min(q_first + BM, sq.nq) - 1;           // position of the tile's last query
+    const int first = max(sq.klo, sq.start + q_first - a.window + 1);   // first position any of its queries sees
+    const float sc = a.scale * kLog2e;
+    for (int kt = (first - sq.klo) / BN * BN; sq.klo + kt <= last; kt += BN) {
+        __syncthreads();
+        for (int i = tid; i < BN * (DQP / 8); i += 256) {
+            const int key = i / (DQP / 8), d0 = (i % (DQP / 8)) * 8;
+            const size_t row = (size_t)min(sq.k0 + kt + key, a.S - 1);
+            u32x4 w = {0u, 0u, 0u, 0u};
+            if (kvec) {
+                if (d0 < a.dim) w = *reinterpret_cast<const u32x4*>(kp + (row * a.heads + head) * a.dim + d0);
+                else if (d0 < dq) w = *reinterpret_cast<const u32x4*>(krp + row * a.rot + d0 - a.dim);
+            } else {
+#pragma unroll
+                for (int j = 0; j < 8; ++j) {
+                    const int d = d0 + j;
+                    if (d < dq) w[j >> 1] |= (uint32_t)(d < a.dim ? kp[(row * a.heads + head) * a.dim + d] : krp[row * a.rot + d - a.dim]) << (16 * (j & 1));
+                }
+            }
+            *reinterpret_cast<u32x4*>(ks + key * LK + d0) = w;
+        }
+        for (int i = tid; i < DVP * (BN / 8); i += 256) {  // (S and every sequence's key base are multiples of 8: 16-byte loads)
+            const int v = i / (BN / 8), c0 = (i % (BN / 8)) * 8;
+            u32x4 w = {0u, 0u, 0u, 0u};
+            if (v < a.vdim && sq.k0 + kt + c0 < a.S) w = *reinterpret_cast<const u32x4*>(vp + (size_t)v * a.S + sq.k0 + kt + c0);
+            *reinterpret_cast<u32x4*>(vs + v * LV + c0) = w;
+        }
+        __syncthreads();
+        f32x4 s[NQ][KT];
+#pragma unroll
+        for (int t = 0; t < KT; ++t) {
+#pragma unroll
+            for (int n = 0; n < NQ; ++n) s[n][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int q = 0; q < KS; ++q) {
+                const u32x4 kf = *reinterpret_cast<const u32x4*>(ks + (t * 16 + l16) * LK + q * 32 + g * 8);
+#pragma unroll
+                for (int n = 0; n < NQ; ++n) s[n][t] = mfma16<BF16>(kf, qf[n][q], s[n][t]);
+            }
+        }
+        u32x4 ph[NQ][BN / 32], pl[NQ][BN / 32];
+#pragma unroll
+        for (int n = 0; n < NQ; ++n) {
+            float mx = m[n];
+#pragma unroll
+            for (int t = 0; t < KT; ++t)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const int kpos = sq.klo + kt + t * 16 + g * 4 + r;
+                    const bool ok = kpos <= qpos[n] && kpos > qpos[n] - a.window;
+                    s[n][t][r] = ok ? s[n][t][r] * sc : -INFINITY;
+                    mx = fmaxf(mx, s[n][t][r]);
+                }
+            mx = fmaxf(mx, __shfl_xor(mx, 16));
+            mx = fmaxf(mx, __shfl_xor(mx, 32));
+            const float ms = mx == -INFINITY ? 0.0f : mx;
+            const float al = exp2f(m[n] - ms);
+            m[n] = mx;
+            float ls = 0.0f;
+#pragma unroll
+            for (int b = 0; b < BN / 32; ++b)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {  // word j of the operand: keys 2j, 2j + 1 of the lane's eight (tile 2b, then tile 2b + 1)
+                    const float p0 = exp2f(s[n][2 * b + (j >> 1)][2 * (j & 1)] - ms), p1 = exp2f(s[n][2 * b + (j >> 1)][2 * (j & 1) + 1] - ms);
+                    uint32_t h0, l0, h1, l1;
+                    split16<BF16>(p0, h0, l0);
+                    split16<BF16>(p1, h1, l1);
+                    ph[n][b][j] = h0 | (h1 << 16);
+                    pl[n][b][j] = l0 | (l1 << 16);
+                    ls += p0 + p1;
+                }
+            l[n] = l[n] * al + ls;
+#pragma unroll
+            for (int v = 0; v < VT; ++v) o[n][v] *= al;
+        }
+#pragma unroll
+        for (int b = 0; b < BN / 32; ++b)
+#pragma unroll
+            for (int v = 0; v < VT; ++v) {
+                const uint16_t* base = vs + (v * 16 + l16) * LV + b * 32 + g * 4;
+                const u32x2 w0 = *reinterpret_cast<const u32x2*>(base), w1 = *reinterpret_cast<const u32x2*>(base + 16);
+                const u32x4 vf = {w0[0], w0[1], w1[0], w1[1]};
+#pragma unroll
+                for (int n = 0; n < NQ; ++n) {
+                    o[n][v] = mfma16<BF16>(vf, ph[n][b], o[n][v]);
+                    o[n][v] = mfma16<BF16>(vf, pl[n][b], o[n][v]);
+                }
+            }
+    }
+#pragma unroll
+    for (int n = 0; n < NQ; ++n) {
+        float lt = l[n] + __shfl_xor(l[n], 16);
+        lt += __shfl_xor(lt, 32);
+        if (a.sink) lt += exp2f(sink2 - m[n]);
+        if (qpos[n] < 0) continue;
+        const float inv = 1.0f / lt;
+        const size_t t = (size_t)(sq.q0 + qpos[n] - sq.start);
+        uint16_t* out = reinterpret_cast<uint16_t*>(a.out) + t * a.ldo + head * a.vdim;
+        const uint16_t* gt = a.gate ? reinterpret_cast<const uint16_t*>(a.gate) + t * a.ldg + head * a.vdim : nullptr;
+        const bool ovec = !(a.vdim & 3) && !(a.ldo & 3) && !(a.ldg & 3);
+#pragma unroll
+        for (int v = 0; v < VT; ++v) {
+            const int d = v * 16 + g * 4;
+            if (d >= a.vdim) continue;
+            if (ovec) {
+                float r[4];
+#pragma unroll
+                for (int j = 0; j < 4; ++j) r[j] = o[n][v][j] * inv;
+                if (gt) {
+                    const u32x2 gw = *reinterpret_cast<const u32x2*>(gt + d);
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) r[j] *= sigmoid_f(bits_to_float(j & 1 ? gw[j >> 1] >> 16 : gw[j >> 1] & 0xFFFFu, BF16));
+                }
+                *reinterpret_cast<u32x2*>(out + d) = u32x2{(uint32_t)float_to_bits<BF16>(r[0]) | ((uint32_t)float_to_bits<BF16>(r[1]) << 16),
+                                                           (uint32_t)float_to_bits<BF16>(r[2]) | ((uint32_t)float_to_bits<BF16>(r[3]) << 16)};
+            } else {
+#pragma unroll
+                for (int j = 0; j < 4; ++j)
+                    if (d + j < a.vdim) out[d + j] = float_to_bits<BF16>(o[n][v][j] * inv * (gt ? sigmoid_f(bits_to_float(gt[d + j], BF16)) : 1.0f));
+            }
+        }
+    }
+}
+
+// The same attention without the matrix cores: 32-bit elements, or head sizes beyond the tiles.  One workgroup per (query, head).
+template <int DT>
+__global__ __launch_bounds__(256) void latent_prompt_attention_scalar_kernel(const LatentPromptArgs a) {
+    using N = Num<DT>;
+    using S = typename N::S;
+    extern __shared__ __align__(16) unsigned char smem[];
+    float* q = reinterpret_cast<float*>(smem);  // [dim + rot]
+    float* p = q + a.dim + a.rot;               // [256] weights of a chunk of keys
+    float* part = p + 256;                      // [256] partial sums
+    __shared__ float red[4];
+    const int tid = threadIdx.x, head = blockIdx.y, dq = a.dim + a.rot;
+    const SeqSpan sq = a.seqs[a.tiles[2 * blockIdx.x]];
+    const int qi = a.tiles[2 * blockIdx.x + 1], pos = sq.start + qi;
+    const S* src = reinterpret_cast<const S*>(a.q) + (size_t)(sq.q0 + qi) * a.ldq + head * dq;
+    for (int i = tid; i < dq; i += 256) q[i] = N::ld(src + i);
+    __syncthreads();
+    const S* kp = reinterpret_cast<const S*>(a.k);
+    const S* krp = reinterpret_cast<const S*>(a.kr);
+    const S* vp = reinterpret_cast<const S*>(a.vt) + (size_t)head * a.vdim * a.S;
+    const int first = max(sq.klo, pos - a.window + 1);
+    // pass 1: the largest score; pass 2: weights, their sum and the weighted values (scores are computed twice, nothing is rescaled)
+    auto score = [&](const int j) {
+        const size_t row = (size_t)(sq.k0 + j - sq.klo);
+        float s = 0.0f;
+        const S* k = kp + (row * a.heads + head) * a.dim;
+        for (int d = 0; d < a.dim; ++d) s = fmaf(q[d], N::ld(k + d), s);
+        for (int d = 0; d < a.rot; ++d) s = fmaf(q[a.dim + d], N::ld(krp + row * a.rot + d), s);
+        return s * a.scale;
+    };
+    const float sink = a.sink ? N::ld(reinterpret_cast<const S*>(a.sink) + head) : -INFINITY;
+    float mx = sink;
+    for (int j = first + tid; j <= pos; j += 256) mx = fmaxf(mx, score(j));
+    mx = block_max<256>(mx, red, tid);
+    float ls = 0.0f;
+    // thread (v, part): value column v of this round, one of the parts that share the keys of a chunk
+    const int rounds = (a.vdim + 255) / 256;
+    const int cols = min(a.vdim, 256), parts = 256 / cols;
+    for (int r = 0; r < rounds; ++r) {
+        const int v = r * 256 + tid % cols, pt = tid / cols;
+        float acc = 0.0f;
+        for (int j0 = first; j0 <= pos; j0 += 256) {
+            const int j = j0 + tid;
+            const float w = j <= pos ? expf(score(j) - mx) : 0.0f;
+            if (r == 0) ls += w;
+            __syncthreads();
+            p[tid] = w;
+            __syncthreads();
+            if (pt < parts && v < a.vdim)
+                for (int i = pt; i < min(256, pos - j0 + 1); i += parts) acc = fmaf(p[i], N::ld(vp + (size_t)v * a.S + sq.k0 + j0 + i - sq.klo), acc);
+        }
+        if (r == 0) ls = block_sum<256>(ls, red, tid) + (a.sink ? expf(sink - mx) : 0.0f);
+        __syncthreads();
+        part[tid] = acc;
+        __syncthreads();
+        if (tid < cols && v < a.vdim) {
+            float t = 0.0f;
+            for (int i = 0; i < parts; ++i) t += part[i * cols + tid];
+            const size_t tok = (size_t)(sq.q0 + qi);
+            t /= ls;
+            if (a.gate) t *= sigmoid_f(N::ld(reinterpret_cast<const S*>(a.gate) + tok * a.ldg + head * a.vdim + v));
+            reinterpret_cast<S*>(a.out)[tok * a.ldo + head * a.vdim + v] = N::cvt(t);
+        }
+    }
+}
+
+// ------------------------------------------------------------------------------------------------
+// Single tokens, part 1: grid (heads * chunks [+ 1], batch).  Workgroup (head, chunk): 128 columns of the absorbed query
+// W_uk,head^T q (chunk 0 also rotates the query's rotated part); the extra workgroup: the token's cache row.
+// qcat [batch][heads][ldq]: q_abs (rank), rotated part (rot), zeros up to ldq — one fp32 row, or a high and a low 16-bit row.
+// ------------------------------------------------------------------------------------------------
+struct LatentStepArgs {
+    LatentRowArgs kv;        // proj = [batch][ldp]; pos per batch entry; cache of the layer (kv0 < 0: another layer's, untouched)
+    const int32_t* slot;     // [batch] page-table row
+    const int32_t* table;    // [slots][max_pages]
+    const void* uk;          // [heads * dim][rank]
+    void* qcat;
+    int max_pages, shift, chunks, ldq;
+};
+
+template <int DT>
+__global__ __launch_bounds__(256) void latent_step_query_kernel(const LatentStepArgs a) {
+    using N = Num<DT>;
+    using S = typename N::S;
+    extern __shared__ __align__(16) unsigned char smem[];
+    float* q = reinterpret_cast<float*>(smem);  // [dim]
+    __shared__ float red[4], part[16][129];
+    const LatentRowArgs& k = a.kv;
+    const int tid = threadIdx.x, b = blockIdx.y, p = k.pos[b];
+    const S* proj = reinterpret_cast<const S*>(k.proj) + (size_t)b * k.ldp;
+    if ((int)blockIdx.x == k.heads * a.chunks) {
+        const int row = page_row(a.table + (size_t)a.slot[b] * a.max_pages, min(p, (a.max_pages << a.shift) - 1), a.shift);
+        latent_row<DT>(k, proj + k.kv0, p, reinterpret_cast<S*>(k.cache) + (size_t)row * k.ldc, red, tid);
+        return;
+    }
+    const int head = blockIdx.x / a.chunks, r0 = (blockIdx.x % a.chunks) * 128;
+    const S* qh = proj + head * (k.dim + k.rot);
+    for (int i = tid; i < k.dim; i += 256) q[i] = N::ld(qh + i);
+    __syncthreads();
+    const int c0 = (tid & 15) * 8, dg = tid >> 4;
+    const S* w = reinterpret_cast<const S*>(a.uk) + (size_t)head * k.dim * k.rank + r0 + c0;
+    float acc[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) acc[j] = 0.0f;
+    const int left = k.rank - r0 - c0;
+    if (left >= 8) {
+        const bool vec = !(k.rank & 7);
+#pragma unroll 4
+        for (int d = dg; d < k.dim; d += 16) {
+            float v[8];
+            ld8<DT>(w + (size_t)d * k.rank, v, vec);
+#pragma unroll
+            for (int j = 0; j < 8; ++j) acc[j] = fmaf(q[d], v[j], acc[j]);
+        }
+    } else if (left > 0) {
+        for (int d = dg; d < k.dim; d += 16)
+            for (int j = 0; j < left; ++j) acc[j] = fmaf(q[d], N::ld(w + (size_t)d * k.rank + j), acc[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) part[dg][c0 + j] = acc[j];
+    __syncthreads();
+    auto put = [&](const int i, const float v) {  // element i of this head's row
+        const size_t at = (size_t)b * k.heads + head;
+        if constexpr (DT == TEAL_F32) {
+            reinterpret_cast<float*>(a.qcat)[at * a.ldq + i] = v;
+        } else {
+            uint32_t hi, lo;
+            split16<DT == TEAL_BF16>(v, hi, lo);
+            reinterpret_cast<uint16_t*>(a.qcat)[at * 2 * a.ldq + i] = (uint16_t)hi;
+            reinterpret_cast<uint16_t*>(a.qcat)[(at * 2 + 1) * a.ldq + i] = (uint16_t)lo;
+        }
+    };
+    if (tid < 128 && r0 + tid < k.rank) {
+        float t = 0.0f;
+#pragma unroll
+        for (int i = 0; i < 16; ++i) t += part[i][tid];
+        put(r0 + tid, t);
+    }
+    if (r0 == 0) {
+        for (int i = tid; i < k.rot / 2; i += 256) {
+            float x, y;
+            rotate_pair(N::ld(qh + k.dim + 2 * i), N::ld(qh + k.dim + 2 * i + 1), p, k.inv_freq[i], x, y);
+            put(k.rank + 2 * i, x);
+            put(k.rank + 2 * i + 1, y);
+        }
+        for (int i = k.rank + k.rot + tid; i < a.ldq; i += 256) put(i, 0.0f);
+    }
+}
+
+// ------------------------------------------------------------------------------------------------
+// Single tokens, part 2: attention over the cached rows.  grid (splits, 16-head groups, batch), four waves.  A split takes a run of
+// 32-key tiles of the window.  Per tile: the waves share the score product by its inner dimension (both 16-key tiles, K steps
+// wave, wave + 4, ...; partial scores through LDS), then each wave owns a quarter of the latent's columns in the value product.
+// The tile's rows are staged transposed ([column][key]) for that product; the score product's operand comes straight from memory.
+// part [batch][heads][splits][rank + 2] = {max (log2 units), sum, weighted latent}.
+// ------------------------------------------------------------------------------------------------
+struct LatentDecodeArgs {
+    const void* qcat;
+    const void* cache;
+    const int32_t* pos;
+    const int32_t* slot;
+    const int32_t* table;
+    float* part;
+    int max_pages, shift, ldq, ldc, heads, rank, rot, window, splits;
+    float scale;
+};
+
+struct KeyRange { int lo, hi; };  // first position, one past the last
+
+// the share of [max(0, p - window + 1), p] a split takes: whole tiles of `tile` keys, aligned in position
+__device__ __forceinline__ KeyRange split_range(const int p, const int window, const int split, const int splits, const int tile) {
+    const int lo = max(0, p - window + 1);
+    const int t0 = lo / tile, nt = p / tile - t0 + 1;
+    const int per = (nt + splits - 1) / splits;
+    KeyRange r;
+    r.lo = max(lo, (t0 + split * per) * tile);
+    r.hi = min(p + 1, (t0 + (split + 1) * per) * tile);
+    return r;
+}
+
+template <bool BF16, int RT>
+__global__ __launch_bounds__(256) void latent_decode_attention_kernel(const LatentDecodeArgs a) {
+    constexpr int RPW = RT / 4, LT = 36;  // 16-column tiles per wave; row stride (keys) of the transposed tile
+    extern __shared__ __align__(16) unsigned char smem[];
+    const int LQ = a.ldq + 8;
+    uint16_t* qs = reinterpret_cast<uint16_t*>(smem);          // [2][16][LQ] high, low
+    uint16_t* ct = qs + 2 * 16 * LQ;                           // [RT * 16][LT]
+    float* sp = reinterpret_cast<float*>(ct + RT * 16 * LT);   // [4][2][64][4] partial scores (lane-major)
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, g = lane >> 4;
+    const int split = blockIdx.x, h0 = blockIdx.y * 16, b = blockIdx.z;
+    const int nh = min(16, a.heads - h0);
+    const int p = a.pos[b];
+    const int* table = a.table + (size_t)a.slot[b] * a.max_pages;
+    const int plast = (a.max_pages << a.shift) - 1;  // (a position past the table would read past it: clamp)
+    const KeyRange kr = split_range(min(p, plast), a.window, split, a.splits, 32);
+    for (int i = tid; i < 2 * 16 * (a.ldq / 8); i += 256) {
+        const int half = i / (16 * (a.ldq / 8)), rest = i % (16 * (a.ldq / 8)), h = rest / (a.ldq / 8), d0 = (rest % (a.ldq / 8)) * 8;
+        u32x4 w = {0u, 0u, 0u, 0u};
+        if (h < nh) w = *reinterpret_cast<const u32x4*>(reinterpret_cast<const uint16_t*>(a.qcat) + (((size_t)b * a.heads + h0 + h) * 2 + half) * a.ldq + d0);
+        *reinterpret_cast<u32x4*>(qs + (half * 16 + h) * LQ + d0) = w;
+    }
+    __syncthreads();
+    const uint16_t* cache = reinterpret_cast<const uint16_t*>(a.cache);
+    const float sc = a.scale * kLog2e;
+    const int ksteps = a.ldq / 32;
+    float m = -INFINITY, l = 0.0f;
+    f32x4 o[RPW];
+#pragma unroll
+    for (int r = 0; r < RPW; ++r) o[r] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int kp = tid & 15, cg = tid >> 4;  // staging: key pair, column group (8 columns, then every 128th)
+    for (int j0 = kr.lo / 32 * 32; j0 < kr.hi; j0 += 32) {
+        const int base = page_row(table, j0, a.shift);  // (a tile of 32 keys never crosses a page: pages hold 2^shift >= 32)
+        {   // rows of keys 2 kp, 2 kp + 1, transposed; keys outside the share read as zero (their rows may be another sequence's leftovers)
+            const bool in0 = j0 + 2 * kp >= kr.lo && j0 + 2 * kp < kr.hi, in1 = j0 + 2 * kp + 1 >= kr.lo && j0 + 2 * kp + 1 < kr.hi;
+            const uint16_t* r0 = cache + (size_t)(base + 2 * kp) * a.ldc;
+#pragma unroll
+            for (int i = 0; i < (RT + 7) / 8; ++i) {
+                const int c0 = (cg + 16 * i) * 8;
+                if (c0 < RT * 16) {
+                    u32x4 x = {0u, 0u, 0u, 0u}, y = {0u, 0u, 0u, 0u};
+                    if (c0 < a.ldc) {
+                        if (in0) x = *reinterpret_cast<const u32x4*>(r0 + c0);
+                        if (in1) y = *reinterpret_cast<const u32x4*>(r0 + a.ldc + c0);
+                    }
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) {
+                        *reinterpret_cast<uint32_t*>(ct + (c0 + 2 * j) * LT + 2 * kp) = (x[j] & 0xFFFFu) | (y[j] << 16);
+                        *reinterpret_cast<uint32_t*>(ct + (c0 + 2 * j + 1) * LT + 2 * kp) = (x[j] >> 16) | (y[j] & 0xFFFF0000u);
+                    }
+                }
+            }
+        }
+        f32x4 s[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+        for (int q = wave; q < ksteps; q += 4) {
+            const u32x4 qh = *reinterpret_cast<const u32x4*>(qs + l16 * LQ + q * 32 + g * 8);
+            const u32x4 ql = *reinterpret_cast<const u32x4*>(qs + (16 + l16) * LQ + q * 32 + g * 8);
+#pragma unroll
+            for (int t = 0; t < 2; ++t) {
+                const u32x4 kf = *reinterpret_cast<const u32x4*>(cache + (size_t)(base + t * 16 + l16) * a.ldc + q * 32 + g * 8);
+                s[t] = mfma16<BF16>(kf, qh, s[t]);
+                s[t] = mfma16<BF16>(kf, ql, s[t]);
+            }
+        }
+#pragma unroll
+        for (int t = 0; t < 2; ++t) *reinterpret_cast<f32x4*>(sp + ((wave * 2 + t) * 64 + lane) * 4) = s[t];
+        __syncthreads();
+        float mx = m;
+#pragma unroll
+        for (int t = 0; t < 2; ++t) {
+            f32x4 v = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int w = 0; w < 4; ++w) v += *reinterpret_cast<const f32x4*>(sp + ((w * 2 + t) * 64 + lane) * 4);
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int j = j0 + t * 16 + g * 4 + r;
+                s[t][r] = (j >= kr.lo && j < kr.hi) ? v[r] * sc : -INFINITY;
+                mx = fmaxf(mx, s[t][r]);
+            }
+        }
+        mx = fmaxf(mx, __shfl_xor(mx, 16));
+        mx = fmaxf(mx, __shfl_xor(mx, 32));
+        const float ms = mx == -INFINITY ? 0.0f : mx;
+        const float al = exp2f(m - ms);
+        m = mx;
+        u32x4 ph, pl;
+        float ls = 0.0f;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const float p0 = exp2f(s[j >> 1][2 * (j & 1)] - ms), p1 = exp2f(s[j >> 1][2 * (j & 1) + 1] - ms);
+            uint32_t a0, b0, a1, b1;
+            split16<BF16>(p0, a0, b0);
+            split16<BF16>(p1, a1, b1);
+            ph[j] = a0 | (a1 << 16);
+            pl[j] = b0 | (b1 << 16);
+            ls += p0 + p1;
+        }
+        l = l * al + ls;
+#pragma unroll
+        for (int r = 0; r < RPW; ++r) {
+            const uint16_t* bp = ct + ((wave * RPW + r) * 16 + l16) * LT + g * 4;
+            const u32x2 w0 = *reinterpret_cast<const u32x2*>(bp), w1 = *reinterpret_cast<const u32x2*>(bp + 16);
+            const u32x4 cf = {w0[0], w0[1], w1[0], w1[1]};
+            o[r] *= al;
+            o[r] = mfma16<BF16>(cf, ph, o[r]);
+            o[r] = mfma16<BF16>(cf, pl, o[r]);
+        }
+        __syncthreads();
+    }
+    l += __shfl_xor(l, 16);
+    l += __shfl_xor(l, 32);
+    if (l16 < nh) {
+        float* out = a.part + (((size_t)b * a.heads + h0 + l16) * a.splits + split) * (a.rank + 2);
+        if (wave == 0 && g == 0) { out[0] = m; out[1] = l; }
+#pragma unroll
+        for (int r = 0; r < RPW; ++r)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int c = (wave * RPW + r) * 16 + g * 4 + j;
+                if (c < a.rank) out[2 + c] = o[r][j];
+            }
+    }
+}
+
+// The same without the matrix cores (32-bit elements, or ranks beyond the tiles): one workgroup per (split, head, batch entry)
+template <int DT>
+__global__ __launch_bounds__(256) void latent_decode_attention_scalar_kernel(const LatentDecodeArgs a) {
+    using N = Num<DT>;
+    using S = typename N::S;
+    extern __shared__ __align__(16) unsigned char smem[];
+    const int D = a.rank + a.rot;
+    float* q = reinterpret_cast<float*>(smem);  // [D]
+    float* o = q + D;                           // [rank]
+    __shared__ float pw[256], red[4];
+    __shared__ int rows[256];
+    const int tid = threadIdx.x, split = blockIdx.x, head = blockIdx.y, b = blockIdx.z;
+    const int p = min(a.pos[b], (a.max_pages << a.shift) - 1);
+    const int* table = a.table + (size_t)a.slot[b] * a.max_pages;
+    const size_t at = (size_t)b * a.heads + head;
+    for (int i = tid; i < D; i += 256) {
+        if constexpr (DT == TEAL_F32) q[i] = reinterpret_cast<const float*>(a.qcat)[at * a.ldq + i];
+        else q[i] = N::ld(reinterpret_cast<const S*>(a.qcat) + at * 2 * a.ldq + i) + N::ld(reinterpret_cast<const S*>(a.qcat) + (at * 2 + 1) * a.ldq + i);
+        if (i < a.rank) o[i] = 0.0f;
+    }
+    __syncthreads();
+    const KeyRange kr = split_range(p, a.window, split, a.splits, 32);
+    const S* cache = reinterpret_cast<const S*>(a.cache);
+    float m = -INFINITY, l = 0.0f;
+    for (int j0 = kr.lo; j0 < kr.hi; j0 += 256) {
+        const int j = j0 + tid, row = page_row(table, min(j, kr.hi - 1), a.shift);
+        float s = 0.0f;
+        const S* c = cache + (size_t)row * a.ldc;
+        for (int d = 0; d < D; ++d) s = fmaf(q[d], N::ld(c + d), s);
+        s = j < kr.hi ? s * a.scale * kLog2e : -INFINITY;
+        const float mx = fmaxf(m, block_max<256>(s, red, tid));
+        const float al = exp2f(m - mx), w = j < kr.hi ? exp2f(s - mx) : 0.0f;
+        m = mx;
+        l = l * al + block_sum<256>(w, red, tid);
+        pw[tid] = w;
+        rows[tid] = row;
+        __syncthreads();
+        const int n = min(256, kr.hi - j0);
+        for (int r = tid; r < a.rank; r += 256) {
+            float acc = o[r] * al;
+            for (int i = 0; i < n; ++i) acc = fmaf(pw[i], N::ld(cache + (size_t)rows[i] * a.ldc + r), acc);
+            o[r] = acc;
+        }
+        __syncthreads();
+    }
+    float* out = a.part + (at * a.splits + split) * (a.rank + 2);
+    if (tid == 0) { out[0] = m; out[1] = l; }
+    for (int r = tid; r < a.rank; r += 256) out[2 + r] = o[r];
+}
+
+// ------------------------------------------------------------------------------------------------
+// Single tokens, part 3: merge the splits (and the sink), apply W_uv and the gate.  grid (column chunks of 32, heads, batch).
+// ------------------------------------------------------------------------------------------------
+struct LatentMergeArgs {
+    const float* part;
+    const void* uv;     // [heads * vdim][rank]
+    const void* sink;   // or null: [heads]
+    const void* gate;   // or null: [batch][ldg], heads x vdim
+    void* y;            // [batch][ldy]
+    int heads, rank, vdim, splits, ldg, ldy;
+};
+
+template <int DT>
+__global__ __launch_bounds__(256) void latent_decode_merge_kernel(const LatentMergeArgs a) {
+    using N = Num<DT>;
+    using S = typename N::S;
+    extern __shared__ __align__(16) unsigned char smem[];
+    float* o = reinterpret_cast<float*>(smem);  // [rank rounded up to 8]
+    float* f = o + ((a.rank + 7) & ~7);         // [splits]
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, head = blockIdx.y, b = blockIdx.z;
+    const float* part = a.part + ((size_t)b * a.heads + head) * a.splits * (a.rank + 2);
+    const float sink2 = a.sink ? N::ld(reinterpret_cast<const S*>(a.sink) + head) * kLog2e : -INFINITY;
+    float M = sink2;
+    for (int s = 0; s < a.splits; ++s) M = fmaxf(M, part[(size_t)s * (a.rank + 2)]);
+    if (tid < a.splits) f[tid] = exp2f(part[(size_t)tid * (a.rank + 2)] - M);
+    __syncthreads();
+    float L = a.sink ? exp2f(sink2 - M) : 0.0f;
+    for (int s = 0; s < a.splits; ++s) L = fmaf(part[(size_t)s * (a.rank + 2) + 1], f[s], L);
+    const float inv = 1.0f / L;
+    for (int r = tid; r < ((a.rank + 7) & ~7); r += 256) {
+        float t = 0.0f;
+        if (r < a.rank)
+            for (int s = 0; s < a.splits; ++s) t = fmaf(part[(size_t)s * (a.rank + 2) + 2 + r], f[s], t);
+        o[r] = t * inv;
+    }
+    __syncthreads();
+    const int v0 = blockIdx.x * 32 + wave * 8, nv = min(8, a.vdim - v0);
+    if (nv <= 0) return;
+    const S* w = reinterpret_cast<const S*>(a.uv) + (size_t)(head * a.vdim + v0) * a.rank;
+    float acc[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) acc[i] = 0.0f;
+    const bool vec = !(a.rank & 7);
+    for (int c0 = lane * 8; c0 < a.rank; c0 += 512) {
+        const int m = min(8, a.rank - c0);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            const S* wr = w + (size_t)min(i, nv - 1) * a.rank + c0;
+            if (m == 8) {
+                float v[8];
+                ld8<DT>(wr, v, vec);
+#pragma unroll
+                for (int j = 0; j < 8; ++j) acc[i] = fmaf(v[j], o[c0 + j], acc[i]);
+            } else {
+                for (int j = 0; j < m; ++j) acc[i] = fmaf(N::ld(wr + j), o[c0 + j], acc[i]);
+            }
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < 8; ++i) acc[i] = wave_sum_f(acc[i]);
+    if (lane < nv) {
+        float t = acc[0];
+#pragma unroll
+        for (int i = 1; i < 8; ++i) t = lane == i ? acc[i] : t;
+        const int col = head * a.vdim + v0 + lane;
+        if (a.gate) t *= sigmoid_f(N::ld(reinterpret_cast<const S*>(a.gate) + (size_t)b * a.ldg + col));
+        reinterpret_cast<S*>(a.y)[(size_t)b * a.ldy + col] = N::cvt(t);
+    }
+}
+
+constexpr size_t kLatentMaxLds = 128 * 1024;
+
+// first use of a device (device_ctx()): the absorbed attention may take more than the default 64 KB of a CU's LDS
+bool latent_device_init() {
+    bool ok = true;
+#define TEAL_OPT(BF, RT) ok = ok && hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_decode_attention_kernel<BF, RT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)kLatentMaxLds) == hipSuccess
+    TEAL_OPT(false, 8); TEAL_OPT(false, 16); TEAL_OPT(false, 32); TEAL_OPT(true, 8); TEAL_OPT(true, 16); TEAL_OPT(true, 32);
+#undef TEAL_OPT
+    if (!ok) (void)hipGetLastError();
+    return ok;
+}
+
+inline size_t decode_lds(const int ldq, const int rt) { return (size_t)2 * 16 * (ldq + 8) * 2 + (size_t)rt * 16 * 36 * 2 + (size_t)4 * 2 * 64 * 4 * sizeof(float); }
+
+template <bool BF16, int NQ>
+int launch_prompt(const LatentPromptArgs& a, const int n_tiles, hipStream_t st) {
+    const int dq = a.dim + a.rot;
+    const dim3 grid(n_tiles, a.heads), block(256);
+#define TEAL_LP(DQ, DV, BN) do { hipLaunchKernelGGL((latent_prompt_attention_kernel<BF16, DQ, DV, NQ, BN>), grid, block, 0, st, a); return launched(); } while (0)
+#define TEAL_LP_V(DQ) do { if (a.vdim <= 64) TEAL_LP(DQ, 64, 64); if (a.vdim <= 128) TEAL_LP(DQ, 128, 64); if constexpr (NQ == 1) TEAL_LP(DQ, 256, 32); } while (0)
+    if (dq <= 64) TEAL_LP_V(64);
+    else if (dq <= 128) TEAL_LP_V(128);
+    else if (dq <= 192) TEAL_LP_V(192);
+    else if (dq <= 256) TEAL_LP_V(256);
+    return TEAL_ERR_SHAPE;
+#undef TEAL_LP_V
+#undef TEAL_LP
+}
+
+}  // namespace teal
+
+using namespace teal;
+
+extern "C" {
+
+int teal_latent_prompt_rows(void* proj, int ldp, int kv0, int n_tokens, const int32_t* pos, const int32_t* row, const float* inv_freq, const void* norm_w,
+                            float eps, int heads, int dim, int rot, int rank, void* cache, int ldc, int dtype, void* stream) {
+    if (!proj || !pos || n_tokens <= 0 || heads <= 0 || dim < 0 || rot < 0 || dim + rot <= 0 || (rot > 0 && !inv_freq)) return TEAL_ERR_ARG;
+    if (kv0 >= 0 && (!row || !norm_w || !cache || rank <= 0)) return TEAL_ERR_ARG;
+    if ((rot & 1) || ldp < heads * (dim + rot) || (kv0 >= 0 && (kv0 < heads * (dim + rot) || ldp < kv0 + rank + rot || ldc < rank + rot))) return TEAL_ERR_SHAPE;
+    const LatentRowArgs a = {proj, pos, row, inv_freq, norm_w, cache, ldp, kv0, heads, dim, rot, rank, ldc, eps};
+    hipStream_t st = reinterpret_cast<hipStream_t>(stream);
+    return with_dtype(dtype, [&](auto dt) {
+        hipLaunchKernelGGL((latent_prompt_rows_kernel<decltype(dt)::value>), dim3(n_tokens), dim3(256), 0, st, a);
+        return launched();
+    });
+}
+
+int teal_latent_gather(const void* cache, int ldc, const int32_t* row, int n_rows, int rank, int rot, void* c, void* kr, int dtype, void* stream) {
+    if (!cache || !row || !c || (rot > 0 && !kr) || n_rows <= 0 || rank <= 0 || rot < 0) return TEAL_ERR_ARG;
+    if (ldc < rank + rot) return TEAL_ERR_SHAPE;
+    hipStream_t st = reinterpret_cast<hipStream_t>(stream);
+    return with_dtype(dtype, [&](auto dt) {
+        using S = typename Num<decltype(dt)::value>::S;
+        hipLaunchKernelGGL((latent_gather_kernel<decltype(dt)::value>), dim3(n_rows), dim3(64), 0, st, reinterpret_cast<const S*>(cache), ldc, row, rank, rot,
+                           reinterpret_cast<S*>(c), reinterpret_cast<S*>(kr));
+        return launched();
+    });
+}
+
+int teal_latent_prompt_tile(int dim, int rot, int vdim, int n_queries, int dtype) {
+    if (dtype == TEAL_F32 || dim + rot > 256 || vdim > 256) return 1;  // the scalar kernel: one query per workgroup
+    return n_queries > 64 && vdim <= 128 ? 128 : 64;
+}
+
+int teal_latent_prompt_attention(const void* q, int ldq, const void* k, const void* kr, const void* vt, int n_keys, const void* sink, const void* gate,
+                                 int ldg, void* out, int ldo, const int32_t* seqs, const int32_t* tiles, int n_tiles, int tile, int heads, int dim, int rot,
+                                 int vdim, int window, float scale, int dtype, void* stream) {
+    if (!q || !k || (rot > 0 && !kr) || !vt || !out || !seqs || !tiles || n_tiles <= 0 || heads <= 0 || dim < 0 || rot < 0 || vdim <= 0 || window <= 0) return TEAL_ERR_ARG;
+    if (dim + rot <= 0 || dim + rot > 8192 || heads > 65535 || ldq < heads * (dim + rot) || ldo < heads * vdim || (gate && ldg < heads * vdim) || n_keys <= 0 || (n_keys & 7))
+        return TEAL_ERR_SHAPE;
+    if (tile != 1 && (dim + rot > 256 || vdim > 256 || (tile != 64 && tile != 128) || (tile == 128 && vdim > 128))) return TEAL_ERR_SHAPE;
+    if (tile != 1 && (!aligned16(q) || !aligned16(k) || !aligned16(kr) || !aligned16(vt) || (reinterpret_cast<uintptr_t>(gate) & 7u) || (reinterpret_cast<uintptr_t>(out) & 7u)))
+        return TEAL_ERR_ALIGN;
+    if (tile != 1 && dtype == TEAL_F32) return TEAL_ERR_DTYPE;
+    const LatentPromptArgs a = {q, k, kr, vt, sink, gate, out, reinterpret_cast<const SeqSpan*>(seqs), tiles, ldq, gate ? ldg : 0, ldo, heads, dim, rot, vdim, n_keys, window, scale};
+    hipStream_t st = reinterpret_cast<hipStream_t>(stream);
+    if (tile == 1)
+        return with_dtype(dtype, [&](auto dt) {
+            hipLaunchKernelGGL((latent_prompt_attention_scalar_kernel<decltype(dt)::value>), dim3(n_tiles, heads), dim3(256), (size_t)(dim + rot + 512) * sizeof(float), st, a);
+            return launched();
+        });
+    if (dtype == TEAL_BF16) return tile == 128 ? launch_prompt<true, 2>(a, n_tiles, st) : launch_prompt<true, 1>(a, n_tiles, st);
+    if (dtype == TEAL_F16) return tile == 128 ? launch_prompt<false, 2>(a, n_tiles, st) : launch_prompt<false, 1>(a, n_tiles, st);
+    return TEAL_ERR_DTYPE;
+}
+
+int teal_latent_step_query(const void* proj, int ldp, int kv0, int batch, const int32_t* pos, const int32_t* slot, const int32_t* table, int max_pages, int page_shift,
+                           const float* inv_freq, const void* norm_w, float eps, const void* uk, int heads, int dim, int rot, int rank, void* cache, int ldc, void* qcat,
+                           int ldq, int dtype, void* stream) {
+    if (!proj || !pos || !slot || !table || !uk || !qcat || batch <= 0 || heads <= 0 || dim <= 0 || rot < 0 || rank <= 0 || max_pages <= 0 || (rot > 0 && !inv_freq)) return TEAL_ERR_ARG;
+    if (kv0 >= 0 && (!norm_w || !cache)) return TEAL_ERR_ARG;
+    if ((rot & 1) || dim > 8192 || batch > 65535 || page_shift < 5 || page_shift > 20 || (ldq & 31) || ldq < rank + rot || ldp < heads * (dim + rot) ||
+        (kv0 >= 0 && (kv0 < heads * (dim + rot) || ldp < kv0 + rank + rot || ldc < rank + rot)))
+        return TEAL_ERR_SHAPE;
+    if (!aligned16(uk) || !aligned16(qcat)) return TEAL_ERR_ALIGN;
+    const int chunks = (rank + 127) / 128;
+    const LatentStepArgs a = {{const_cast<void*>(proj), pos, nullptr, inv_freq, norm_w, cache, ldp, kv0, heads, dim, rot, rank, ldc, eps}, slot, table, uk, qcat, max_pages, page_shift, chunks, ldq};
+    hipStream_t st = reinterpret_cast<hipStream_t>(stream);
+    return with_dtype(dtype, [&](auto dt) {
+        hipLaunchKernelGGL((latent_step_query_kernel<decltype(dt)::value>), dim3(heads * chunks + (kv0 >= 0 ? 1 : 0), batch), dim3(256), (size_t)dim * sizeof(float), st, a);
+        return launched();
+    });
+}
+
+int teal_latent_step_attention(const void* qcat, int ldq, const void* cache, int ldc, const int32_t* pos, const int32_t* slot, const int32_t* table, int max_pages,
+                               int page_shift, int batch, int heads, int rank, int rot, int window, float scale, int splits, float* part, size_t part_bytes, int dtype,
+                               void* stream) {
+    if (!qcat || !cache || !pos || !slot || !table || !part || batch <= 0 || heads <= 0 || rank <= 0 || rot < 0 || window <= 0 || max_pages <= 0) return TEAL_ERR_ARG;
+    if (splits < 1 || splits > 256 || batch > 65535 || heads > 65535 || page_shift < 5 || page_shift > 20 || (ldq & 31) || ldq < rank + rot || (ldc & 31) || ldc < rank + rot || rank + rot > 6144)
+        return TEAL_ERR_SHAPE;
+    if (!aligned16(qcat) || !aligned16(cache)) return TEAL_ERR_ALIGN;
+    if (part_bytes < (size_t)batch * heads * splits * (rank + 2) * sizeof(float)) return TEAL_ERR_WORKSPACE;
+    DeviceCtx* ctx = device_ctx();
+    if (!ctx) return TEAL_ERR_NO_DEVICE;
+    const LatentDecodeArgs a = {qcat, cache, pos, slot, table, part, max_pages, page_shift, ldq, ldc, heads, rank, rot, window, splits, scale};
+    hipStream_t st = reinterpret_cast<hipStream_t>(stream);
+    const int rt = rank <= 128 ? 8 : (rank <= 256 ? 16 : 32);
+    const size_t lds = decode_lds(ldq, rt);
+    if (dtype != TEAL_F32 && rank <= 512 && ldq == ldc && lds <= kLatentMaxLds && (lds <= 64 * 1024 || ctx->latent_lds_ok)) {
+        const dim3 grid(splits, (heads + 15) / 16, batch), block(256);
+#define TEAL_LD(BF, RT) hipLaunchKernelGGL((latent_decode_attention_kernel<BF, RT>), grid, block, lds, st, a)
+        if (dtype == TEAL_BF16) { if (rt == 8) TEAL_LD(true, 8); else if (rt == 16) TEAL_LD(true, 16); else TEAL_LD(true, 32); }
+        else if (dtype == TEAL_F16) { if (rt == 8) TEAL_LD(false, 8); else if (rt == 16) TEAL_LD(false, 16); else TEAL_LD(false, 32); }
+        else return TEAL_ERR_DTYPE;
+#undef TEAL_LD
+        return launched();
+    }
+    return with_dtype(dtype, [&](auto dt) {
+        hipLaunchKernelGGL((latent_decode_attention_scalar_kernel<decltype(dt)::value>), dim3(splits, heads, batch), dim3(256), (size_t)(2 * rank + rot) * sizeof(float), st, a);
+        return launched();
+    });
+}
+
+int teal_latent_step_merge(const float* part, int splits, const void* uv, const void* sink, const void* gate, int ldg, void* y, int ldy, int batch, int heads, int rank,
+                           int vdim, int dtype, void* stream) {
+    if (!part || !uv || !y || batch <= 0 || heads <= 0 || rank <= 0 || vdim <= 0 || splits < 1) return TEAL_ERR_ARG;
+    if (splits > 256 || rank > 8192 || batch > 65535 || heads > 65535 || ldy < heads * vdim || (gate && ldg < heads * vdim)) return TEAL_ERR_SHAPE;
+    if (!aligned16(uv)) return TEAL_ERR_ALIGN;
+    const LatentMergeArgs a = {part, uv, sink, gate, y, heads, rank, vdim, splits, ldg, ldy};
+    hipStream_t st = reinterpret_cast<hipStream_t>(stream);
+    return with_dtype(dtype, [&](auto dt) {
+        hipLaunchKernelGGL((latent_decode_merge_kernel<decltype(dt)::value>), dim3((vdim + 31) / 32, heads, batch), dim3(256), (size_t)(rank + 8 + splits) * sizeof(float), st, a);
+        return launched();
+    });
+}
+
+}  // extern "C"

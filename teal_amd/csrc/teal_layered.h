@@ -1,0 +1,97 @@
+// teal_layered.h — element types and small device helpers of the layered designs' kernels (teal_layered.hip, teal_latent.hip):
+// the same kernels in fp16, bf16 and true 32-bit.  Internal header; the public boundary is include/teal_hip.h.
+#pragma once
+#include "teal_common.h"
+
+namespace teal {
+
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+
+// dtype code -> storage type, conversions (fp32 <-> storage, round to nearest even)
+template <int DT>
+struct Num {
+    using S = uint16_t;
+    static __device__ __forceinline__ float ld(const S* p) { return bits_to_float(*p, DT == TEAL_BF16); }
+    static __device__ __forceinline__ S cvt(const float f) { return float_to_bits<DT == TEAL_BF16>(f); }
+};
+template <>
+struct Num<TEAL_F32> {
+    using S = float;
+    static __device__ __forceinline__ float ld(const S* p) { return *p; }
+    static __device__ __forceinline__ S cvt(const float f) { return f; }
+};
+
+// eight consecutive elements as fp32; `vec`: p is 16-byte aligned (32-bit elements: always element loads pairs of 16 bytes)
+template <int DT>
+__device__ __forceinline__ void ld8(const typename Num<DT>::S* __restrict__ p, float (&o)[8], const bool vec) {
+    if (vec) {
+        if constexpr (DT == TEAL_F32) {
+            const f32x4 a = *reinterpret_cast<const f32x4*>(p), b = *reinterpret_cast<const f32x4*>(p + 4);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) { o[j] = a[j]; o[4 + j] = b[j]; }
+        } else {
+            const u32x4 w = *reinterpret_cast<const u32x4*>(p);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) { o[2 * j] = bits_to_float(w[j] & 0xFFFFu, DT == TEAL_BF16); o[2 * j + 1] = bits_to_float(w[j] >> 16, DT == TEAL_BF16); }
+        }
+    } else {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) o[j] = Num<DT>::ld(p + j);
+    }
+}
+
+// sum over the NT threads of a workgroup (red: NT / 64 floats of LDS, free on entry after a barrier); every thread gets it
+template <int NT>
+__device__ __forceinline__ float block_sum(float v, float* red, const int tid) {
+    v = wave_sum_f(v);
+    __syncthreads();
+    if ((tid & 63) == 0) red[tid >> 6] = v;
+    __syncthreads();
+    float t = 0.0f;
+#pragma unroll
+    for (int w = 0; w < NT / 64; ++w) t += red[w];
+    return t;
+}
+
+template <int NT>
+__device__ __forceinline__ float block_max(float v, float* red, const int tid) {
+    v = wave_max_f(v);
+    __syncthreads();
+    if ((tid & 63) == 0) red[tid >> 6] = v;
+    __syncthreads();
+    float t = red[0];
+#pragma unroll
+    for (int w = 1; w < NT / 64; ++w) t = fmaxf(t, red[w]);
+    return t;
+}
+
+__device__ __forceinline__ float gelu_tanh_f(const float z) {
+    return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * fmaf(0.044715f * z * z, z, z)));
+}
+__device__ __forceinline__ float sigmoid_f(const float z) { return 1.0f / (1.0f + expf(-z)); }
+
+// rotation of one adjacent pair (u, v) by position * inv_freq, all in fp32
+__device__ __forceinline__ void rotate_pair(const float u, const float v, const int pos, const float inv_freq, float& a, float& b) {
+    float s, c;
+    sincosf((float)pos * inv_freq, &s, &c);
+    a = fmaf(u, c, -(v * s));
+    b = fmaf(v, c, u * s);
+}
+
+// cache row of position p of a sequence: its page table holds one page id per 2^shift positions
+__device__ __forceinline__ int page_row(const int* __restrict__ table, const int p, const int shift) {
+    return (table[p >> shift] << shift) + (p & ((1 << shift) - 1));
+}
+
+template <typename F>
+int with_dtype(const int dtype, F&& f) {
+    switch (dtype) {
+        case TEAL_F16: return f(std::integral_constant<int, TEAL_F16>{});
+        case TEAL_BF16: return f(std::integral_constant<int, TEAL_BF16>{});
+        case TEAL_F32: return f(std::integral_constant<int, TEAL_F32>{});
+        default: return TEAL_ERR_DTYPE;
+    }
+}
+inline int launched() { return hipGetLastError() == hipSuccess ? TEAL_OK : TEAL_ERR_LAUNCH; }
+
+}  // namespace teal

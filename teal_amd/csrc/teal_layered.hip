@@ -1,0 +1,236 @@
+// teal_layered.hip — row kernels of the layered decoder designs (teal_amd/gpt_fast/layered.py): what stands between two matrix
+// products of a block, with the residual stream held in fp32.  gfx950 / CDNA4, wave64; fp16, bf16 and true 32-bit activations.
+//
+//   resid_norm_kernel   x = embedding row | x + [post norm](y + bias), then h = RMSNorm(x) * w   (one workgroup per token)
+//   gated_act_kernel    h = act(gate + bias) * (up + bias)
+//   softcap_kernel      logits -> fp32, cap * tanh(logits / cap)
+#include "teal_layered.h"
+
+namespace teal {
+
+struct ResidNormArgs {
+    float* x;               // residual stream [rows][D], updated in place
+    const int32_t* tokens;  // or null: x = embed[tokens[row]]
+    const void* embed;      // [vocab][D]
+    const void* y;          // or null: sublayer output [rows][ldy]
+    const void* y_bias;     // or null: [D], added to y
+    const void* post_w;     // or null: y is RMS-normed with this weight before it joins the residual
+    const void* pre_w;      // or null: h = RMSNorm(x) * pre_w
+    void* h;                // [launch rows][D]
+    const int32_t* rows;    // or null: row of x / y / tokens a workgroup handles (a subset of the rows); h is packed
+    int D, ldy, vocab;
+    float eps;
+};
+
+template <int DT, int NT, int VEC>
+__global__ __launch_bounds__(NT) void resid_norm_kernel(const ResidNormArgs a) {
+    using N = Num<DT>;
+    using S = typename N::S;
+    extern __shared__ __align__(16) unsigned char smem[];
+    float* buf = reinterpret_cast<float*>(smem);  // [D]
+    __shared__ float red[NT / 64];
+    const int tid = threadIdx.x, D = a.D;
+    const size_t row = a.rows ? (size_t)a.rows[blockIdx.x] : (size_t)blockIdx.x;
+    float* x = a.x + row * D;
+    const S* y = a.y ? reinterpret_cast<const S*>(a.y) + row * a.ldy : nullptr;
+    const S* yb = reinterpret_cast<const S*>(a.y_bias);
+    const S* pw = reinterpret_cast<const S*>(a.post_w);
+    const S* nw = reinterpret_cast<const S*>(a.pre_w);
+    auto ldv = [](const S* p, float (&o)[VEC]) {
+        if constexpr (VEC == 4 && DT != TEAL_F32) {
+            const u32x2 w = *reinterpret_cast<const u32x2*>(p);
+#pragma unroll
+            for (int j = 0; j < 2; ++j) { o[2 * j] = bits_to_float(w[j] & 0xFFFFu, DT == TEAL_BF16); o[2 * j + 1] = bits_to_float(w[j] >> 16, DT == TEAL_BF16); }
+        } else if constexpr (VEC == 4) {
+            const f32x4 w = *reinterpret_cast<const f32x4*>(p);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) o[j] = w[j];
+        } else {
+            o[0] = N::ld(p);
+        }
+    };
+    auto ldx = [](const float* p, float (&o)[VEC]) {
+        if constexpr (VEC == 4) {
+            const f32x4 w = *reinterpret_cast<const f32x4*>(p);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) o[j] = w[j];
+        } else {
+            o[0] = *p;
+        }
+    };
+    auto stx = [](float* p, const float (&o)[VEC]) {
+        if constexpr (VEC == 4) *reinterpret_cast<f32x4*>(p) = f32x4{o[0], o[1], o[2], o[3]};
+        else *p = o[0];
+    };
+    float rstd_y = 1.0f;
+    if (y) {
+        float ss = 0.0f;
+        for (int i = tid * VEC; i < D; i += NT * VEC) {
+            float v[VEC];
+            ldv(y + i, v);
+            if (yb) {
+                float b[VEC];
+                ldv(yb + i, b);
+#pragma unroll
+                for (int j = 0; j < VEC; ++j) v[j] += b[j];
+            }
+            stx(buf + i, v);  // (each thread reads back only what it wrote)
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) ss = fmaf(v[j], v[j], ss);
+        }
+        if (pw) rstd_y = 1.0f / sqrtf(block_sum<NT>(ss, red, tid) / (float)D + a.eps);
+    }
+    const S* erow = nullptr;
+    if (a.tokens) {
+        const int t = min(max(a.tokens[row], 0), a.vocab - 1);
+        erow = reinterpret_cast<const S*>(a.embed) + (size_t)t * D;
+    }
+    float ss = 0.0f;
+    for (int i = tid * VEC; i < D; i += NT * VEC) {
+        float v[VEC];
+        if (erow) ldv(erow + i, v);
+        else ldx(x + i, v);
+        if (y) {
+            float u[VEC];
+            ldx(buf + i, u);
+            if (pw) {
+                float w[VEC];
+                ldv(pw + i, w);
+#pragma unroll
+                for (int j = 0; j < VEC; ++j) u[j] = u[j] * rstd_y * w[j];
+            }
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) v[j] += u[j];
+        }
+        if (erow || y) stx(x + i, v);
+        stx(buf + i, v);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) ss = fmaf(v[j], v[j], ss);
+    }
+    if (!nw) return;
+    const float rstd = 1.0f / sqrtf(block_sum<NT>(ss, red, tid) / (float)D + a.eps);
+    S* h = reinterpret_cast<S*>(a.h) + (size_t)blockIdx.x * D;
+    for (int i = tid * VEC; i < D; i += NT * VEC) {
+        float v[VEC], w[VEC];
+        ldx(buf + i, v);
+        ldv(nw + i, w);
+        if constexpr (VEC == 4 && DT != TEAL_F32) {
+            uint32_t o[4];
+#pragma unroll
+            for (int j = 0; j < 4; ++j) o[j] = N::cvt(v[j] * rstd * w[j]);
+            *reinterpret_cast<u32x2*>(h + i) = u32x2{o[0] | (o[1] << 16), o[2] | (o[3] << 16)};
+        } else {
+#pragma unroll
+            for (int j = 0; j < VEC; ++j) h[i + j] = N::cvt(v[j] * rstd * w[j]);
+        }
+    }
+}
+
+// h[t][n] = act(gu[t][n] + bg[n]) * (gu[t][up0 + n] + bu[n]); act 0 = silu, 1 = gelu (tanh form)
+template <int DT>
+__global__ __launch_bounds__(256) void gated_act_kernel(const typename Num<DT>::S* __restrict__ gu, const int ldg, const int up0,
+                                                        const typename Num<DT>::S* __restrict__ bg, const typename Num<DT>::S* __restrict__ bu,
+                                                        typename Num<DT>::S* __restrict__ h, const int ldh, const int F, const int act, const bool vec) {
+    using N = Num<DT>;
+    const size_t t = blockIdx.x;
+    const int n0 = (blockIdx.y * 256 + threadIdx.x) * 8;
+    if (n0 >= F) return;
+    const typename N::S* g = gu + t * ldg;
+    typename N::S* o = h + t * ldh;
+    const int m = min(8, F - n0);
+    float gv[8], uv[8], bgv[8], buv[8];
+    if (m == 8) {
+        ld8<DT>(g + n0, gv, vec);
+        ld8<DT>(g + up0 + n0, uv, vec);
+        if (bg) ld8<DT>(bg + n0, bgv, vec);
+        if (bu) ld8<DT>(bu + n0, buv, vec);
+    } else {
+        for (int j = 0; j < m; ++j) {
+            gv[j] = N::ld(g + n0 + j);
+            uv[j] = N::ld(g + up0 + n0 + j);
+            if (bg) bgv[j] = N::ld(bg + n0 + j);
+            if (bu) buv[j] = N::ld(bu + n0 + j);
+        }
+    }
+    typename N::S r[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+        const float z = bg ? gv[j] + bgv[j] : gv[j];
+        const float u = bu ? uv[j] + buv[j] : uv[j];
+        r[j] = N::cvt((act == 1 ? gelu_tanh_f(z) : z * sigmoid_f(z)) * u);
+    }
+    if (vec && m == 8 && DT != TEAL_F32) {
+        u32x4 w;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) w[j] = (uint32_t)r[2 * j] | ((uint32_t)r[2 * j + 1] << 16);
+        *reinterpret_cast<u32x4*>(o + n0) = w;
+    } else {
+        for (int j = 0; j < m; ++j) o[n0 + j] = r[j];
+    }
+}
+
+template <int DT>
+__global__ __launch_bounds__(256) void softcap_kernel(const typename Num<DT>::S* __restrict__ in, const int ldi, float* __restrict__ out, const int V,
+                                                      const float cap) {
+    const int n = blockIdx.y * 256 + threadIdx.x;
+    if (n >= V) return;
+    const float v = Num<DT>::ld(in + (size_t)blockIdx.x * ldi + n);
+    out[(size_t)blockIdx.x * V + n] = cap > 0.0f ? cap * tanhf(v / cap) : v;
+}
+
+}  // namespace teal
+
+using namespace teal;
+
+extern "C" {
+
+int teal_layer_resid_norm(float* x, int n_rows, int dim, const int32_t* tokens, const void* embed, int vocab, const void* y, int ldy,
+                          const void* y_bias, const void* post_w, const void* pre_w, float eps, void* h, const int32_t* rows, int dtype, void* stream) {
+    if (!x || n_rows <= 0 || dim <= 0 || (tokens && (!embed || vocab <= 0)) || (post_w && !y) || (y_bias && !y) || (pre_w && !h)) return TEAL_ERR_ARG;
+    if (dim > 15360 || (y && ldy < dim)) return TEAL_ERR_SHAPE;
+    if (!device_ctx()) return TEAL_ERR_NO_DEVICE;
+    const ResidNormArgs a = {x, tokens, embed, y, y_bias, post_w, pre_w, h, rows, dim, ldy, vocab, eps};
+    hipStream_t st = reinterpret_cast<hipStream_t>(stream);
+    const void* ps[] = {x, embed, y, y_bias, post_w, pre_w, h};
+    bool vec = (dim & 3) == 0 && (!y || (ldy & 3) == 0);
+    for (const void* p : ps) vec = vec && aligned16(p);
+    return with_dtype(dtype, [&](auto dt) {
+        constexpr int DT = decltype(dt)::value;
+        const size_t lds = (size_t)dim * sizeof(float);
+#define TEAL_RN(NT, V) hipLaunchKernelGGL((resid_norm_kernel<DT, NT, V>), dim3(n_rows), dim3(NT), lds, st, a)
+        if (!vec) TEAL_RN(256, 1);
+        else if (dim <= 2048) TEAL_RN(256, 4);
+        else TEAL_RN(1024, 4);
+#undef TEAL_RN
+        return launched();
+    });
+}
+
+int teal_gated_act(const void* gu, int ldg, int up0, const void* bias_gate, const void* bias_up, void* h, int ldh, int n_rows, int n_cols, int act,
+                   int dtype, void* stream) {
+    if (!gu || !h || n_rows <= 0 || n_cols <= 0 || (act != TEAL_ACT_SILU && act != TEAL_ACT_GELU_TANH)) return TEAL_ERR_ARG;
+    if (ldg < up0 + n_cols || up0 < n_cols || ldh < n_cols) return TEAL_ERR_SHAPE;
+    hipStream_t st = reinterpret_cast<hipStream_t>(stream);
+    const bool vec = !(ldg & 7) && !(up0 & 7) && !(ldh & 7) && aligned16(gu) && aligned16(h) && aligned16(bias_gate) && aligned16(bias_up);
+    return with_dtype(dtype, [&](auto dt) {
+        constexpr int DT = decltype(dt)::value;
+        using S = typename Num<DT>::S;
+        hipLaunchKernelGGL((gated_act_kernel<DT>), dim3(n_rows, (n_cols + 2047) / 2048), dim3(256), 0, st, reinterpret_cast<const S*>(gu), ldg, up0,
+                           reinterpret_cast<const S*>(bias_gate), reinterpret_cast<const S*>(bias_up), reinterpret_cast<S*>(h), ldh, n_cols, act, vec);
+        return launched();
+    });
+}
+
+int teal_logit_softcap(const void* logits, int ld, float* out, int n_rows, int vocab, float cap, int dtype, void* stream) {
+    if (!logits || !out || n_rows <= 0 || vocab <= 0) return TEAL_ERR_ARG;
+    if (ld < vocab) return TEAL_ERR_SHAPE;
+    hipStream_t st = reinterpret_cast<hipStream_t>(stream);
+    return with_dtype(dtype, [&](auto dt) {
+        constexpr int DT = decltype(dt)::value;
+        hipLaunchKernelGGL((softcap_kernel<DT>), dim3(n_rows, (vocab + 255) / 256), dim3(256), 0, st,
+                           reinterpret_cast<const typename Num<DT>::S*>(logits), ld, out, vocab, cap);
+        return launched();
+    });
+}
+
+}  // extern "C"

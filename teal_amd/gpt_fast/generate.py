@@ -67,6 +67,17 @@ def sample(logits: torch.Tensor, temperature: float = 1.0, top_k: Optional[int] 
     return multinomial_sample_one_no_sync(probs), probs
 
 
+def sample_rows(logits: torch.Tensor, temperature: float = 1.0, top_k: Optional[int] = None) -> torch.Tensor:
+    """one token per row of logits [B, vocab]; temperature <= 0: the largest logit"""
+    if temperature <= 0:
+        return logits.argmax(dim=-1).to(torch.int)
+    logits = logits.float() / max(temperature, 1e-5)
+    if top_k is not None:
+        v, _ = torch.topk(logits, min(top_k, logits.size(-1)))
+        logits = torch.where(logits < v[:, -1:], -float("Inf"), logits)
+    return multinomial_sample_one_no_sync(torch.nn.functional.softmax(logits, dim=-1)).view(-1)
+
+
 # ------------------------------------------------------------------------------------------------
 # model construction
 # ------------------------------------------------------------------------------------------------

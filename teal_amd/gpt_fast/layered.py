@@ -1,0 +1,581 @@
+"""Layered decoder designs: models described layer by layer in a config.json (mixer type and sizes, feed-forward, shared caches),
+next to the uniform Llama stack of model.py.
+
+A design (DESIGNS) fixes what its checkpoints do not spell out — norm placement, activation, biases, whether the attention has a
+sink and an output gate —; every size and every other constant comes from the configuration, per layer.  Mixers and feed-forwards
+are looked up by name (MIXERS, MLPS), so a further design adds an entry and, where it needs one, a mixer.
+
+Two passes share one set of weights and one paged cache (paged.PagedCache):
+  prompt pass   ragged batch of portions (each any number of tokens, from any position), packed without padding; matrix products by
+                the vendor library over MFMA, hand-written kernels for everything between them (csrc/teal_layered.hip, teal_latent.hip)
+  step          one token per sequence; latent attention in its absorbed form over the cached rows
+The residual stream is fp32 throughout.  dtype fp16 / bf16 (matrix products and activations) or float32 (everything).
+"""
+from __future__ import annotations
+
+import json
+from dataclasses import dataclass, field
+from pathlib import Path
+from typing import Any, Callable, Dict, List, Optional, Sequence
+
+import numpy as np
+import torch
+import torch.nn as nn
+import torch.nn.functional as F
+
+from ..kernels import layered as K
+from ..monkeypatch import to_column_major
+from .paged import PAGE_SHIFT, PagedCache
+
+
+def pad_to(n: int, k: int) -> int:
+    return -(-n // k) * k
+
+
+# ------------------------------------------------------------------------------------------------
+# configuration
+# ------------------------------------------------------------------------------------------------
+@dataclass(frozen=True)
+class Design:
+    """what all checkpoints of a design have in common"""
+    post_norms: bool = True          # a second norm on every sublayer's output, before the residual add
+    mlp_act: str = "gelu_tanh"
+    mlp_bias: bool = True
+    attn_sink: bool = True
+    attn_gate: bool = True
+    mixers: Sequence[str] = ("latent_attention",)
+
+
+DESIGNS: Dict[str, Design] = {"Bolizen": Design()}
+
+
+@dataclass
+class LatentAttentionArgs:
+    heads: int
+    dim: int                         # unrotated query / key dimensions per head
+    rot_dim: int                     # rotated ones (one key part shared by the heads)
+    vdim: int
+    kv_rank: int
+    scale: float
+    rope_base: float
+    window: Optional[int] = None     # a query sees itself and the window - 1 positions before it; None: all before it
+    kv_from: Optional[int] = None    # reads the latents another layer caches
+    sink: bool = True
+    gate: bool = True
+
+    @classmethod
+    def parse(cls, d: Dict[str, Any], design: Design) -> "LatentAttentionArgs":
+        rot = d["rot"]
+        if int(rot["dims"]) != int(d["rot_dim"]) or int(d["rot_dim"]) % 2:
+            raise ValueError(f"latent_attention rotates all of its {d['rot_dim']} shared dimensions, in pairs (rot.dims = {rot['dims']})")
+        window = (d.get("mask") or {}).get("size")
+        kv_from = d.get("kv_from")
+        return cls(heads=int(d["heads"]), dim=int(d["dim"]), rot_dim=int(d["rot_dim"]), vdim=int(d["vdim"]), kv_rank=int(d["kv_rank"]),
+                   scale=float(d["scale"]), rope_base=float(rot["base"]), window=None if window is None else int(window),
+                   kv_from=None if kv_from is None else int(kv_from), sink=design.attn_sink, gate=design.attn_gate)
+
+
+@dataclass
+class GatedMLPArgs:
+    ff: int
+    act: str = "gelu_tanh"
+    bias: bool = True
+
+    @classmethod
+    def parse(cls, d: Dict[str, Any], design: Design) -> "GatedMLPArgs":
+        return cls(ff=int(d["ff"]), act=design.mlp_act, bias=design.mlp_bias)
+
+
+@dataclass
+class LayerArgs:
+    kind: str
+    mixer: Any
+    mlp_kind: Optional[str] = None
+    mlp: Any = None
+
+
+@dataclass
+class LayeredArgs:
+    architecture: str
+    vocab_size: int
+    dim: int
+    norm_eps: float
+    layers: List[LayerArgs]
+    logit_softcap: Optional[float] = None
+    block_size: int = 1 << 20        # positions are rotated by angle, not by table: the cache is the only limit
+    design: Design = field(default_factory=Design)
+
+    @property
+    def n_layer(self) -> int:
+        return len(self.layers)
+
+    @classmethod
+    def from_dict(cls, d: Dict[str, Any]) -> "LayeredArgs":
+        arch = d.get("architecture")
+        if arch not in DESIGNS:
+            raise KeyError(f"no layered design named {arch!r} (known: {sorted(DESIGNS)})")
+        design, layers = DESIGNS[arch], []
+        for i, ld in enumerate(d["layers"]):
+            kind, mlp = ld["type"], ld.get("mlp")
+            if kind not in MIXERS or kind not in design.mixers:
+                raise ValueError(f"layer {i}: unknown mixer {kind!r} for {arch}")
+            if mlp is not None and mlp["kind"] not in MLPS:
+                raise ValueError(f"layer {i}: unknown feed-forward {mlp['kind']!r}")
+            layers.append(LayerArgs(kind, MIXERS[kind].args.parse(ld["mixer"], design), mlp["kind"] if mlp else None,
+                                    MLPS[mlp["kind"]].args.parse(mlp, design) if mlp else None))
+        for i, ly in enumerate(layers):
+            j = ly.mixer.kv_from
+            if j is None:
+                continue
+            if not 0 <= j < i or layers[j].kind != ly.kind or layers[j].mixer.kv_from is not None:
+                raise ValueError(f"layer {i}: kv_from {j} must name an earlier layer with latents of its own")
+            a, b = ly.mixer, layers[j].mixer
+            if (a.kv_rank, a.rot_dim, a.rope_base) != (b.kv_rank, b.rot_dim, b.rope_base):
+                raise ValueError(f"layer {i}: latent size and rotation differ from layer {j}'s")
+        cap = d.get("logit_softcap")
+        return cls(arch, int(d["vocab"]), int(d["width"]), float(d["norm"]["eps"]), layers, None if cap is None else float(cap), design=design)
+
+    @classmethod
+    def from_name(cls, name: str, n_layer: Optional[int] = None) -> "LayeredArgs":
+        return cls.from_dict(named_config(name, n_layer))
+
+
+# name -> sizes of a synthetic model: like the named Llama shapes of model.transformer_configs, for runs without a checkpoint.
+# share: layers that read the latents of the one before them follow each owner in runs of this many (0: every layer owns its own)
+layered_configs: Dict[str, Dict[str, Any]] = {
+    "Bolizen-tiny-test": dict(architecture="Bolizen", n_layer=4, width=128, vocab=256, ff=384, heads=2, dim=24, rot_dim=8, vdim=40, kv_rank=64, window=48, share=1),
+    "Bolizen-1B": dict(architecture="Bolizen", n_layer=16, width=2048, vocab=32000, ff=5632, heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, window=4096, share=1),
+    "Bolizen-7B": dict(architecture="Bolizen", n_layer=32, width=4096, vocab=32000, ff=11008, heads=32, dim=128, rot_dim=64, vdim=128, kv_rank=512, window=4096, share=1),
+}
+
+
+def is_layered_name(name: str) -> bool:
+    return name in layered_configs
+
+
+def named_config(name: str, n_layer: Optional[int] = None) -> Dict[str, Any]:
+    """the config.json of a named synthetic model"""
+    c = layered_configs[name]
+    layers = []
+    for i in range(n_layer or c["n_layer"]):
+        mixer = dict(heads=c["heads"], dim=c["dim"], rot_dim=c["rot_dim"], vdim=c["vdim"], kv_rank=c["kv_rank"], mask={"size": c["window"]},
+                     rot={"base": 10000.0, "dims": c["rot_dim"]}, scale=(c["dim"] + c["rot_dim"]) ** -0.5)
+        owner = i - i % (c["share"] + 1)
+        if owner != i:
+            mixer["kv_from"] = owner
+        layers.append({"type": "latent_attention", "mixer": mixer, "mlp": {"kind": "dense", "ff": c["ff"]}})
+    return {"architecture": c["architecture"], "layers": layers, "logit_softcap": 30.0, "norm": {"eps": 1e-6}, "vocab": c["vocab"], "width": c["width"]}
+
+
+# ------------------------------------------------------------------------------------------------
+# the two passes' shared metadata
+# ------------------------------------------------------------------------------------------------
+class PromptBatch:
+    """A ragged batch of prompt portions: per entry a slot, its first position and its tokens, packed back to back."""
+
+    def __init__(self, cache: PagedCache, entries, device):
+        """entries: [(slot, start, tokens)]; the cache already has room for them and `sync` has run"""
+        self.cache = cache
+        toks, pos, row, krow, self.spans = [], [], [], [], []
+        q0 = k0 = 0
+        for slot, start, tokens in entries:
+            n = len(tokens)
+            p = np.arange(start, start + n, dtype=np.int64)
+            klo = 0 if cache.window is None else max(0, start - cache.window + 1)
+            keys = np.arange(klo, start + n, dtype=np.int64)
+            span = np.full(pad_to(len(keys), K.TILE), -1, dtype=np.int64)
+            span[: len(keys)] = cache.rows(slot, keys)
+            toks.append(np.asarray(tokens, dtype=np.int64)), pos.append(p), row.append(cache.rows(slot, p)), krow.append(span)
+            self.spans.append((q0, n, start, k0, klo))
+            q0 += n
+            k0 += len(span)
+        self.n_tokens, self.n_keys = q0, k0
+        flat = np.concatenate([np.concatenate(x) for x in (toks, pos, row)] + krow + [np.asarray(self.spans).ravel()]).astype(np.int32)
+        dev = torch.from_numpy(flat).to(device)
+        self.tokens, self.pos, self.row = dev[:q0], dev[q0:2 * q0], dev[2 * q0:3 * q0]
+        self.key_row = dev[3 * q0:3 * q0 + k0]
+        self.seqs = dev[3 * q0 + k0:].view(-1, 5)
+        self.device = device
+        self._tiles: Dict[int, torch.Tensor] = {}
+        self.packed: Dict[int, Any] = {}  # owner layer -> (latents, rotated key parts) of every key row of the batch
+
+    @property
+    def longest(self) -> int:
+        return max(n for _, n, _, _, _ in self.spans)
+
+    def tiles(self, size: int) -> torch.Tensor:
+        if size not in self._tiles:
+            # (last tiles first: with a causal mask they are the long ones)
+            t = [(i, q) for i, (_, n, _, _, _) in enumerate(self.spans) for q in range(0, n, size)][::-1]
+            self._tiles[size] = torch.tensor(t, dtype=torch.int32).to(self.device)
+        return self._tiles[size]
+
+
+@dataclass
+class StepBatch:
+    """one token per sequence; all tensors int32 on the device"""
+    cache: PagedCache
+    tokens: torch.Tensor
+    pos: torch.Tensor
+    slot: torch.Tensor
+    max_pos: int                     # no position of the batch is larger (chooses how far the attention is split; not a limit)
+
+
+# ------------------------------------------------------------------------------------------------
+# modules
+# ------------------------------------------------------------------------------------------------
+def _weight(*shape) -> nn.Parameter:
+    return nn.Parameter(torch.zeros(*shape), requires_grad=False)
+
+
+class LatentAttention(nn.Module):
+    """Latent attention with an optional window, sink, output gate and a cache shared between layers (csrc/teal_latent.hip).
+
+    `proj` holds the projections that read the mixer's input as one image, [q | gate | latent + shared key part], every segment
+    padded with zero rows to whole 64-column tiles; `wo` reads the padded concatenation of the heads."""
+
+    args = LatentAttentionArgs
+
+    def __init__(self, cfg: LayeredArgs, index: int, a: LatentAttentionArgs):
+        super().__init__()
+        self.a, self.index, self.eps = a, index, cfg.norm_eps
+        self.owner = index if a.kv_from is None else a.kv_from
+        self.nq, self.nv = a.heads * (a.dim + a.rot_dim), a.heads * a.vdim
+        self.g0 = pad_to(self.nq, 64)
+        self.kv0 = self.g0 + (pad_to(self.nv, 64) if a.gate else 0)
+        self.nkv = a.kv_rank + a.rot_dim
+        n = self.kv0 + (pad_to(self.nkv, 64) if a.kv_from is None else 0)
+        self.proj = nn.Linear(cfg.dim, n, bias=False)
+        self.wo = nn.Linear(pad_to(self.nv, 64), cfg.dim, bias=False)
+        self.uk, self.uv = _weight(a.heads * a.dim, a.kv_rank), _weight(self.nv, a.kv_rank)
+        self.kv_norm = _weight(a.kv_rank) if a.kv_from is None else None
+        self.sink = _weight(a.heads) if a.sink else None
+        self.register_buffer("inv_freq", torch.zeros(max(1, a.rot_dim // 2)), persistent=False)
+
+    @property
+    def window(self) -> int:
+        return K.NO_WINDOW if self.a.window is None else self.a.window
+
+    def init_buffers(self):
+        i = torch.arange(0, self.a.rot_dim, 2, dtype=torch.float64)
+        self.inv_freq = (float(self.a.rope_base) ** (-i / max(1, self.a.rot_dim))).to(device=self.uk.device, dtype=torch.float32)
+
+    def cache_width(self) -> Optional[int]:
+        return pad_to(self.nkv, 32) if self.a.kv_from is None else None
+
+    def tensors(self, get: Callable[[str], torch.Tensor]) -> None:
+        """fill from a checkpoint's tensors, by name inside the mixer"""
+        a, w = self.a, self.proj.weight
+        w[: self.nq] = get("q")
+        if a.gate:
+            w[self.g0:self.g0 + self.nv] = get("g")
+        if a.kv_from is None:
+            w[self.kv0:self.kv0 + self.nkv] = get("dkv")
+            self.kv_norm.copy_(get("dkv.norm"))
+        self.uk.copy_(get("uk"))
+        self.uv.copy_(get("uv"))
+        if a.sink:
+            self.sink.copy_(get("sink"))
+        self.wo.weight[:, : self.nv] = get("o")
+
+    def shapes(self) -> Dict[str, tuple]:
+        a, d = self.a, self.proj.in_features
+        out = {"q": (self.nq, d), "uk": (a.heads * a.dim, a.kv_rank), "uv": (self.nv, a.kv_rank), "o": (d, self.nv)}
+        if a.kv_from is None:
+            out.update({"dkv": (self.nkv, d), "dkv.norm": (a.kv_rank,)})
+        if a.sink:
+            out["sink"] = (a.heads,)
+        if a.gate:
+            out["g"] = (self.nv, d)
+        return out
+
+    def _gate(self, proj):
+        return proj[:, self.g0:self.g0 + self.nv] if self.a.gate else None
+
+    def _y(self, n, ref):
+        y = torch.empty(n, self.wo.in_features, device=ref.device, dtype=ref.dtype)
+        if self.wo.in_features > self.nv:
+            y[:, self.nv:].zero_()
+        return y
+
+    def prompt(self, h: torch.Tensor, b: PromptBatch) -> torch.Tensor:
+        a, pool = self.a, b.cache.pools[self.owner]
+        own = a.kv_from is None
+        proj = F.linear(h, self.proj.weight)
+        K.latent_prompt_rows(proj, self.kv0 if own else -1, b.pos, b.row if own else None, self.inv_freq, self.kv_norm, self.eps, a.heads, a.dim, a.rot_dim,
+                             a.kv_rank, pool if own else None)
+        if own:
+            b.packed[self.index] = K.latent_gather(pool, b.key_row, a.kv_rank, a.rot_dim)
+        c, kr = b.packed[self.owner]
+        k, vt = torch.matmul(c, self.uk.T), torch.matmul(self.uv, c.T)
+        tile = K.latent_prompt_tile(a.dim, a.rot_dim, a.vdim, b.longest, h.dtype)
+        y = K.latent_prompt_attention(proj, k, kr, vt, self.sink, self._gate(proj), self._y(b.n_tokens, h), b.seqs, b.tiles(tile), tile, a.heads, a.dim,
+                                      a.rot_dim, a.vdim, self.window, a.scale)
+        return F.linear(y, self.wo.weight)
+
+    def splits(self, batch: int, max_pos: int, dtype: torch.dtype) -> int:
+        """workgroups the cached rows of one sequence are split over: about one per CU, two 32-key tiles each at least"""
+        groups = self.a.heads if dtype == torch.float32 else -(-self.a.heads // 16)
+        tiles = min(self.window, max_pos + 1) // 32 + 1
+        return max(1, min(-(-tiles // 2), -(-256 // (batch * groups)), 32))
+
+    def attend(self, proj: torch.Tensor, b: StepBatch, y: Optional[torch.Tensor] = None, buffers=None) -> torch.Tensor:
+        """the step's attention on a computed projection: append the cache row, attend, merge -> the wo projection's input"""
+        a, n, pool = self.a, proj.shape[0], b.cache.pools[self.owner]
+        own = a.kv_from is None
+        splits = self.splits(n, b.max_pos, proj.dtype)
+        if buffers is None:
+            qcat = K.latent_qcat(n, a.heads, pool.shape[-1], proj.dtype, proj.device)
+            part = torch.empty(n * a.heads * splits * (a.kv_rank + 2), device=proj.device, dtype=torch.float32)
+        else:
+            qcat, part = buffers
+        K.latent_step_query(proj, self.kv0 if own else -1, b.pos, b.slot, b.cache.table, PAGE_SHIFT, self.inv_freq, self.kv_norm, self.eps, self.uk, a.heads,
+                            a.dim, a.rot_dim, a.kv_rank, pool, qcat)
+        K.latent_step_attention(qcat, pool, b.pos, b.slot, b.cache.table, PAGE_SHIFT, a.kv_rank, a.rot_dim, self.window, a.scale, splits, part)
+        y = self._y(n, proj) if y is None else y
+        return K.latent_step_merge(part, splits, self.uv, self.sink, self._gate(proj), y, n, a.heads, a.kv_rank, a.vdim)
+
+    def step(self, h: torch.Tensor, b: StepBatch) -> torch.Tensor:
+        return F.linear(self.attend(F.linear(h, self.proj.weight), b), self.wo.weight)
+
+    def linears(self):
+        return [self.proj, self.wo]
+
+
+class GatedMLP(nn.Module):
+    """down(act(gate h + b) * (up h + b)) (+ b, added by the residual kernel); gate | up as one image, both padded to whole tiles"""
+
+    args = GatedMLPArgs
+
+    def __init__(self, cfg: LayeredArgs, a: GatedMLPArgs):
+        super().__init__()
+        self.a, self.fp = a, pad_to(a.ff, 64)
+        self.gate_up = nn.Linear(cfg.dim, 2 * self.fp, bias=False)
+        self.down = nn.Linear(self.fp, cfg.dim, bias=False)
+        self.gate_up_bias = _weight(2 * self.fp) if a.bias else None
+        self.down_bias = _weight(cfg.dim) if a.bias else None
+
+    def tensors(self, get: Callable[[str], torch.Tensor]) -> None:
+        ff, fp = self.a.ff, self.fp
+        self.gate_up.weight[:ff] = get("gate")
+        self.gate_up.weight[fp:fp + ff] = get("up")
+        self.down.weight[:, :ff] = get("down")
+        if self.a.bias:
+            self.gate_up_bias[:ff] = get("gate.b")
+            self.gate_up_bias[fp:fp + ff] = get("up.b")
+            self.down_bias.copy_(get("down.b"))
+
+    def shapes(self) -> Dict[str, tuple]:
+        ff, d = self.a.ff, self.down.out_features
+        out = {"gate": (ff, d), "up": (ff, d), "down": (d, ff)}
+        if self.a.bias:
+            out.update({"gate.b": (ff,), "up.b": (ff,), "down.b": (d,)})
+        return out
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        return F.linear(K.gated_act(F.linear(h, self.gate_up.weight), self.fp, self.fp, self.a.act, self.gate_up_bias), self.down.weight)
+
+    def linears(self):
+        return [self.gate_up, self.down]
+
+
+MIXERS = {"latent_attention": LatentAttention}
+MLPS = {"dense": GatedMLP}
+
+
+class LayeredBlock(nn.Module):
+    def __init__(self, cfg: LayeredArgs, index: int):
+        super().__init__()
+        ly = cfg.layers[index]
+        self.mix = MIXERS[ly.kind](cfg, index, ly.mixer)
+        self.mlp = MLPS[ly.mlp_kind](cfg, ly.mlp) if ly.mlp_kind else None
+        post = cfg.design.post_norms
+        self.norm1, self.norm1b = _weight(cfg.dim), _weight(cfg.dim) if post else None
+        self.norm2 = _weight(cfg.dim) if self.mlp is not None else None
+        self.norm2b = _weight(cfg.dim) if self.mlp is not None and post else None
+
+
+class LayeredTransformer(nn.Module):
+    def __init__(self, config: LayeredArgs):
+        super().__init__()
+        self.config = config
+        self.tok_embeddings = nn.Embedding(config.vocab_size, config.dim)
+        self.layers = nn.ModuleList(LayeredBlock(config, i) for i in range(config.n_layer))
+        self.norm = _weight(config.dim)
+        self.output: Optional[nn.Linear] = None  # the embedding table as the head's image (finalize)
+        self.max_batch_size = self.max_seq_length = -1
+        self.cache: Optional[PagedCache] = None
+
+    # ---- weights ---------------------------------------------------------------------------------------------------
+    def tensor_shapes(self) -> Dict[str, tuple]:
+        """every checkpoint tensor of this configuration, by name"""
+        d = self.config.dim
+        out = {"embed": (self.config.vocab_size, d), "final.norm": (d,)}
+        for i, b in enumerate(self.layers):
+            out.update({f"l{i}.{n}": (d,) for n in ("norm1", "norm1b", "norm2", "norm2b") if getattr(b, n) is not None})
+            out.update({f"l{i}.mix.{n}": s for n, s in b.mix.shapes().items()})
+            if b.mlp is not None:
+                out.update({f"l{i}.mlp.{n}": s for n, s in b.mlp.shapes().items()})
+        return out
+
+    @torch.no_grad()
+    def load_tensors(self, get: Callable[[str], torch.Tensor]) -> "LayeredTransformer":
+        shapes = self.tensor_shapes()
+
+        def checked(name):
+            t = get(name)
+            if tuple(t.shape) != shapes[name]:
+                raise ValueError(f"{name}: shape {tuple(t.shape)}, the configuration needs {shapes[name]}")
+            return t
+
+        self.tok_embeddings.weight.copy_(checked("embed"))
+        self.norm.copy_(checked("final.norm"))
+        for i, b in enumerate(self.layers):
+            for n in ("norm1", "norm1b", "norm2", "norm2b"):
+                if getattr(b, n) is not None:
+                    getattr(b, n).copy_(checked(f"l{i}.{n}"))
+            b.mix.tensors(lambda n, i=i: checked(f"l{i}.mix.{n}"))
+            if b.mlp is not None:
+                b.mlp.tensors(lambda n, i=i: checked(f"l{i}.mlp.{n}"))
+        return self.finalize()
+
+    @torch.no_grad()
+    def finalize(self) -> "LayeredTransformer":
+        """after the weights are in place: derived buffers, and the layout the decode kernels stream (16-bit: the transposed image of
+        every projection, monkeypatch.to_column_major; the head's image is padded to whole 64-column tiles)"""
+        w = self.tok_embeddings.weight
+        for p in self.parameters():
+            p.requires_grad_(False)
+        head = nn.Linear(1, 1, bias=False)
+        if w.dtype == torch.float32:
+            head.weight = nn.Parameter(w.data, requires_grad=False)
+        else:
+            padded = torch.zeros(pad_to(w.shape[0], 64), w.shape[1], dtype=w.dtype, device=w.device)
+            padded[: w.shape[0]] = w
+            head.weight = nn.Parameter(padded, requires_grad=False)
+            to_column_major(head)
+        self.output = head
+        for b in self.layers:
+            b.mix.init_buffers()
+            if w.dtype != torch.float32:
+                for lin in b.mix.linears() + (b.mlp.linears() if b.mlp is not None else []):
+                    to_column_major(lin)
+        return self.eval()
+
+    # ---- cache -----------------------------------------------------------------------------------------------------
+    def new_cache(self, max_tokens: int, max_requests: int = 8) -> PagedCache:
+        w = self.tok_embeddings.weight
+        windows = [ly.mixer.window for ly in self.config.layers]
+        widths = {i: b.mix.cache_width() for i, b in enumerate(self.layers) if b.mix.cache_width() is not None}
+        return PagedCache(widths, w.dtype, w.device, max_tokens, max_requests, None if None in windows else max(windows))
+
+    def setup_caches(self, max_batch_size: int, max_seq_length: int):
+        """model.Transformer's contract: room for max_batch_size sequences of max_seq_length positions, slots 0 .. max_batch_size - 1"""
+        if self.max_seq_length >= max_seq_length and self.max_batch_size >= max_batch_size:
+            return
+        self.max_seq_length, self.max_batch_size = pad_to(max_seq_length, 8), max_batch_size
+        self.cache = self.new_cache(max_batch_size * self.max_seq_length, max_batch_size)
+        for _ in range(max_batch_size):
+            self.cache.extend(self.cache.open(), self.max_seq_length)
+        self.cache.sync()
+        self._slots = torch.arange(max_batch_size, dtype=torch.int32, device=self.tok_embeddings.weight.device)
+
+    # ---- passes ----------------------------------------------------------------------------------------------------
+    def _run(self, b, mixer, want: Optional[torch.Tensor], n_want: int, hook=None) -> Optional[torch.Tensor]:
+        """embedding -> layers -> logits of the rows `want` (None: every row) of the batch b; mixer(layer, h) = its mixer's pass"""
+        cfg, eps, w = self.config, self.config.norm_eps, self.tok_embeddings.weight
+        x = torch.empty(b.tokens.numel(), cfg.dim, device=w.device, dtype=torch.float32)
+        h = K.resid_norm(x, tokens=b.tokens, embed=w, pre_w=self.layers[0].norm1, eps=eps)
+        for i, layer in enumerate(self.layers):
+            last = i + 1 == len(self.layers)
+            after = dict(pre_w=(self.norm if n_want else None) if last else self.layers[i + 1].norm1)
+            if last and hook is None and n_want:
+                after["rows"] = want  # nothing reads the other rows any more
+            first = after if layer.mlp is None else dict(pre_w=layer.norm2)
+            h = K.resid_norm(x, y=mixer(layer.mix, h), post_w=layer.norm1b, eps=eps, **first)
+            if layer.mlp is not None:
+                h = K.resid_norm(x, y=layer.mlp(h), y_bias=layer.mlp.down_bias, post_w=layer.norm2b, eps=eps, **after)
+            if hook is not None:
+                hook(i, x)
+        if not n_want:
+            return None
+        if hook is not None and want is not None:
+            h = h[want.long()]
+        return K.softcap(F.linear(h, self.output.weight), cfg.vocab_size, cfg.logit_softcap)
+
+    @torch.no_grad()
+    def prompt_pass(self, b: PromptBatch, want: Sequence[int], hook=None) -> Optional[torch.Tensor]:
+        """logits (fp32) of the packed rows `want`; the cache rows of every token are written"""
+        w = torch.tensor(list(want), dtype=torch.int32).to(b.tokens.device) if len(want) else None
+        return self._run(b, lambda m, h: m.prompt(h, b), w, len(want), hook)
+
+    @torch.no_grad()
+    def step_pass(self, b: StepBatch, hook=None) -> torch.Tensor:
+        """logits (fp32 [batch, vocab]) of one token per sequence"""
+        return self._run(b, lambda m, h: m.step(h, b), None, b.tokens.numel(), hook)
+
+    @torch.no_grad()
+    def forward(self, idx: torch.Tensor, input_pos: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """model.Transformer's contract: idx [B, S] at positions input_pos [S] of slots 0 .. B - 1 -> logits [B, S, vocab].  S = 1 keeps
+        everything on the device (capturable into a hipGraph)."""
+        assert self.cache is not None, "Caches must be initialized first"
+        B, S = idx.shape
+        if S == 1:
+            pos = input_pos.to(torch.int32).expand(B).contiguous()
+            b = StepBatch(self.cache, idx.view(-1).to(torch.int32), pos, self._slots[:B], self.max_seq_length - 1)
+            return self.step_pass(b).view(B, 1, -1)
+        start = int(input_pos[0])
+        assert start + S <= self.max_seq_length
+        toks = idx.cpu().numpy()
+        b = PromptBatch(self.cache, [(i, start, toks[i]) for i in range(B)], idx.device)
+        return self.prompt_pass(b, range(B * S)).view(B, S, -1)
+
+
+# ------------------------------------------------------------------------------------------------
+# construction
+# ------------------------------------------------------------------------------------------------
+def _empty(cfg: LayeredArgs, device, dtype) -> LayeredTransformer:
+    with torch.device("meta"):
+        model = LayeredTransformer(cfg).to(dtype)
+    model = model.to_empty(device=device)
+    with torch.no_grad():
+        for p in model.parameters():
+            p.zero_()  # (padding rows stay zero)
+    return model
+
+
+def load_layered_checkpoint(path, device, dtype: torch.dtype) -> LayeredTransformer:
+    """a folder with config.json and model.safetensors"""
+    from safetensors import safe_open
+    path = Path(path)
+    with open(path / "config.json") as f:
+        cfg = LayeredArgs.from_dict(json.load(f))
+    model = _empty(cfg, device, dtype)
+    with safe_open(str(path / "model.safetensors"), framework="pt", device="cpu") as st:
+        return model.load_tensors(lambda n: st.get_tensor(n).to(device=device, dtype=dtype))
+
+
+@torch.no_grad()
+def build_layered_model(cfg: LayeredArgs, device, dtype: torch.dtype, seed: int = 1234, std: float = 0.02) -> LayeredTransformer:
+    """random weights at the exact shapes: N(0, std^2) matrices, unit norm weights, zero biases and sinks"""
+    g = torch.Generator(device=device).manual_seed(seed)
+    model = _empty(cfg, device, dtype)
+    shapes = model.tensor_shapes()
+
+    def get(name):
+        shape = shapes[name]
+        if len(shape) == 1:
+            return torch.full(shape, 1.0 if "norm" in name else 0.0, device=device, dtype=dtype)
+        return (torch.randn(shape, device=device, dtype=torch.float32, generator=g) * std).to(dtype)
+
+    return model.load_tensors(get)
+
+
+def is_layered_checkpoint(path) -> bool:
+    """does this folder (or a file in it) belong to a layered design?"""
+    path = Path(path)
+    cfg = (path if path.is_dir() else path.parent) / "config.json"
+    if not cfg.is_file():
+        return False
+    with open(cfg) as f:
+        return json.load(f).get("architecture") in DESIGNS

@@ -1,0 +1,121 @@
+"""Paged per-token cache of the layered designs: fixed-size pages of rows, one page table per live sequence shared by all layers.
+
+Every layer that owns cached rows has a pool [pages * PAGE, row width]; a sequence's page table entry `p // PAGE` names the page
+that holds position p, in every pool.  Pages are handed out as sequences grow and come back when a sequence ends — or, where every
+layer attends through a window, as soon as no query can see them any more (`trim`), so a long sequence holds O(window) pages.
+The table lives on the host (numpy) with a device copy that launches read; `sync()` uploads it when it changed.
+"""
+from __future__ import annotations
+
+from typing import Dict, List, Optional
+
+import numpy as np
+import torch
+
+PAGE_SHIFT = 6
+PAGE = 1 << PAGE_SHIFT
+
+
+class PagedCache:
+    def __init__(self, widths: Dict[int, int], dtype: torch.dtype, device, max_tokens: int, max_requests: int = 8, window: Optional[int] = None):
+        """widths: layer -> elements of its cached row; max_tokens: tokens the live sequences are expected to hold together (the pools
+        grow when it is exceeded); window: the widest span any layer looks back over, itself included (None: everything)."""
+        self.widths, self.dtype, self.device, self.window = dict(widths), dtype, torch.device(device), window
+        self.n_pages = 0
+        self.free: List[int] = []
+        self.pools: Dict[int, torch.Tensor] = {}
+        self.version = 0  # bumped whenever a device buffer is replaced (captured graphs hold its old address)
+        self.slots: List[Optional[List[int]]] = []  # per slot: page ids by position (-1: given back), or None when the slot is free
+        self.lengths: List[int] = []
+        self.host = np.zeros((0, 0), dtype=np.int32)
+        self.table: Optional[torch.Tensor] = None
+        self._dirty = True
+        self._grow_table(max(1, max_requests), max(1, -(-max_tokens // PAGE)))
+        self._grow_pools(-(-max_tokens // PAGE) + max_requests)
+
+    # ---- storage ---------------------------------------------------------------------------------------------------
+    def _grow_pools(self, pages: int) -> None:
+        if pages <= self.n_pages:
+            return
+        for layer, width in self.widths.items():
+            new = torch.zeros(pages * PAGE, width, dtype=self.dtype, device=self.device)
+            if self.n_pages:
+                new[: self.n_pages * PAGE] = self.pools[layer]
+            self.pools[layer] = new
+        self.free.extend(range(pages - 1, self.n_pages - 1, -1))  # (taken from the end: lowest page first)
+        self.n_pages = pages
+        self.version += 1
+
+    def _grow_table(self, rows: int, cols: int) -> None:
+        r, c = self.host.shape
+        if rows <= r and cols <= c:
+            return
+        host = np.zeros((max(rows, r), max(cols, c)), dtype=np.int32)
+        host[:r, :c] = self.host
+        self.host = host
+        while len(self.slots) < host.shape[0]:
+            self.slots.append(None)
+            self.lengths.append(0)
+        self.table = torch.zeros(host.shape, dtype=torch.int32, device=self.device)
+        self._dirty = True
+        self.version += 1
+
+    def bytes(self) -> int:
+        return sum(p.numel() * p.element_size() for p in self.pools.values())
+
+    # ---- sequences -------------------------------------------------------------------------------------------------
+    def open(self) -> int:
+        """a slot for a new sequence"""
+        if None not in self.slots:
+            self._grow_table(2 * len(self.slots), self.host.shape[1])
+        s = self.slots.index(None)
+        self.slots[s], self.lengths[s] = [], 0
+        return s
+
+    def extend(self, slot: int, length: int) -> None:
+        """room for positions 0 .. length - 1 of the slot's sequence"""
+        pages = self.slots[slot]
+        need = -(-length // PAGE)
+        if need > self.host.shape[1]:
+            self._grow_table(self.host.shape[0], max(need, 2 * self.host.shape[1]))
+        while len(pages) < need:
+            if not self.free:
+                self._grow_pools(self.n_pages + max(8, self.n_pages // 2))
+            pg = self.free.pop()
+            self.host[slot, len(pages)] = pg
+            pages.append(pg)
+            self._dirty = True
+        self.lengths[slot] = max(self.lengths[slot], length)
+
+    def trim(self, slot: int) -> None:
+        """give back the pages that the next position's window no longer reaches"""
+        if self.window is None:
+            return
+        pages = self.slots[slot]
+        keep = max(0, self.lengths[slot] - self.window + 1) // PAGE
+        for i in range(keep - 1, -1, -1):
+            if pages[i] < 0:
+                break
+            self.free.append(pages[i])
+            pages[i] = -1
+            self.host[slot, i] = 0  # (a valid page; nothing reads it through this entry again)
+            self._dirty = True
+
+    def close(self, slot: int) -> None:
+        self.free.extend(p for p in reversed(self.slots[slot]) if p >= 0)
+        self.slots[slot], self.lengths[slot] = None, 0
+        self.host[slot] = 0
+        self._dirty = True
+
+    def rows(self, slot: int, positions: np.ndarray) -> np.ndarray:
+        """pool rows of a sequence's positions"""
+        return self.host[slot][positions >> PAGE_SHIFT] * PAGE + (positions & (PAGE - 1))
+
+    def sync(self) -> None:
+        if self._dirty:
+            self.table.copy_(torch.from_numpy(self.host))
+            self._dirty = False
+
+    @property
+    def pages_in_use(self) -> int:
+        return self.n_pages - len(self.free)

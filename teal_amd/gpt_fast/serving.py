@@ -1,0 +1,111 @@
+"""Batched serving of the layered designs: requests of different lengths in one step, over one paged cache.
+
+`BatchEngine.step` takes the next tokens of any number of requests and returns the logits asked for: single tokens of running
+requests go through the decode step, anything else (new prompts, portions of prompts, a mixture) through the ragged prompt pass.
+`generate_batch` is the scheduler on top: it admits requests, prefills them (in portions when asked), decodes the running batch
+token by token with the framework's sampler and retires each request at its own length.
+"""
+from __future__ import annotations
+
+from dataclasses import dataclass
+from typing import Dict, Hashable, List, Optional, Sequence
+
+import numpy as np
+import torch
+
+from .layered import LayeredTransformer, PromptBatch, StepBatch
+
+
+class BatchEngine:
+    def __init__(self, model: LayeredTransformer, max_tokens: int = 4096, max_requests: int = 8):
+        self.model = model
+        self.device = model.tok_embeddings.weight.device
+        self.cache = model.new_cache(max_tokens, max_requests)
+        self.slot: Dict[Hashable, int] = {}
+
+    def length(self, rid: Hashable) -> int:
+        return self.cache.lengths[self.slot[rid]] if rid in self.slot else 0
+
+    def step(self, entries: Sequence[tuple], hook=None) -> Optional[torch.Tensor]:
+        """entries: [(request, its next tokens, places among them whose logits are wanted)].  Returns fp32 [wanted, vocab] in the order
+        of the entries and places, or None when nothing is wanted."""
+        vocab = self.model.config.vocab_size
+        batch, want, at = [], [], 0
+        for rid, tokens, places in entries:
+            if not len(tokens) or min(tokens) < 0 or max(tokens) >= vocab or any(not 0 <= k < len(tokens) for k in places):
+                raise ValueError(f"request {rid!r}: no tokens, a token outside the vocabulary or a place outside the tokens")
+        if len({e[0] for e in entries}) != len(entries):
+            raise ValueError("a request appears twice in one step")
+        for rid, tokens, places in entries:
+            if rid not in self.slot:
+                self.slot[rid] = self.cache.open()
+            s = self.slot[rid]
+            start = self.cache.lengths[s]
+            self.cache.extend(s, start + len(tokens))
+            batch.append((s, start, tokens))
+            want.extend(at + k for k in places)
+            at += len(tokens)
+        self.cache.sync()
+        if all(start > 0 and len(t) == 1 for _, start, t in batch):
+            flat = np.asarray([[t[0] for _, _, t in batch], [st for _, st, _ in batch], [s for s, _, _ in batch]], dtype=np.int32)
+            dev = torch.from_numpy(flat).to(self.device)
+            logits = self.model.step_pass(StepBatch(self.cache, dev[0], dev[1], dev[2], int(flat[1].max())), hook)
+            out = None if not want else logits if len(want) == len(batch) else logits[torch.tensor(want, device=self.device)]
+        else:
+            out = self.model.prompt_pass(PromptBatch(self.cache, batch, self.device), want, hook)
+        for s, _, _ in batch:
+            self.cache.trim(s)
+        return out
+
+    def release(self, rid: Hashable) -> None:
+        """the request is finished: its pages and slot go back"""
+        self.cache.close(self.slot.pop(rid))
+
+
+@dataclass
+class Request:
+    prompt: Sequence[int]
+    max_new_tokens: int
+
+
+@torch.no_grad()
+def generate_batch(model: LayeredTransformer, requests: Sequence[Request], temperature: float = 0.0, top_k: Optional[int] = None,
+                   max_batch: int = 64, portion: Optional[int] = None, engine: Optional[BatchEngine] = None) -> List[List[int]]:
+    """New tokens of every request.  At most max_batch run at a time, a waiting request is admitted as soon as one retires;
+    prompts enter whole or `portion` tokens at a time.  temperature <= 0: greedy; else the framework's top-k sampler."""
+    from .generate import sample_rows
+    eng = engine or BatchEngine(model, max_tokens=max(sum(len(r.prompt) + r.max_new_tokens for r in requests[:max_batch]), 64), max_requests=max_batch)
+    out: List[List[int]] = [[] for _ in requests]
+    waiting = [i for i, r in enumerate(requests) if r.max_new_tokens > 0]
+    running: List[int] = []
+
+    def emit(ids, logits):
+        for i, t in zip(ids, sample_rows(logits, temperature, top_k).tolist()):
+            out[i].append(t)
+            if len(out[i]) >= requests[i].max_new_tokens:
+                eng.release(i)
+                if i in running:
+                    running.remove(i)
+            elif i not in running:
+                running.append(i)
+
+    while waiting or running:
+        new = [waiting.pop(0) for _ in range(min(len(waiting), max_batch - len(running)))]
+        if new:
+            size = portion or max(len(requests[i].prompt) for i in new)
+            left = {i: list(requests[i].prompt) for i in new}
+            while left:
+                entries, done = [], []
+                for i in list(left):
+                    part, left[i] = left[i][:size], left[i][size:]
+                    if not left[i]:
+                        del left[i]
+                        done.append(i)
+                    entries.append((i, part, [len(part) - 1] if i in done else []))
+                logits = eng.step(entries)
+                if done:
+                    emit(done, logits)
+        if running:
+            ids = list(running)
+            emit(ids, eng.step([(i, [out[i][-1]], [0]) for i in ids]))
+    return out
