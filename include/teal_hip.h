@@ -175,6 +175,11 @@ int teal_sparse_gateup_silu(const void* x, const void* w1T, const void* w3T, voi
                               * teal_decode_attention_split(y = NULL, nsplit = 4 or 8): x points at the fp32
                               * partials [Z/head_dim][nsplit][head_dim + 2]; att_head_dim = head_dim,
                               * att_nsplit = nsplit (0 means 4); Z <= 16384 (nsplit 4) / 8192 (nsplit 8) */
+#define TEAL_IN_RESID32_NORM 5 /* the layered designs' residual, held in fp32: x = resid + y * (1 / rms(y)) * post, y = sum slabs + bias
+                              * (no slabs: x = resid), then RMSNorm(x) * pre.  resid_in fp32 [Z] (with row_index: the 16-bit table
+                              * [rows][Z]), norm_weight = three 16-bit vectors [3][Z] = pre | post | bias, resid_out fp32 [Z]; slabs
+                              * interleaved.  Z % 64 == 0, Z <= 8192, segments whole 64-column tiles of 16-bit weights; other shapes
+                              * return TEAL_ERR_CONFIG without launching.  Out modes ROUNDED, SLABS, SLAB_SUM */
 #define TEAL_OUT_ROUNDED 0   /* y rounded to dtype (runs the ordered slab reduce when split-K is used) */
 #define TEAL_OUT_SLABS 1     /* leave the fp32 split-K slabs for the next launch's RESID_NORM producer */
 #define TEAL_OUT_QKV_ROPE 3  /* nseg == 3 = q | k | v of ONE fused wqkv image, RESID_NORM input: when the launch needs no
@@ -256,6 +261,10 @@ typedef struct teal_gemv_out {
                                 * call made, NUL-terminated (as rocprofv3 prints it; e.g. to name the kernel in a benchmark
                                 * record) — per call, no library state */
     int desc_bytes;            /* capacity of desc (160 is enough) */
+    /* TEAL_IN_RESID32_NORM launches only (zero otherwise), ROUNDED and SLAB_SUM outputs: */
+    const void* bias;          /* 16-bit [sum ncols]: added to the complete sums; act_seg0 = 2 then applies gelu (tanh form) to
+                                * segment 0 */
+    float softcap;             /* > 0: the output is softcap * tanh(sum / softcap) */
 } teal_gemv_out_t;
 
 /* One launch: [fused producer] -> mask + compaction -> gathered GEMV over every segment.
@@ -394,6 +403,11 @@ int teal_gated_act(const void* gu, int ldg, int up0, const void* bias_gate, cons
                    int act, int dtype, void* stream);
 /* out (fp32 [n_rows][vocab]) = cap * tanh(logits / cap); cap <= 0: the conversion alone */
 int teal_logit_softcap(const void* logits, int ld, float* out, int n_rows, int vocab, float cap, int dtype, void* stream);
+/* One token per row of fp32 logits [n_rows][ld]: top-k filter (ties at the k-th stay; top_k <= 0 or >= vocab: none), softmax, exponential
+ * race; temperature <= 0: the largest logit (the lowest index of equals).  rng_state = device uint64 [n_rows][2] {seed, draw counter},
+ * bumped per draw; optional loop state: pos_inout[row] += 1, history[row][draw counter] = token. */
+int teal_sample_rows(const float* logits, int ld, int n_rows, int vocab, int top_k, float temperature, void* rng_state, int32_t* token_out,
+                     int32_t* pos_inout, int32_t* history, int history_len, void* stream);
 
 /* ---- latent attention, teal_amd/csrc/teal_latent.hip -------------------------------------------------------------------
  * Sizes: heads; per head dim unrotated + rot rotated query / key dimensions and vdim value dimensions; rank = size of the latent.

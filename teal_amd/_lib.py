@@ -56,7 +56,7 @@ DIAG_LIB_PATH = os.path.join(_PKG, "libteal_hip_diag.so")
 # lacks are tolerated (OPTIONAL_WITH_OVERRIDE).
 LIB_OVERRIDE = os.environ.get("TEAL_LIB_PATH") or None
 OPTIONAL_WITH_OVERRIDE = ("teal_decode_attention_split_roped", "teal_prefill_gemm", "teal_prefill_resid_norm", "teal_prefill_attention",
-                          "teal_layer_resid_norm", "teal_gated_act", "teal_logit_softcap", "teal_latent_prompt_rows", "teal_latent_gather",
+                          "teal_layer_resid_norm", "teal_gated_act", "teal_logit_softcap", "teal_sample_rows", "teal_latent_prompt_rows", "teal_latent_gather",
                           "teal_latent_prompt_tile", "teal_latent_prompt_attention", "teal_latent_step_query", "teal_latent_step_attention",
                           "teal_latent_step_merge")
 
@@ -68,7 +68,7 @@ EXPORTS = (
     "teal_workspace_init", "teal_workspace_release", "teal_sample_topk_ws", "teal_decode_attention_split_ws", "teal_cmp_flag_gemv",
     "teal_decode_attention_split_roped",
     "teal_prefill_gemm", "teal_prefill_resid_norm", "teal_prefill_attention",
-    "teal_layer_resid_norm", "teal_gated_act", "teal_logit_softcap",
+    "teal_layer_resid_norm", "teal_gated_act", "teal_logit_softcap", "teal_sample_rows",
     "teal_latent_prompt_rows", "teal_latent_gather", "teal_latent_prompt_tile", "teal_latent_prompt_attention",
     "teal_latent_step_query", "teal_latent_step_attention", "teal_latent_step_merge",
 )
@@ -201,6 +201,7 @@ def _open(path: str, diag: bool) -> ctypes.CDLL:
         L.teal_layer_resid_norm.argtypes = [vp, ci, ci, vp, vp, ci, vp, ci, vp, vp, vp, cf, vp, vp, ci, vp]
         L.teal_gated_act.argtypes = [vp, ci, ci, vp, vp, vp, ci, ci, ci, ci, ci, vp]
         L.teal_logit_softcap.argtypes = [vp, ci, vp, ci, ci, cf, ci, vp]
+        L.teal_sample_rows.argtypes = [vp, ci, ci, ci, ci, cf, vp, vp, vp, vp, ci, vp]
         L.teal_latent_prompt_rows.argtypes = [vp, ci, ci, ci, vp, vp, vp, vp, cf, ci, ci, ci, ci, vp, ci, ci, vp]
         L.teal_latent_gather.argtypes = [vp, ci, vp, ci, ci, ci, vp, vp, ci, vp]
         L.teal_latent_prompt_tile.argtypes = [ci, ci, ci, ci, ci]

@@ -48,6 +48,7 @@ struct InSpec {
     int slabs_il;              // mode 1: slabs are interleaved [Z][(nslabs + 3) & ~3] (one 16-byte load per element)
     const unsigned long long* masks;  // mode 3: keep masks (one per 64 activations) emitted by the producer
     float eps;
+    // mode 5: residual fp32 (resid_in; the 16-bit table with row_index), norm_w = [3][Z] pre-norm weight | post-norm weight | bias
     int gate_act;              // mode 2: the gate half already holds round(silu(gate)): x = round(gate * up)
 };
 
@@ -77,6 +78,8 @@ struct Params {
     int rope_hd, rope_max_seq;
     int act0;                   // rounded output of segment 0 goes through silu (and is rounded again)
     int sum32;                  // TEAL_OUT_SLAB_SUM: seg[0].y is fp32 and receives the unrounded slice-order sum (lean kernel only)
+    const uint16_t* bias;       // mode 5: added to the complete sums (16-bit, element 0 = first column of segment 0)
+    float softcap;              // mode 5: cap * tanh(sum / cap)
     Seg seg[kMaxSeg];
 };
 
@@ -294,6 +297,13 @@ __device__ __forceinline__ float row_slices_sum(float v) {
     }
 }
 
+
+// counter-based random bits of the samplers: (seed, draw counter, index)
+__device__ __forceinline__ uint32_t hash3(uint32_t a, uint32_t b, uint32_t c) {
+    uint32_t h = a * 0x9E3779B1u ^ (b + 0x7F4A7C15u) * 0x85EBCA77u ^ (c + 0x165667B1u) * 0xC2B2AE3Du;
+    h ^= h >> 16; h *= 0x85EBCA6Bu; h ^= h >> 13; h *= 0xC2B2AE35u; h ^= h >> 16;
+    return h;
+}
 
 __device__ __forceinline__ int lane_rank(unsigned long long mask) {
     return __builtin_amdgcn_mbcnt_hi((uint32_t)(mask >> 32),

@@ -39,13 +39,17 @@ namespace teal {
 //   gate|up contiguous [2Z] at in0 (gpt-fast/model.py:258-259, the roundings of the unfused sequence); 3 x + producer
 //   masks (in0 x, in1 masks); 4 split-KV attention partials (in0).  Element-wise modes (0, 2, 3, 4) cache the rounds of
 //   the workgroup's own slice only: register k <-> chunk slice + split * (wave + 16 k).
-//   EXACT (MODE 1): Z == 1024 * KR, every cached chunk exists — no clamps, no guards.
+//   5 the fp32 residual of the layered designs: x = resid + [post norm](slabs + bias), then RMSNorm (in0 fp32 residual — or the 16-bit
+//   embedding table with row_index —, in1 slabs, in2 the three vectors [3][Z] pre-norm weight | post-norm weight | bias); its epilogue
+//   can add a bias, apply gelu to segment 0 and cap logits (FastArgs.bias / act0 / softcap).
+//   EXACT (MODE 1, 5): Z == 1024 * KR, every cached chunk exists — no clamps, no guards.
 template <bool BF16, int MODE, bool PAIR, int LPR, int KR, bool EXACT, bool PHASE, int U = 4, bool W8 = false, bool ROPE = false>
 __global__ __launch_bounds__(1024) void gemv_fast_kernel(const void* in0, const void* in1, const void* in2,
                                                          const int* row_index, const int Z, const int nslabs,
                                                          const float eps, const int split_p, const FastArgs a) {
     static_assert(!(W8 && PAIR), "int8 gate|up runs unpaired (two images of 128-byte row segments)");
     static_assert(!ROPE || (MODE == 1 && !PAIR && !W8), "the RoPE / KV-append epilogue belongs to the fused wqkv projection");
+    constexpr bool WHOLE = MODE == 1 || MODE == 5;  // a normalising producer: every workgroup caches the whole vector
     constexpr int WAVES = 16;
     constexpr int RPW = 64 / LPR;
     // a lane owns 8 columns: 16 bytes of 16-bit weights, 8 bytes of int8 weights (the same lane <-> row mapping, hence the
@@ -80,8 +84,8 @@ __global__ __launch_bounds__(1024) void gemv_fast_kernel(const void* in0, const 
     float sumsq_part = 0.0f;
     int rope_p = 0;            // ROPE: clamped position of the token
     uint32_t rope_cs = 0u;     // ROPE: (cos | sin << 16) of this thread's column pair
-    float rv[MODE == 1 ? KR : 1];
-    uint32_t wb[MODE == 1 ? KR : 1];
+    float rv[WHOLE ? KR : 1];
+    uint32_t wb[WHOLE ? KR : 1];
     unsigned long long mk[MODE == 3 ? KR : 1];
     {
         // Which chunks (64 activations) a workgroup streams — balanced over the slices to within one chunk (round 4; whole
@@ -93,7 +97,7 @@ __global__ __launch_bounds__(1024) void gemv_fast_kernel(const void* in0, const 
         // sparse_gemv_kernel (teal_gemv_kernel.h: chunk_of / kmod) uses the same rule: bit-identical outputs.
         // (own[] is filled in right before the compaction)
 #pragma unroll
-        for (int k = 0; k < KR; ++k) cidx[k] = MODE == 1 ? wave + WAVES * k : slice + split * (wave + WAVES * k);
+        for (int k = 0; k < KR; ++k) cidx[k] = WHOLE ? wave + WAVES * k : slice + split * (wave + WAVES * k);
     }
     if constexpr (MODE == 1) {
         const uint16_t* resid = x16;
@@ -183,6 +187,78 @@ __global__ __launch_bounds__(1024) void gemv_fast_kernel(const void* in0, const 
             const float xn = bits_to_float(float_to_bits<BF16>(rv[k] * rstd), BF16);
             xr[k] = float_to_bits<BF16>(xn * bits_to_float(wb[k], BF16));
             if (writer && (EXACT || cidx[k] < nch)) rout[(uint32_t)cidx[k] * 64u + lane] = float_to_bits<BF16>(rv[k]);
+        }
+    } else if constexpr (MODE == 5) {
+        typedef float f32x4 __attribute__((ext_vector_type(4)));
+        const uint16_t* vec3 = reinterpret_cast<const uint16_t*>(in2);
+        const float* slabs = reinterpret_cast<const float*>(in1);
+        const uint32_t stride = (uint32_t)(nslabs + 3) & ~3u;
+        uint32_t pb[KR], bb[KR], mel[KR];
+        f32x4 v0[KR], v1[KR];
+#pragma unroll
+        for (int k = 0; k < KR; ++k) {
+            mel[k] = (uint32_t)(EXACT ? cidx[k] : min(cidx[k], nch - 1)) * 64u + lane;
+            wb[k] = vec3[mel[k]];
+            pb[k] = vec3[(uint32_t)Z + mel[k]];
+            bb[k] = vec3[2u * (uint32_t)Z + mel[k]];
+        }
+        if (row_index) {
+            const uint16_t* e = x16 + (size_t)row_index[0] * (size_t)Z;
+#pragma unroll
+            for (int k = 0; k < KR; ++k) rv[k] = bits_to_float(e[mel[k]], BF16);
+        } else {
+#pragma unroll
+            for (int k = 0; k < KR; ++k) rv[k] = reinterpret_cast<const float*>(in0)[mel[k]];
+        }
+        if (nslabs > 0) {
+#pragma unroll
+            for (int k = 0; k < KR; ++k) v0[k] = *reinterpret_cast<const f32x4*>(slabs + mel[k] * stride);
+        }
+        if (nslabs > 4) {
+#pragma unroll
+            for (int k = 0; k < KR; ++k) v1[k] = *reinterpret_cast<const f32x4*>(slabs + mel[k] * stride + 4);
+        }
+        TEAL_FAST_ARGS_BATCH(a);
+        float* sumsq = reinterpret_cast<float*>(smem);
+        // sum over the workgroup; the barrier in front lets the scratch be used twice
+        auto total = [&](const float part) {
+            const float ws = wave_sum_f(part);
+            __syncthreads();
+            if (lane == 0) sumsq[wave] = ws;
+            __syncthreads();
+            return wave_sum_f(lane < WAVES ? sumsq[lane] : 0.0f);
+        };
+        if (nslabs > 0) {
+            float yv[KR], part = 0.0f;
+#pragma unroll
+            for (int k = 0; k < KR; ++k) {
+                float sacc = 0.0f;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) sacc += (j < nslabs) ? v0[k][j] : 0.0f;
+                if (nslabs > 4) {
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) sacc += (4 + j < nslabs) ? v1[k][j] : 0.0f;
+                }
+                yv[k] = sacc + bits_to_float(bb[k], BF16);
+                if (!EXACT) yv[k] = (cidx[k] < nch) ? yv[k] : 0.0f;
+                part = fmaf(yv[k], yv[k], part);
+            }
+            const float rstd_y = 1.0f / sqrtf(total(part) / (float)Z + eps);
+#pragma unroll
+            for (int k = 0; k < KR; ++k) rv[k] += yv[k] * rstd_y * bits_to_float(pb[k], BF16);
+        }
+#pragma unroll
+        for (int k = 0; k < KR; ++k) {
+            if (!EXACT) rv[k] = (cidx[k] < nch) ? rv[k] : 0.0f;
+            sumsq_part = fmaf(rv[k], rv[k], sumsq_part);
+        }
+        const float rstd = 1.0f / sqrtf(total(sumsq_part) / (float)Z + eps);
+        float* rout = reinterpret_cast<float*>(a.resid_out);
+        const bool writer = rout && blockIdx.x == 0 && blockIdx.y == 0;
+#pragma unroll
+        for (int k = 0; k < KR; ++k) {
+            xr[k] = float_to_bits<BF16>(rv[k] * rstd * bits_to_float(wb[k], BF16));
+            if (writer && (EXACT || cidx[k] < nch)) rout[mel[k]] = rv[k];
         }
     } else if constexpr (MODE == 4) {
         // attention output merged from the split-KV partials {max, sum, o[hd]} per (head, split): see the merge
@@ -283,10 +359,10 @@ __global__ __launch_bounds__(1024) void gemv_fast_kernel(const void* in0, const 
     const float tau_s = s == 0 ? a.tau0 : (s == 1 ? a.tau1 : a.tau2);
     const float tau = PAIR ? fminf(a.tau0, a.tau1) : tau_s;  // PAIR: union of the two keep sets
     {
-        int kmod = (MODE == 1 && split > 1) ? wave % split : 0;
+        int kmod = (WHOLE && split > 1) ? wave % split : 0;
 #pragma unroll
         for (int k = 0; k < KR; ++k) {
-            own[k] = (EXACT || cidx[k] < nch) && (MODE != 1 || kmod == slice);
+            own[k] = (EXACT || cidx[k] < nch) && (!WHOLE || kmod == slice);
             kmod = (kmod + 1 == split) ? 0 : kmod + 1;
         }
     }
@@ -462,6 +538,14 @@ __global__ __launch_bounds__(1024) void gemv_fast_kernel(const void* in0, const 
     }
     __syncthreads();
     stamp(6);
+    // MODE 5: column c's complete sum on its way out
+    [[maybe_unused]] auto finish5 = [&](float v, const uint32_t c) {
+        if (a.bias) v += bits_to_float(a.bias[c], BF16);
+        if (s == 0 && a.act0 == 2) v = 0.5f * v * (1.0f + tanhf(0.7978845608028654f * fmaf(0.044715f * v * v, v, v)));
+        if (a.softcap > 0.0f) v = a.softcap * tanhf(v / a.softcap);
+        if (a.sum32) reinterpret_cast<float*>(a.y)[c] = v;
+        else reinterpret_cast<uint16_t*>(a.y)[c] = float_to_bits<BF16>(v);
+    };
     if (tid < BN) {  // whole waves: BN is a multiple of 64
         const uint32_t c = (uint32_t)tile * BN + tid;
         float gs = 0.0f, us = 0.0f;
@@ -491,7 +575,9 @@ __global__ __launch_bounds__(1024) void gemv_fast_kernel(const void* in0, const 
             const unsigned long long mko = __ballot(keep_rule(hv, a.mask_tau) || (hv != hv));
             if (a.mask_out && lane == 0) a.mask_out[c >> 6] = mko;
         } else if (a.ws_stride == 0) {
-            if constexpr (ROPE) {
+            if constexpr (MODE == 5) {
+                finish5(gs, c);
+            } else if constexpr (ROPE) {
                 // gpt-fast/model.py:170-178: q and the new k row are rotated (pairs of adjacent columns: lane ^ 1 holds the
                 // partner), k and v go straight into their cache rows; the roundings are those of the unfused sequence
                 // (projection rounded, rotation in fp32, rounded again — what the attention launch did with the same helpers)
@@ -542,7 +628,8 @@ __global__ __launch_bounds__(1024) void gemv_fast_kernel(const void* in0, const 
                 float sum = 0.0f;
                 for (int sl = 0; sl < split; ++sl)
                     sum += __hip_atomic_load(&a.ws[c * (uint32_t)a.ws_stride + sl], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-                if (a.sum32) reinterpret_cast<float*>(a.y)[c] = sum;  // TEAL_OUT_SLAB_SUM: slice-order fp32 sum, rounded by the consumer
+                if constexpr (MODE == 5) finish5(sum, c);
+                else if (a.sum32) reinterpret_cast<float*>(a.y)[c] = sum;  // TEAL_OUT_SLAB_SUM: slice-order fp32 sum, rounded by the consumer
                 else reinterpret_cast<uint16_t*>(a.y)[c] = (a.act0 && s == 0) ? silu_bits<BF16>(sum) : float_to_bits<BF16>(sum);
                 if (tid == 0) __hip_atomic_store(&a.ticket[tile], 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
             }
@@ -595,7 +682,7 @@ hipError_t launch_fast_e(const FastLaunch& f, hipStream_t st) {
 
 template <bool BF16, int MODE, bool PAIR, int LPR, int KR, bool W8 = false>
 hipError_t launch_fast_k(const FastLaunch& f, hipStream_t st) {
-    if constexpr (MODE == 1) {
+    if constexpr (MODE == 1 || MODE == 5) {
         if (f.Z == 1024 * KR) return launch_fast_e<BF16, MODE, PAIR, LPR, KR, true, W8>(f, st);
     }
     return launch_fast_e<BF16, MODE, PAIR, LPR, KR, false, W8>(f, st);
@@ -608,6 +695,12 @@ hipError_t launch_fast_r(const FastLaunch& f, hipStream_t st) {
             case 4: return launch_fast_k<BF16, MODE, PAIR, LPR, 4, W8>(f, st);
             case 8: return launch_fast_k<BF16, MODE, PAIR, LPR, 8, W8>(f, st);
             case 16: return launch_fast_k<BF16, MODE, PAIR, LPR, 16, W8>(f, st);
+            default: return hipErrorInvalidValue;
+        }
+    } else if constexpr (MODE == 5) {
+        switch (f.kr) {
+            case 4: return launch_fast_k<BF16, MODE, PAIR, LPR, 4, W8>(f, st);
+            case 8: return launch_fast_k<BF16, MODE, PAIR, LPR, 8, W8>(f, st);
             default: return hipErrorInvalidValue;
         }
     } else {
@@ -629,6 +722,7 @@ hipError_t launch_fast_m(const FastLaunch& f, hipStream_t st) {
         case 2: return launch_fast_r<BF16, 2, false, LPR>(f, st);
         case 3: return launch_fast_r<BF16, 3, false, LPR>(f, st);
         case 4: return launch_fast_r<BF16, 4, false, LPR>(f, st);
+        case 5: return launch_fast_r<BF16, 5, false, LPR>(f, st);
         default: return hipErrorInvalidValue;
     }
 }

@@ -34,6 +34,9 @@ struct FastArgs {
     int act0;                       // rounded output of threshold segment 0 goes through silu (the gate of gate | up)
     int gate_act;                   // MODE 2: the gate half already holds round(silu(gate))
     int sum32;                      // TEAL_OUT_SLAB_SUM: y is fp32 [ncols] and receives the unrounded sum over the row slices (slice order)
+    // MODE 5 epilogue (whatever of it is set): + bias[column], the activation of segment 0 (act0 = 2: gelu, tanh form), the soft cap
+    const uint16_t* bias;
+    float softcap;
 };
 
 // Launch description filled by run_gemv when the shape qualifies (teal_kernels.hip: fast_eligible)

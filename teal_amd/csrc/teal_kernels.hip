@@ -250,7 +250,8 @@ bool fast_eligible(const Params& p, const Config& c, bool to_ws, size_t ws_bytes
     if (p.w8 && (c.lpr != 16 || p.pair)) return false;
     if ((p.Z & 63) || p.Z > 65536 || !p.wl) return false;
     const int mode = p.in.mode;
-    if (mode != 0 && mode != 1 && mode != 2 && mode != 3 && mode != 4) return false;
+    if (mode != 0 && mode != 1 && mode != 2 && mode != 3 && mode != 4 && mode != 5) return false;
+    if (mode == 5 && (p.w8 || p.pair)) return false;
     const int bn = c.lpr * 8, nch = p.Z >> 6, owned_all = (nch + 15) / 16;
     // outputs: interleaved slabs for the next launch; one rounded vector (split == 1); or split > 1 folded into ONE
     // launch by arrival tickets (the last slice of a tile sums the partials in slice order)
@@ -275,8 +276,8 @@ bool fast_eligible(const Params& p, const Config& c, bool to_ws, size_t ws_bytes
     }
     if (p.pair && (mode != 1 || p.seg[0].ncols != p.seg[1].ncols)) return false;
     int kr, rounds_owned;
-    if (mode == 1) {
-        if (owned_all > 16 || c.split > owned_all) return false;
+    if (mode == 1 || mode == 5) {
+        if (owned_all > (mode == 5 ? 8 : 16) || c.split > owned_all) return false;
         kr = owned_all <= 4 ? 4 : (owned_all <= 8 ? 8 : 16);
         rounds_owned = (kr + c.split - 1) / c.split;
     } else {
@@ -299,6 +300,9 @@ bool fast_eligible(const Params& p, const Config& c, bool to_ws, size_t ws_bytes
                 if (p.in.nslabs > 0 && !p.in.slabs_il && p.in.nslabs != 1) return false;
                 if (p.in.nslabs > 8) return false;
                 if (p.in.nslabs == 1 && !p.in.slabs_il) f.nslabs = 1 | 0x100;
+                break;
+        case 5: f.in0 = p.in.resid_in; f.in1 = p.in.slabs; f.in2 = p.in.norm_w; f.row_index = p.in.row_index;
+                if (p.in.nslabs > 8 || (p.in.nslabs > 0 && !p.in.slabs_il)) return false;
                 break;
         case 2: f.in0 = p.x; break;  // gate | up contiguous [2Z]
         case 3: f.in0 = p.x; f.in1 = p.in.masks; break;
@@ -328,6 +332,8 @@ bool fast_eligible(const Params& p, const Config& c, bool to_ws, size_t ws_bytes
     f.a.seg_tile2 = (!p.pair && p.nseg > 2) ? p.seg[2].tile0 : INT_MAX;
     f.a.act0 = p.act0;
     f.a.sum32 = p.sum32;
+    f.a.bias = p.bias;
+    f.a.softcap = p.softcap;
     if (p.sum32 && (to_ws || p.pair || p.nseg != 1 || p.act0 || p.rope)) return false;
     f.a.gate_act = p.in.gate_act;
     f.a.ws_stride = (to_ws || ticketed) ? ((c.split + 3) & ~3) : 0;
@@ -408,6 +414,16 @@ int run_gemv(Params& p, int dtype, void* ws, size_t ws_bytes, bool to_ws, hipStr
         // workgroups (Llama-2-70B down, Z = 28672: 128 tiles x 3 slices = 1.5 rounds -> x 4 = 2 full rounds)
         while (tiles * c.split > ncu && (tiles * c.split) % ncu != 0 && c.split < 8) ++c.split;
     }
+    if (p.in.mode == 5 && !g_override.lpr && !g_override.split) {
+        // the lean kernel only: 128- or 64-column tiles, row slices within what the producer caches
+        bool wide = c.lpr >= 16;
+        for (int i = 0; i < p.nseg; ++i) wide = wide && p.seg[i].ncols % 128 == 0;
+        c.lpr = wide ? 16 : 8;
+        const int rounds = (((p.Z + 63) >> 6) + 15) / 16;
+        if (c.split > rounds) c.split = rounds;
+        if (c.split > 8) c.split = 8;
+        if (!to_ws && !p.tickets) c.split = 1;
+    }
     if (p.w8) {
         // int8: 8 bytes per lane.  The stream is bound by cache-line REQUESTS per CU (measured: a 64-byte and a
         // 128-byte row segment cost the same, ~3.2 ns per row and CU), so a row segment should be a whole 128-byte
@@ -477,7 +493,7 @@ int run_gemv(Params& p, int dtype, void* ws, size_t ws_bytes, bool to_ws, hipStr
         const int owned = (nch + c.waves - 1) / c.waves;  // rounds of `waves` chunks
         // element-wise producers (everything but the RMSNorm, which needs the whole vector in every workgroup)
         // cache only the rounds of the workgroup's slice
-        const bool slice_local = p.in.mode != 1 && c.split > 1;
+        const bool slice_local = p.in.mode != 1 && p.in.mode != 5 && c.split > 1;
         const int need = slice_local ? (owned + c.split - 1) / c.split : owned;
         const int krt = need <= 4 ? 4 : (need <= 8 ? 8 : 16);
         const int capw = (slice_local ? need : (krt + c.split - 1) / c.split) * 64;  // entries one wave can own
@@ -510,6 +526,7 @@ int run_gemv(Params& p, int dtype, void* ws, size_t ws_bytes, bool to_ws, hipStr
         FastLaunch f;
         const bool lean = fast_eligible(p, c, to_ws, ws_bytes, f);
         if (p.rope && !lean) return TEAL_ERR_CONFIG;  // the RoPE epilogue exists in the lean kernel only: never fall through unrotated
+        if (p.in.mode == 5 && !lean) return TEAL_ERR_CONFIG;
         if (p.sum32 && !lean) return TEAL_ERR_CONFIG; // so does the fp32 slice-sum output (needs a prepared workspace when split-K is used)
         if (lean) {
             if (rope_taken) *rope_taken = f.a.rope != nullptr;
@@ -824,6 +841,9 @@ int teal_fused_gemv(const teal_gemv_in_t* in, const teal_gemv_out_t* out, int Z,
             p.x = in->x;
             p.in.masks = reinterpret_cast<const unsigned long long*>(in->masks);
             break;
+        case TEAL_IN_RESID32_NORM:
+            if (Z & 63) return TEAL_ERR_SHAPE;
+            [[fallthrough]];
         case TEAL_IN_RESID_NORM:
             if (!in->resid_in || !in->norm_weight || in->nslabs < 0 || (in->nslabs > 0 && !in->slabs)) return TEAL_ERR_ARG;
             if (in->resid_out == in->resid_in && !in->row_index) return TEAL_ERR_ARG;  // must ping-pong
@@ -856,6 +876,14 @@ int teal_fused_gemv(const teal_gemv_in_t* in, const teal_gemv_out_t* out, int Z,
     if (out->weight_bits != 0 && out->weight_bits != 16 && out->weight_bits != 8) return TEAL_ERR_ARG;
     p.w8 = out->weight_bits == 8 ? 1 : 0;
     hipStream_t st = reinterpret_cast<hipStream_t>(stream);
+    if (in->mode == TEAL_IN_RESID32_NORM) {
+        if (p.w8 || (out->mode != TEAL_OUT_ROUNDED && out->mode != TEAL_OUT_SLABS && out->mode != TEAL_OUT_SLAB_SUM)) return TEAL_ERR_ARG;
+        if (out->mode == TEAL_OUT_SLABS && (out->bias || out->softcap > 0.0f)) return TEAL_ERR_ARG;
+        p.bias = reinterpret_cast<const uint16_t*>(out->bias);
+        p.softcap = out->softcap;
+    } else if (out->bias || out->softcap > 0.0f || out->act_seg0 > 1) {
+        return TEAL_ERR_ARG;
+    }
     Config used = {};
     int rc;
     if (out->mode == TEAL_OUT_PAIR_SILU) {
@@ -881,7 +909,8 @@ int teal_fused_gemv(const teal_gemv_in_t* in, const teal_gemv_out_t* out, int Z,
         rc = run_gemv(p, dtype, ws, ws_bytes, false, st, &used, true, false, true, nullptr, out->desc, out->desc_bytes);
         if (rc == TEAL_OK && nslabs_out) { *nslabs_out = 1; return rc; }
     } else if (out->mode == TEAL_OUT_ROUNDED) {
-        p.act0 = out->act_seg0 ? 1 : 0;
+        p.act0 = in->mode == TEAL_IN_RESID32_NORM ? out->act_seg0 : (out->act_seg0 ? 1 : 0);
+        if (in->mode == TEAL_IN_RESID32_NORM && p.act0 != 0 && p.act0 != 2) return TEAL_ERR_ARG;
         rc = run_gemv(p, dtype, ws, ws_bytes, false, st, &used, false, false, true, nullptr, out->desc, out->desc_bytes);
     } else if (out->mode == TEAL_OUT_QKV_ROPE) {
         if (out->nseg != 3 || in->mode != TEAL_IN_RESID_NORM || !out->y[0] || !out->rope || !out->rope_pos || !out->k_cache ||

@@ -68,6 +68,7 @@ __device__ __forceinline__ void latent_row(const LatentRowArgs& a, const typenam
         out[a.rank + 2 * i] = N::cvt(x);
         out[a.rank + 2 * i + 1] = N::cvt(y);
     }
+    for (int i = a.rank + a.rot + tid; i < a.ldc; i += 256) out[i] = (typename N::S)0;  // (the step's score product runs over whole rows)
 }
 
 template <int DT>

@@ -4,6 +4,7 @@
 //   resid_norm_kernel   x = embedding row | x + [post norm](y + bias), then h = RMSNorm(x) * w   (one workgroup per token)
 //   gated_act_kernel    h = act(gate + bias) * (up + bias)
 //   softcap_kernel      logits -> fp32, cap * tanh(logits / cap)
+//   sample_rows_kernel  one token per row of fp32 logits: top-k filter, softmax, exponential race (or the largest logit)
 #include "teal_layered.h"
 
 namespace teal {
@@ -178,6 +179,114 @@ __global__ __launch_bounds__(256) void softcap_kernel(const typename Num<DT>::S*
     out[(size_t)blockIdx.x * V + n] = cap > 0.0f ? cap * tanhf(v / cap) : v;
 }
 
+// ------------------------------------------------------------------------------------------------
+// Sampler over fp32 logits, one workgroup per row: the 16-bit samplers of teal_attention.hip for logits that are not rounded.  The
+// k-th largest logit is found exactly: keys order like the floats, d = (largest key) - key; a 256-bin histogram of d >> sh covers the
+// keys nearest to the maximum (the others do no atomics), widened until it holds k of them, then the pivot's bin is resolved eight
+// bits at a time.  Ties at the pivot stay in.  The race is the one of the 16-bit samplers: argmax exp((x - max) / T) / Exp(1).
+// ------------------------------------------------------------------------------------------------
+__device__ __forceinline__ uint32_t order_key32(const float f) {
+    const uint32_t b = __float_as_uint(f);
+    return (b & 0x80000000u) ? ~b : (b | 0x80000000u);
+}
+
+__global__ __launch_bounds__(1024) void sample_rows_kernel(const float* __restrict__ logits, const int ld, const int V, const int top_k, const float inv_temp,
+                                                           unsigned long long* __restrict__ rng, int32_t* __restrict__ token_out, int32_t* __restrict__ pos_inout,
+                                                           int32_t* __restrict__ history, const int history_len) {
+    __shared__ unsigned hist[256], sel[2];
+    __shared__ float fred[16];
+    __shared__ int ired[16];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, row = blockIdx.x;
+    const float* x = logits + (size_t)row * ld;
+    float mx = -INFINITY;
+    for (int i = tid; i < V; i += 1024) mx = fmaxf(mx, x[i]);
+    mx = block_max<1024>(mx, fred, tid);
+    const uint32_t kmax = order_key32(mx);
+    uint32_t limit = 0xFFFFFFFFu;  // keep keys with kmax - key <= limit
+    if (top_k > 0 && top_k < V && inv_temp > 0.0f) {
+        // histogram of (d - lo) >> sh for d in [lo, lo + (256 << sh)); leaves the bin of the need-th key in sel[0], its rank there in sel[1],
+        // or sel[1] = 0 when the window holds fewer
+        auto window = [&](const uint32_t lo, const int sh, const unsigned need) {
+            if (tid < 256) hist[tid] = 0u;
+            __syncthreads();
+            for (int i = tid; i < V; i += 1024) {
+                const uint32_t d = kmax - order_key32(x[i]);
+                if (d >= lo && ((d - lo) >> sh) < 256u) atomicAdd(&hist[(d - lo) >> sh], 1u);
+            }
+            __syncthreads();
+            if (tid < 64) {
+                unsigned own = 0u;
+#pragma unroll
+                for (int j = 0; j < 4; ++j) own += hist[4 * tid + j];
+                unsigned incl = own;
+#pragma unroll
+                for (int k = 1; k < 64; k <<= 1) {
+                    const unsigned t = (unsigned)__shfl_up((int)incl, k);
+                    if (tid >= k) incl += t;
+                }
+                unsigned before = incl - own;
+                if (tid == 63 && incl < need) sel[1] = 0u;
+                for (int j = 0; j < 4; ++j) {
+                    const unsigned h = hist[4 * tid + j];
+                    if (before < need && before + h >= need) { sel[0] = 4u * tid + j; sel[1] = need - before; }
+                    before += h;
+                }
+            }
+            __syncthreads();
+        };
+        int sh = 14;
+        window(0u, sh, (unsigned)top_k);
+        while (sel[1] == 0u && sh < 24) {  // (at sh = 24 the window is every key)
+            sh = min(sh + 5, 24);
+            __syncthreads();
+            window(0u, sh, (unsigned)top_k);
+        }
+        uint32_t lo = sel[0] << sh;
+        unsigned need = sel[1];
+        while (sh > 0) {
+            const int step = min(8, sh);
+            __syncthreads();
+            window(lo, sh - step, need);  // (bins past this one's end hold keys of the next: the need-th key comes before them)
+            sh -= step;
+            lo += sel[0] << sh;
+            need = sel[1];
+        }
+        limit = lo;
+    }
+    const uint32_t seed = (uint32_t)rng[2 * row], ctr = (uint32_t)rng[2 * row + 1];
+    float best = -INFINITY;
+    int besti = 0x7FFFFFFF;
+    for (int i = tid; i < V; i += 1024) {
+        const float v = x[i];
+        if (kmax - order_key32(v) > limit) continue;
+        float sc = v;
+        if (inv_temp > 0.0f) {
+            const float u = ((float)(hash3(seed, ctr, (uint32_t)i) >> 8) + 0.5f) * (1.0f / 16777216.0f);
+            sc = expf((v - mx) * inv_temp) / (-logf(u));
+        }
+        if (sc > best || (sc == best && i < besti)) { best = sc; besti = i; }
+    }
+#pragma unroll
+    for (int d = 32; d >= 1; d >>= 1) {
+        const float ob = __shfl_xor(best, d);
+        const int oi = __shfl_xor(besti, d);
+        if (ob > best || (ob == best && oi < besti)) { best = ob; besti = oi; }
+    }
+    __syncthreads();
+    if (lane == 0) { fred[wave] = best; ired[wave] = besti; }
+    __syncthreads();
+    if (tid == 0) {
+        for (int w = 1; w < 16; ++w)
+            if (fred[w] > best || (fred[w] == best && ired[w] < besti)) { best = fred[w]; besti = ired[w]; }
+        besti = besti < V ? besti : 0;  // (a row of NaNs)
+        token_out[row] = besti;
+        const unsigned long long c = rng[2 * row + 1];
+        if (history && c < (unsigned long long)history_len) history[(size_t)row * history_len + c] = besti;
+        rng[2 * row + 1] = c + 1ull;
+        if (pos_inout) pos_inout[row] += 1;
+    }
+}
+
 }  // namespace teal
 
 using namespace teal;
@@ -231,6 +340,15 @@ int teal_logit_softcap(const void* logits, int ld, float* out, int n_rows, int v
                            reinterpret_cast<const typename Num<DT>::S*>(logits), ld, out, vocab, cap);
         return launched();
     });
+}
+
+int teal_sample_rows(const float* logits, int ld, int n_rows, int vocab, int top_k, float temperature, void* rng_state, int32_t* token_out, int32_t* pos_inout,
+                     int32_t* history, int history_len, void* stream) {
+    if (!logits || !rng_state || !token_out || n_rows <= 0 || vocab <= 0 || (history && history_len <= 0)) return TEAL_ERR_ARG;
+    if (ld < vocab) return TEAL_ERR_SHAPE;
+    hipLaunchKernelGGL(sample_rows_kernel, dim3(n_rows), dim3(1024), 0, reinterpret_cast<hipStream_t>(stream), logits, ld, vocab, top_k,
+                       temperature > 0.0f ? 1.0f / temperature : 0.0f, reinterpret_cast<unsigned long long*>(rng_state), token_out, pos_inout, history, history_len);
+    return launched();
 }
 
 }  // extern "C"

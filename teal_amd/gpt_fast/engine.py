@@ -30,7 +30,7 @@ from .. import _lib, runtime
 from ..monkeypatch import UP_SHIFT_BYTES, to_column_major
 from .model import Transformer
 
-TEAL_IN_PLAIN, TEAL_IN_RESID_NORM, TEAL_IN_SILU_MUL, TEAL_IN_MASKED, TEAL_IN_ATTN_MERGE = 0, 1, 2, 3, 4
+TEAL_IN_PLAIN, TEAL_IN_RESID_NORM, TEAL_IN_SILU_MUL, TEAL_IN_MASKED, TEAL_IN_ATTN_MERGE, TEAL_IN_RESID32_NORM = 0, 1, 2, 3, 4, 5
 TEAL_OUT_ROUNDED, TEAL_OUT_SLABS, TEAL_OUT_PAIR_SILU, TEAL_OUT_QKV_ROPE, TEAL_OUT_SLAB_SUM = 0, 1, 2, 3, 4
 MAX_SLABS = 32
 
@@ -52,7 +52,8 @@ class GemvOut(ctypes.Structure):  # teal_gemv_out_t
                 ("scale_ld", ctypes.c_int * 3), ("groupsize", ctypes.c_int),
                 ("rope", ctypes.c_void_p), ("rope_pos", ctypes.c_void_p), ("k_cache", ctypes.c_void_p), ("v_cache", ctypes.c_void_p),
                 ("rope_head_dim", ctypes.c_int), ("rope_max_seq", ctypes.c_int), ("act_seg0", ctypes.c_int),
-                ("desc", ctypes.c_char_p), ("desc_bytes", ctypes.c_int)]
+                ("desc", ctypes.c_char_p), ("desc_bytes", ctypes.c_int),
+                ("bias", ctypes.c_void_p), ("softcap", ctypes.c_float)]
 
 
 def _out(segs, mode, slabs: Optional[torch.Tensor] = None) -> GemvOut:
@@ -78,7 +79,134 @@ def _out(segs, mode, slabs: Optional[torch.Tensor] = None) -> GemvOut:
     return o
 
 
-class DecodeEngine:
+class DecodeLoop:
+    """The device-resident decode loop around a fused step: sampling with in-graph loop state, hipGraph capture of one or several
+    steps, and decode_n.  A subclass is the step — __call__(token [1, 1], position [1]) -> logits — and owns cfg, dtype (of the
+    logits), code, logits, ws, max_seq and reduce (None: one rank); `_init_loop` makes the loop's state."""
+
+    def _init_loop(self, dev) -> None:
+        self.rng_state = torch.tensor([1234, 0], dtype=torch.int64, device=dev)  # {seed, draw counter}
+        self._seed, self._calls = 1234, 0
+        self.token = torch.zeros(1, dtype=torch.int32, device=dev)
+        self.tok_buf = torch.zeros(1, 1, dtype=torch.int32, device=dev)   # loop-carried token
+        self.pos_buf = torch.zeros(1, dtype=torch.int32, device=dev)      # loop-carried position
+        self.history = torch.zeros(max(8, self.max_seq), dtype=torch.int32, device=dev)
+        self._graph, self._graph_key, self._graphs = None, None, {}
+
+    def sample_fused(self, logits: torch.Tensor, temperature: float = 1.0, top_k: Optional[int] = None,
+                     feed: bool = False) -> torch.Tensor:
+        """One launch: top-k filter + softmax + exponential-race multinomial (generate.py:49-66).
+        feed=True also carries the loop state on the device: the token goes into the buffer the next
+        step reads, the position is advanced and the token is appended to `history`."""
+        tok_out = self.tok_buf if feed else self.token
+        rc = self.L.teal_sample_topk_ws(logits.data_ptr(), self.cfg.vocab_size, self.code, int(top_k or 0), float(temperature),
+                                        self.rng_state.data_ptr(), tok_out.data_ptr(),
+                                        self.pos_buf.data_ptr() if feed else None,
+                                        self.history.data_ptr() if feed else None, self.history.numel(),
+                                        self.ws.data_ptr(), self.ws.numel() * 4, runtime.stream_ptr())
+        if rc != 0:
+            _lib.check(rc, "teal_sample_topk")
+        return tok_out
+
+    def manual_seed(self, seed: int):
+        self._seed, self._calls = int(seed), 0
+        self.rng_state.copy_(torch.tensor([seed, 0], dtype=torch.int64))
+
+    # ---- device-resident decode loop: one hipGraph replay == one token, no host-side glue ---------
+    def _self_step(self, temperature, top_k):
+        logits = self(self.tok_buf, self.pos_buf)
+        self.sample_fused(logits, temperature, top_k, feed=True)
+
+    def capture_loop(self, temperature: float, top_k: Optional[int], tokens: int = 1):
+        """hipGraph of `tokens` consecutive decode steps (token, position and RNG counter stay on the device between them, so
+        a graph can span any number of tokens; each replay costs one host launch and one graph boundary on the GPU)."""
+        if self.reduce is not None and not getattr(self.reduce, "capturable", False):
+            raise RuntimeError("this tensor-parallel engine's all-reduce cannot be captured into a hipGraph (gloo / host-staged); "
+                               "decode eagerly (use_graph=False) or run the ranks over RCCL")
+        key = (float(temperature), int(top_k or 0), int(tokens))
+        if self._graph is not None and self._graph_key == key:
+            return self._graph
+        if self._graph is None:
+            self._graphs = {}
+        if key in self._graphs:
+            self._graph, self._graph_key = self._graphs[key], key
+            return self._graph
+        state = (self.tok_buf.clone(), self.pos_buf.clone(), self.rng_state.clone())
+        s = torch.cuda.Stream()
+        s.wait_stream(torch.cuda.current_stream())
+        with torch.cuda.stream(s):  # warm-up outside capture (KV rows it writes are rewritten by the real run)
+            self._self_step(temperature, top_k)
+        torch.cuda.current_stream().wait_stream(s)
+        self.tok_buf.copy_(state[0]); self.pos_buf.copy_(state[1]); self.rng_state.copy_(state[2])
+        g = torch.cuda.CUDAGraph()
+        try:
+            with runtime.graph_capture(g):
+                for _ in range(int(tokens)):
+                    self._self_step(temperature, top_k)
+        finally:  # (also when the capture fails — decode_n then decodes a sharded model eagerly from the same state)
+            self.tok_buf.copy_(state[0]); self.pos_buf.copy_(state[1]); self.rng_state.copy_(state[2])
+        self._graphs[key] = g
+        self._graph, self._graph_key = g, key
+        return g
+
+    @torch.no_grad()
+    def begin_sequence(self):
+        """a new sample: its own random stream (seed + running count of samples), draw counter 0"""
+        self._calls += 1
+        self.rng_state.copy_(torch.tensor([self._seed + self._calls, 0], dtype=torch.int64))
+
+    def sample_first(self, logits_row: torch.Tensor, temperature: float = 0.8, top_k: Optional[int] = 200) -> torch.Tensor:
+        """the token after the prompt, drawn by the fused sampler from the prompt pass's last-position logits (one launch where
+        the torch sampler of generate.sample takes ~10): opens the sample's random stream; follow with decode_n(..., drawn=1)"""
+        assert logits_row.is_contiguous() and logits_row.numel() == self.cfg.vocab_size and logits_row.dtype == self.dtype
+        self.begin_sequence()
+        return self.sample_fused(logits_row, temperature, top_k, feed=False)
+
+    def decode_n(self, first_token: torch.Tensor, pos: int, n: int, temperature: float = 0.8,
+                 top_k: Optional[int] = 200, use_graph: bool = True, drawn: int = 0) -> torch.Tensor:
+        """n decode steps starting from `first_token` at position `pos`; returns the n sampled tokens.  drawn: tokens already
+        drawn from this sample's random stream (sample_first: 1) — the loop continues it instead of opening a new one."""
+        assert n + drawn <= self.history.numel() and pos + n <= self.max_seq
+        self.tok_buf.copy_(first_token.view(1, 1))
+        self.pos_buf.fill_(pos)
+        if not drawn:
+            self.begin_sequence()
+        if use_graph and self.reduce is not None and not getattr(self.reduce, "capturable", False):
+            use_graph = False  # host-staged all-reduce (gloo): the step cannot live in a hipGraph
+        if use_graph and getattr(self, "tp_capture_error", None):
+            use_graph = False  # an earlier capture of this sharded step failed: stay eager
+        g = None
+        if use_graph:
+            try:
+                g = self.capture_loop(temperature, top_k)
+            except Exception as e:  # noqa: BLE001
+                # Under tensor parallelism the step holds two all-reduces per layer (RCCL, captured as graph nodes).  If this stack
+                # cannot capture them, degrade to eager decode and say why instead of aborting the run; an unsharded step holds
+                # only this library's launches — a capture failure there is a bug and propagates.
+                if self.reduce is None:
+                    raise
+                self.tp_capture_error = f"{type(e).__name__}: {e}"
+                print(f"teal_amd: hipGraph capture of the tensor-parallel decode step failed ({self.tp_capture_error}); decoding eagerly")
+                torch.cuda.synchronize()
+        if g is not None:
+            for _ in range(n):
+                g.replay()
+        else:
+            for _ in range(n):
+                self._self_step(temperature, top_k)
+        return self.history[drawn:drawn + n].clone()  # (the sampler files a token under its draw counter)
+
+    # nn.Module-ish surface so GraphedDecoder can drive either a Transformer or an engine
+    @property
+    def config(self):
+        return self.cfg
+
+    @property
+    def device(self):
+        return self.logits.device
+
+
+class DecodeEngine(DecodeLoop):
     """One-token decode of `model` at batch 1 through the fused HIP kernels.
 
     `thresholds[i]` = {"q","k","v","o","gate","up","down": tau} for layer i (what monkeypatch_layer
@@ -261,13 +389,7 @@ class DecodeEngine:
         self.n_wo = ctypes.c_int(0)
         self.n_down = ctypes.c_int(0)
         self.n_qkv = ctypes.c_int(0)
-        self.rng_state = torch.tensor([1234, 0], dtype=torch.int64, device=dev)  # {seed, draw counter}
-        self._seed, self._calls = 1234, 0
-        self.token = torch.zeros(1, dtype=torch.int32, device=dev)
-        self.tok_buf = torch.zeros(1, 1, dtype=torch.int32, device=dev)   # loop-carried token
-        self.pos_buf = torch.zeros(1, dtype=torch.int32, device=dev)      # loop-carried position
-        self.history = torch.zeros(max(8, model.max_seq_length), dtype=torch.int32, device=dev)
-        self._graph, self._graph_key, self._graphs = None, None, {}
+        self._init_loop(dev)
         self._build(thresholds)
 
     # ---- static launch descriptors (pointers never change: hipGraph-capture friendly) -------------
@@ -724,118 +846,6 @@ class DecodeEngine:
         self._walk(first_token, pos0, n_steps, n_samples, visit)
         return {p: sum(v) / len(v) for p, v in acc.items()}
 
-    def sample_fused(self, logits: torch.Tensor, temperature: float = 1.0, top_k: Optional[int] = None,
-                     feed: bool = False) -> torch.Tensor:
-        """One launch: top-k filter + softmax + exponential-race multinomial (generate.py:49-66).
-        feed=True also carries the loop state on the device: the token goes into the buffer the next
-        step reads, the position is advanced and the token is appended to `history`."""
-        tok_out = self.tok_buf if feed else self.token
-        rc = self.L.teal_sample_topk_ws(logits.data_ptr(), self.cfg.vocab_size, self.code, int(top_k or 0), float(temperature),
-                                        self.rng_state.data_ptr(), tok_out.data_ptr(),
-                                        self.pos_buf.data_ptr() if feed else None,
-                                        self.history.data_ptr() if feed else None, self.history.numel(),
-                                        self.ws.data_ptr(), self.ws.numel() * 4, runtime.stream_ptr())
-        if rc != 0:
-            _lib.check(rc, "teal_sample_topk")
-        return tok_out
-
-    def manual_seed(self, seed: int):
-        self._seed, self._calls = int(seed), 0
-        self.rng_state.copy_(torch.tensor([seed, 0], dtype=torch.int64))
-
-    # ---- device-resident decode loop: one hipGraph replay == one token, no host-side glue ---------
-    def _self_step(self, temperature, top_k):
-        logits = self(self.tok_buf, self.pos_buf)
-        self.sample_fused(logits, temperature, top_k, feed=True)
-
-    def capture_loop(self, temperature: float, top_k: Optional[int], tokens: int = 1):
-        """hipGraph of `tokens` consecutive decode steps (token, position and RNG counter stay on the device between them, so
-        a graph can span any number of tokens; each replay costs one host launch and one graph boundary on the GPU)."""
-        if self.reduce is not None and not getattr(self.reduce, "capturable", False):
-            raise RuntimeError("this tensor-parallel engine's all-reduce cannot be captured into a hipGraph (gloo / host-staged); "
-                               "decode eagerly (use_graph=False) or run the ranks over RCCL")
-        key = (float(temperature), int(top_k or 0), int(tokens))
-        if self._graph is not None and self._graph_key == key:
-            return self._graph
-        if self._graph is None:
-            self._graphs = {}
-        if key in self._graphs:
-            self._graph, self._graph_key = self._graphs[key], key
-            return self._graph
-        state = (self.tok_buf.clone(), self.pos_buf.clone(), self.rng_state.clone())
-        s = torch.cuda.Stream()
-        s.wait_stream(torch.cuda.current_stream())
-        with torch.cuda.stream(s):  # warm-up outside capture (KV rows it writes are rewritten by the real run)
-            self._self_step(temperature, top_k)
-        torch.cuda.current_stream().wait_stream(s)
-        self.tok_buf.copy_(state[0]); self.pos_buf.copy_(state[1]); self.rng_state.copy_(state[2])
-        g = torch.cuda.CUDAGraph()
-        try:
-            with runtime.graph_capture(g):
-                for _ in range(int(tokens)):
-                    self._self_step(temperature, top_k)
-        finally:  # (also when the capture fails — decode_n then decodes a sharded model eagerly from the same state)
-            self.tok_buf.copy_(state[0]); self.pos_buf.copy_(state[1]); self.rng_state.copy_(state[2])
-        self._graphs[key] = g
-        self._graph, self._graph_key = g, key
-        return g
-
-    @torch.no_grad()
-    def begin_sequence(self):
-        """a new sample: its own random stream (seed + running count of samples), draw counter 0"""
-        self._calls += 1
-        self.rng_state.copy_(torch.tensor([self._seed + self._calls, 0], dtype=torch.int64))
-
-    def sample_first(self, logits_row: torch.Tensor, temperature: float = 0.8, top_k: Optional[int] = 200) -> torch.Tensor:
-        """the token after the prompt, drawn by the fused sampler from the prompt pass's last-position logits (one launch where
-        the torch sampler of generate.sample takes ~10): opens the sample's random stream; follow with decode_n(..., drawn=1)"""
-        assert logits_row.is_contiguous() and logits_row.numel() == self.cfg.vocab_size and logits_row.dtype == self.dtype
-        self.begin_sequence()
-        return self.sample_fused(logits_row, temperature, top_k, feed=False)
-
-    def decode_n(self, first_token: torch.Tensor, pos: int, n: int, temperature: float = 0.8,
-                 top_k: Optional[int] = 200, use_graph: bool = True, drawn: int = 0) -> torch.Tensor:
-        """n decode steps starting from `first_token` at position `pos`; returns the n sampled tokens.  drawn: tokens already
-        drawn from this sample's random stream (sample_first: 1) — the loop continues it instead of opening a new one."""
-        assert n + drawn <= self.history.numel() and pos + n <= self.max_seq
-        self.tok_buf.copy_(first_token.view(1, 1))
-        self.pos_buf.fill_(pos)
-        if not drawn:
-            self.begin_sequence()
-        if use_graph and self.reduce is not None and not getattr(self.reduce, "capturable", False):
-            use_graph = False  # host-staged all-reduce (gloo): the step cannot live in a hipGraph
-        if use_graph and getattr(self, "tp_capture_error", None):
-            use_graph = False  # an earlier capture of this sharded step failed: stay eager
-        g = None
-        if use_graph:
-            try:
-                g = self.capture_loop(temperature, top_k)
-            except Exception as e:  # noqa: BLE001
-                # Under tensor parallelism the step holds two all-reduces per layer (RCCL, captured as graph nodes).  If this stack
-                # cannot capture them, degrade to eager decode and say why instead of aborting the run; an unsharded step holds
-                # only this library's launches — a capture failure there is a bug and propagates.
-                if self.reduce is None:
-                    raise
-                self.tp_capture_error = f"{type(e).__name__}: {e}"
-                print(f"teal_amd: hipGraph capture of the tensor-parallel decode step failed ({self.tp_capture_error}); decoding eagerly")
-                torch.cuda.synchronize()
-        if g is not None:
-            for _ in range(n):
-                g.replay()
-        else:
-            for _ in range(n):
-                self._self_step(temperature, top_k)
-        return self.history[drawn:drawn + n].clone()  # (the sampler files a token under its draw counter)
-
-    # nn.Module-ish surface so GraphedDecoder can drive either a Transformer or an engine
-    @property
-    def config(self):
-        return self.cfg
-
-    @property
-    def device(self):
-        return self.logits.device
-
 
 def make_engine_stepper(model: Transformer, a, ths: Optional[List[Dict[str, float]]] = None):
     """bench.py helper: thresholds (synthetic calibration) + prefill through the module path + the
@@ -913,7 +923,11 @@ def make_engine_stepper(model: Transformer, a, ths: Optional[List[Dict[str, floa
 
 
 def pick_engine(model: Transformer, need_caches: bool = True):
-    """(DecodeEngine, None) if the fused decode step can run `model` as it stands (16-bit, int8 or int4 group-quantised
-    projections), else (None, reason): the caller keeps the op-by-op module path."""
+    """(engine class, None) if a fused decode step can run `model` as it stands (DecodeEngine: 16-bit, int8 or int4 group-quantised
+    projections; layered designs: LayeredEngine), else (None, reason): the caller keeps the op-by-op path."""
+    if not isinstance(model, Transformer):
+        from .layered_engine import LayeredEngine
+        why = LayeredEngine.supports(model, need_caches)
+        return (LayeredEngine, None) if why is None else (None, why)
     why = DecodeEngine.supports(model, need_caches)
     return (DecodeEngine, None) if why is None else (None, why)

@@ -67,17 +67,6 @@ def sample(logits: torch.Tensor, temperature: float = 1.0, top_k: Optional[int] 
     return multinomial_sample_one_no_sync(probs), probs
 
 
-def sample_rows(logits: torch.Tensor, temperature: float = 1.0, top_k: Optional[int] = None) -> torch.Tensor:
-    """one token per row of logits [B, vocab]; temperature <= 0: the largest logit"""
-    if temperature <= 0:
-        return logits.argmax(dim=-1).to(torch.int)
-    logits = logits.float() / max(temperature, 1e-5)
-    if top_k is not None:
-        v, _ = torch.topk(logits, min(top_k, logits.size(-1)))
-        logits = torch.where(logits < v[:, -1:], -float("Inf"), logits)
-    return multinomial_sample_one_no_sync(torch.nn.functional.softmax(logits, dim=-1)).view(-1)
-
-
 # ------------------------------------------------------------------------------------------------
 # model construction
 # ------------------------------------------------------------------------------------------------
@@ -415,6 +404,8 @@ class EngineDecoder:
 
     def _cache_key(self):
         m = self.torch_model
+        if hasattr(m, "cache_key"):
+            return m.cache_key()
         return (m.max_seq_length,) + tuple(p for layer in m.layers for p in (layer.attention.kv_cache.k_cache.data_ptr(),
                                                                               layer.attention.kv_cache.v_cache.data_ptr()))
 
@@ -483,6 +474,83 @@ def generate(model: Transformer, prompt: torch.Tensor, max_new_tokens: int, deco
 
 
 # ------------------------------------------------------------------------------------------------
+def _prompt_ids(text: str) -> List[List[int]]:
+    """--prompt_ids "1,2,3;4,5": one list of token ids per request"""
+    return [[int(t) for t in part.replace(",", " ").split()] for part in text.split(";") if part.strip()]
+
+
+def main_layered(args, device: str) -> Dict:
+    """generate for a layered design (registry.py): one prompt decodes through generate() and, in 16 bits, the fused engine; several
+    prompts (--prompt_ids "..;..", --batch) or fp32 through serving.generate_batch."""
+    from teal_amd.gpt_fast import registry
+    from teal_amd.gpt_fast.layered_engine import KEEP_ALL, LayeredEngine, calibrate_thresholds
+    from teal_amd.gpt_fast.serving import Request, generate_batch
+    dtype = {"fp16": torch.float16, "bf16": torch.bfloat16, "fp32": torch.float32}[args.precision]
+    if args.hist_path is not None or args.greedy_lookup is not None:
+        raise SystemExit("--hist_path / --greedy_lookup describe Llama blocks; a layered design takes --sparsity (synthetic calibration)")
+    runtime.init()
+    t0 = time.time()
+    tokenizer = None
+    if args.synthetic:
+        model = registry.build_model(args.synthetic, device, dtype, n_layer=args.n_layer)
+    else:
+        model = registry.load_model(args.checkpoint_path, device, dtype)
+    if args.prompt_ids:
+        prompts = _prompt_ids(args.prompt_ids)
+    elif args.synthetic:
+        g = torch.Generator().manual_seed(7)
+        prompts = [torch.randint(0, model.config.vocab_size, (args.prompt_tokens,), generator=g).tolist() for _ in range(args.batch)]
+    else:
+        folder = args.checkpoint_path if args.checkpoint_path.is_dir() else args.checkpoint_path.parent
+        if not (folder / "tokenizer.model").is_file():
+            raise SystemExit(f"no tokenizer.model in {folder}: give token ids with --prompt_ids")
+        from teal_amd.gpt_fast.tokenizer import get_tokenizer
+        tokenizer = get_tokenizer(folder / "tokenizer.model", args.checkpoint_path)
+        prompts = [[tokenizer.bos_id()] + tokenizer.encode(args.prompt)] * args.batch
+    fused = len(prompts) == 1 and LayeredEngine.supports(model, need_caches=False) is None
+    thresholds = None
+    if args.sparsity > 0 and not args.dense:
+        if not fused:
+            raise SystemExit("--sparsity applies to the fused single-request step (one prompt, fp16 / bf16)")
+        thresholds = calibrate_thresholds(model, args.sparsity)
+    torch.cuda.synchronize()
+    print(f"Time to load model: {time.time() - t0:.02f} seconds")
+    torch.manual_seed(1234)
+    model_size = _get_model_size(model)
+    decoder = None
+    if fused:
+        decoder = EngineDecoder(model, thresholds or [dict.fromkeys(("q", "g", "kv", "o", "gate", "up", "down"), KEEP_ALL)] * len(model.layers),
+                                args.compile, args.temperature, args.top_k)
+    tps, seqs = [], []
+    for i in range(-1 if args.compile else 0, args.num_samples):
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        if fused:
+            prompt = torch.tensor(prompts[0], dtype=torch.int, device=device)
+            out = [generate(model, prompt, args.max_new_tokens, decoder, temperature=args.temperature, top_k=args.top_k).tolist()]
+        else:
+            new = generate_batch(model, [Request(p, args.max_new_tokens) for p in prompts], args.temperature, args.top_k, max_batch=args.max_batch,
+                                 seed=1234 + i * len(prompts), graphs=args.compile)
+            out = [list(p) + n for p, n in zip(prompts, new)]
+        torch.cuda.synchronize()
+        t = time.perf_counter() - t0
+        if i == -1:
+            print(f"Graph capture + warm-up time: {t:.2f} seconds")
+            continue
+        tps.append(args.max_new_tokens * len(prompts) / t)
+        seqs.extend(out)
+        for s in out:
+            print(tokenizer.decode(s) if tokenizer is not None else " ".join(map(str, s)))
+        print(f"Time for inference {i + 1}: {t:.02f} sec total, {tps[-1]:.02f} tokens/sec")
+        print(f"Bandwidth achieved: {model_size * tps[-1] / len(prompts) / 1e9:.02f} GB/s (dense parameter bytes x steps/s)")
+    print("==========")
+    mean = sum(tps) / max(1, len(tps))
+    print(f"Average tokens/sec: {mean:.2f}")
+    print(f"Memory used: {torch.cuda.max_memory_reserved() / 1e9:.02f} GB")
+    return {"tokens_per_sec": tps, "mean_tokens_per_sec": mean, "thresholds": thresholds, "decoder": type(decoder).__name__ if fused else "generate_batch",
+            "sequences": seqs, "prefill": None}
+
+
 def main(args) -> Dict:
     device = args.device
     assert "cuda" in device, "the sparse decode path is GPU-only (HIP kernels, no CPU fallback)"
@@ -491,6 +559,11 @@ def main(args) -> Dict:
                          "untested with TEAL); run without a draft model")
     if getattr(args, "interactive", False) and args.synthetic:
         raise SystemExit("--interactive needs a tokenizer (a checkpoint directory), not --synthetic")
+    from teal_amd.gpt_fast import layered
+    if layered.is_layered_name(args.synthetic) if args.synthetic else layered.is_layered_checkpoint(args.checkpoint_path):
+        return main_layered(args, args.device)
+    if args.precision == "fp32":
+        raise SystemExit("--precision fp32 runs the layered designs only")
     dtype = {"fp16": torch.float16, "bf16": torch.bfloat16}[args.precision]
     # tensor parallelism as in the reference (gpt-fast/generate.py:249-256, tp.py): one process per GPU under
     # torch.distributed.run; FIRST, so that every rank builds / loads its shard on its own device.  A single process (the
@@ -629,7 +702,12 @@ def build_parser() -> argparse.ArgumentParser:
     p.add_argument("--hist_path", type=str, default=None)
     p.add_argument("--sparsity", type=float, default=0.0)
     # extensions
-    p.add_argument("--precision", choices=["fp16", "bf16"], default="fp16")
+    p.add_argument("--precision", choices=["fp16", "bf16", "fp32"], default="fp16", help="fp32: layered designs only")
+    # layered designs (config.json + model.safetensors, or a name of layered.layered_configs)
+    p.add_argument("--prompt_ids", type=str, default=None, help='layered designs: token ids instead of --prompt, "1,2,3;4,5" = two requests')
+    p.add_argument("--prompt_tokens", type=int, default=6, help="layered designs, --synthetic: length of the random prompts")
+    p.add_argument("--batch", type=int, default=1, help="layered designs: requests to run together")
+    p.add_argument("--max_batch", type=int, default=64, help="layered designs: most requests in one step; the others wait")
     p.add_argument("--greedy_lookup", type=str, default=None, help="models/<name>/lookup directory (block-wise greedy sparsities)")
     p.add_argument("--synthetic", type=str, default=None, help="architecture name, e.g. 7B, llama-3-8b, 70B")
     p.add_argument("--n_layer", type=int, default=None, help="override the layer count (synthetic smoke runs)")

@@ -21,7 +21,6 @@ from typing import Any, Callable, Dict, List, Optional, Sequence
 import numpy as np
 import torch
 import torch.nn as nn
-import torch.nn.functional as F
 
 from ..kernels import layered as K
 from ..monkeypatch import to_column_major
@@ -301,7 +300,7 @@ class LatentAttention(nn.Module):
     def prompt(self, h: torch.Tensor, b: PromptBatch) -> torch.Tensor:
         a, pool = self.a, b.cache.pools[self.owner]
         own = a.kv_from is None
-        proj = F.linear(h, self.proj.weight)
+        proj = self.proj(h)
         K.latent_prompt_rows(proj, self.kv0 if own else -1, b.pos, b.row if own else None, self.inv_freq, self.kv_norm, self.eps, a.heads, a.dim, a.rot_dim,
                              a.kv_rank, pool if own else None)
         if own:
@@ -311,7 +310,7 @@ class LatentAttention(nn.Module):
         tile = K.latent_prompt_tile(a.dim, a.rot_dim, a.vdim, b.longest, h.dtype)
         y = K.latent_prompt_attention(proj, k, kr, vt, self.sink, self._gate(proj), self._y(b.n_tokens, h), b.seqs, b.tiles(tile), tile, a.heads, a.dim,
                                       a.rot_dim, a.vdim, self.window, a.scale)
-        return F.linear(y, self.wo.weight)
+        return self.wo(y)
 
     def splits(self, batch: int, max_pos: int, dtype: torch.dtype) -> int:
         """workgroups the cached rows of one sequence are split over: about one per CU, two 32-key tiles each at least"""
@@ -336,7 +335,7 @@ class LatentAttention(nn.Module):
         return K.latent_step_merge(part, splits, self.uv, self.sink, self._gate(proj), y, n, a.heads, a.kv_rank, a.vdim)
 
     def step(self, h: torch.Tensor, b: StepBatch) -> torch.Tensor:
-        return F.linear(self.attend(F.linear(h, self.proj.weight), b), self.wo.weight)
+        return self.wo(self.attend(self.proj(h), b))
 
     def linears(self):
         return [self.proj, self.wo]
@@ -373,7 +372,7 @@ class GatedMLP(nn.Module):
         return out
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
-        return F.linear(K.gated_act(F.linear(h, self.gate_up.weight), self.fp, self.fp, self.a.act, self.gate_up_bias), self.down.weight)
+        return self.down(K.gated_act(self.gate_up(h), self.fp, self.fp, self.a.act, self.gate_up_bias))
 
     def linears(self):
         return [self.gate_up, self.down]
@@ -480,6 +479,10 @@ class LayeredTransformer(nn.Module):
         self.cache.sync()
         self._slots = torch.arange(max_batch_size, dtype=torch.int32, device=self.tok_embeddings.weight.device)
 
+    def cache_key(self):
+        """what launch descriptors and captured graphs hold pointers to"""
+        return (self.max_seq_length, self.cache.version, id(self.cache))
+
     # ---- passes ----------------------------------------------------------------------------------------------------
     def _run(self, b, mixer, want: Optional[torch.Tensor], n_want: int, hook=None) -> Optional[torch.Tensor]:
         """embedding -> layers -> logits of the rows `want` (None: every row) of the batch b; mixer(layer, h) = its mixer's pass"""
@@ -501,7 +504,7 @@ class LayeredTransformer(nn.Module):
             return None
         if hook is not None and want is not None:
             h = h[want.long()]
-        return K.softcap(F.linear(h, self.output.weight), cfg.vocab_size, cfg.logit_softcap)
+        return K.softcap(self.output(h), cfg.vocab_size, cfg.logit_softcap)
 
     @torch.no_grad()
     def prompt_pass(self, b: PromptBatch, want: Sequence[int], hook=None) -> Optional[torch.Tensor]:

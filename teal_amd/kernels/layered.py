@@ -64,6 +64,16 @@ def softcap(logits, vocab: int, cap: Optional[float], out=None):
     return out
 
 
+def sample_rows(logits, rng, temperature: float, top_k: Optional[int], out=None, pos=None, history=None):
+    """one token per row of fp32 logits; rng int64 [rows, 2] {seed, draw counter}; temperature <= 0: the largest logit"""
+    assert logits.dtype == torch.float32 and rng.dtype == torch.int64 and rng.is_contiguous() and rng.numel() >= 2 * logits.shape[0]
+    if out is None:
+        out = torch.empty(logits.shape[0], dtype=torch.int32, device=logits.device)
+    _run("teal_sample_rows", _p(logits), _rows(logits), logits.shape[0], logits.shape[1], int(top_k or 0), float(temperature), _p(rng), _p(out), _p(pos), _p(history),
+         0 if history is None else history.shape[-1])
+    return out
+
+
 def latent_prompt_rows(proj, kv0, pos, row, inv_freq, norm_w, eps, heads, dim, rot, rank, pool):
     """rotate proj's queries in place; kv0 >= 0: write each token's cache row"""
     assert pos.dtype == torch.int32 and pos.numel() == proj.shape[0]

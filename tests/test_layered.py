@@ -1,0 +1,191 @@
+"""CPU: the layered designs' host side — configuration, checkpoint loading, the paged cache, the registry and the command line — and
+the plain restatement (oracle/layered_oracle.py) the GPU tests compare with: that the test models notice each mechanism."""
+import copy
+import json
+
+import numpy as np
+import pytest
+import torch
+
+from layered_models import CONFIGS, config, error, mixer, random_tensors, random_tokens, save_checkpoint
+from oracle import layered_oracle as O
+from teal_amd.gpt_fast import generate, layered, registry
+from teal_amd.gpt_fast.layered import LayeredArgs
+from teal_amd.gpt_fast.paged import PAGE, PagedCache
+
+FP32_TOL, BF16_TOL = 2e-5, 0.05  # what tests/test_layered_gpu.py allows
+
+
+# ---- the oracle ------------------------------------------------------------------------------------------------------
+def test_rotation_turns_adjacent_pairs_and_keeps_the_rest():
+    x = torch.randn(5, 2, 10, dtype=torch.float64)
+    pos = torch.tensor([0, 1, 7, 100, 3])
+    y = O.rotate_pairs(x, pos, 6, 50.0)
+    assert torch.equal(y[..., 6:], x[..., 6:]) and torch.equal(y[0], x[0])
+    z = torch.view_as_complex(x[..., :6].reshape(5, 2, 3, 2).contiguous())
+    f = 50.0 ** (-torch.arange(3, dtype=torch.float64) / 3)
+    want = torch.view_as_real(z * torch.exp(1j * pos[:, None, None] * f)).reshape(5, 2, 6)
+    assert torch.allclose(y[..., :6], want, atol=1e-12)
+    # a product of two rotated vectors depends on the distance alone
+    a, b = torch.randn(6, dtype=torch.float64), torch.randn(6, dtype=torch.float64)
+    dot = [O.rotate_pairs(a[None], torch.tensor([p]), 6, 50.0)[0] @ O.rotate_pairs(b[None], torch.tensor([p - 4]), 6, 50.0)[0] for p in (4, 90)]
+    assert abs(dot[0] - dot[1]) < 1e-10
+
+
+def test_window_and_sink_by_hand():
+    assert list(O.window_keys(9, 3)) == [7, 8, 9] and list(O.window_keys(1, 3)) == [0, 1] and list(O.window_keys(5, 1)) == [5]
+    assert list(O.window_keys(3, None)) == [0, 1, 2, 3]
+    w = O.softmax_with_sink(torch.tensor([0.0, np.log(3.0)], dtype=torch.float64), np.log(4.0))
+    assert torch.allclose(w, torch.tensor([1 / 8, 3 / 8], dtype=torch.float64))
+
+
+def _mutations(cfg, T):
+    """(name, changed configuration or tensor edit) a correct implementation must be told apart from"""
+    out = []
+    for i, ly in enumerate(cfg["layers"]):
+        for d in (-1, 1):
+            w = ly["mixer"]["mask"]["size"] + d
+            if 1 <= w < T:
+                c = copy.deepcopy(cfg)
+                c["layers"][i]["mixer"]["mask"]["size"] = w
+                out.append((f"window {d:+d} in layer {i}", c, None))
+        out.append((f"no sink in layer {i}", cfg, lambda t, i=i: t.update({f"l{i}.mix.sink": torch.full_like(t[f"l{i}.mix.sink"], -1e4)})))
+        if ly["mlp"]:
+            out.append((f"no down bias in layer {i}", cfg, lambda t, i=i: t[f"l{i}.mlp.down.b"].zero_()))
+    c = copy.deepcopy(cfg)
+    c["logit_softcap"] *= 1.02
+    out.append(("soft cap", c, None))
+    c = copy.deepcopy(cfg)
+    c["norm"]["eps"] *= 30
+    out.append(("eps", c, None))
+    return out
+
+
+@pytest.mark.parametrize("name", ["ragged", "even"])
+def test_the_models_of_the_gpu_tests_notice_every_mistake(name):
+    """each planted mistake (in the oracle) moves some position's logits by far more than the 32-bit comparison allows"""
+    cfg = CONFIGS[name]
+    t, T = random_tensors(cfg, 1), 90
+    toks = random_tokens(cfg, T, 2)
+    want = O.forward(cfg, t, toks)
+    for what, c, edit in _mutations(cfg, T):
+        tt = {k: v.clone() for k, v in t.items()}
+        if edit is not None:
+            edit(tt)
+        assert float(error(O.forward(c, tt, toks), want).max()) > 20 * FP32_TOL, what
+
+
+def test_oracle_positions_depend_on_earlier_tokens_only():
+    cfg = CONFIGS["ragged"]
+    t, toks = random_tensors(cfg, 3), random_tokens(cfg, 40, 4)
+    assert torch.allclose(O.forward(cfg, t, toks)[:25], O.forward(cfg, t, toks[:25]), atol=1e-10)
+
+
+# ---- configuration and loading ----------------------------------------------------------------------------------------
+def test_config_is_read_per_layer(tmp_path):
+    cfg = CONFIGS["ragged"]
+    a = LayeredArgs.from_dict(json.loads(json.dumps(cfg)))
+    assert (a.vocab_size, a.dim, a.norm_eps, a.logit_softcap, a.n_layer) == (101, 72, 3e-3, 7.0, 5)
+    m = [ly.mixer for ly in a.layers]
+    assert [x.window for x in m] == [33, 7, 70, 64, 1] and [x.kv_from for x in m] == [None, 0, None, 0, 2]
+    assert [ly.mlp.ff if ly.mlp else None for ly in a.layers] == [52, None, 30, 90, 41]
+    assert m[2].scale == 0.4 and m[2].rope_base == 500.0
+
+
+@pytest.mark.parametrize("edit,what", [
+    (lambda c: c.update(architecture="Nobody"), "no layered design"),
+    (lambda c: c["layers"][0].update(type="mamba"), "unknown mixer"),
+    (lambda c: c["layers"][0].update(mlp={"kind": "moe", "ff": 8}), "unknown feed-forward"),
+    (lambda c: c["layers"][1]["mixer"].update(kv_from=1), "kv_from"),
+    (lambda c: c["layers"][3]["mixer"].update(kv_from=1), "kv_from"),
+    (lambda c: c["layers"][3]["mixer"].update(kv_rank=37), "latent size"),
+    (lambda c: c["layers"][0]["mixer"]["rot"].update(dims=4), "rotates all"),
+])
+def test_config_errors_name_the_fault(edit, what):
+    c = copy.deepcopy(CONFIGS["ragged"])
+    edit(c)
+    with pytest.raises((KeyError, ValueError), match=what):
+        LayeredArgs.from_dict(c)
+
+
+def test_checkpoint_loads_into_padded_images(tmp_path):
+    cfg = CONFIGS["ragged"]
+    t = random_tensors(cfg, 5)
+    path = save_checkpoint(tmp_path / "m", cfg, t)
+    assert layered.is_layered_checkpoint(path) and layered.is_layered_checkpoint(path / "model.safetensors")
+    model = registry.load_model(path, "cpu", torch.bfloat16)
+    assert set(model.tensor_shapes()) == set(t) and all(tuple(t[k].shape) == s for k, s in model.tensor_shapes().items())
+    for i, b in enumerate(model.layers):
+        mx = b.mix
+        assert torch.equal(mx.proj.weight[: mx.nq], t[f"l{i}.mix.q"]) and torch.equal(mx.proj.weight[mx.g0:mx.g0 + mx.nv], t[f"l{i}.mix.g"])
+        assert not mx.proj.weight[mx.nq:mx.g0].any() and mx.proj.weight.stride(0) == 1 and mx.proj.out_features % 64 == 0
+        assert torch.equal(mx.wo.weight[:, : mx.nv], t[f"l{i}.mix.o"]) and not mx.wo.weight[:, mx.nv:].any()
+        if mx.a.kv_from is None:
+            assert torch.equal(mx.proj.weight[mx.kv0:mx.kv0 + mx.nkv], t[f"l{i}.mix.dkv"])
+    assert torch.equal(model.output.weight[:101], t["embed"]) and not model.output.weight[101:].any()
+    bad = dict(t, embed=t["embed"][:50])
+    with pytest.raises(ValueError, match="embed"):
+        registry.load_model(save_checkpoint(tmp_path / "bad", cfg, bad), "cpu", torch.bfloat16)
+
+
+def test_registry_and_named_configs():
+    assert layered.is_layered_name("Bolizen-tiny-test") and not layered.is_layered_name("7B")
+    m = registry.build_model("Bolizen-tiny-test", "cpu", torch.float32)
+    assert m.config.n_layer == 4 and [ly.mixer.kv_from for ly in m.config.layers] == [None, 0, None, 2]
+    assert registry.build_model("Bolizen-tiny-test", "cpu", torch.float32, n_layer=1).config.n_layer == 1
+    assert registry.build_model("tiny-test", "cpu", torch.float32).config.dim == 256  # the Llama names still build
+
+
+def test_command_line_knows_the_layered_options(tmp_path):
+    a = generate.build_parser().parse_args(["--checkpoint_path", str(tmp_path), "--prompt_ids", "1,2,3;4 5", "--precision", "fp32"])
+    assert generate._prompt_ids(a.prompt_ids) == [[1, 2, 3], [4, 5]] and a.precision == "fp32"
+    (tmp_path / "config.json").write_text(json.dumps({"architecture": "Other"}))
+    with pytest.raises(ValueError, match="Other"):
+        registry.load_model(tmp_path, "cpu", torch.float32)
+
+
+# ---- the paged cache --------------------------------------------------------------------------------------------------
+def test_pages_grow_trim_and_come_back():
+    c = PagedCache({0: 32, 3: 64}, torch.float32, "cpu", max_tokens=2 * PAGE, max_requests=2, window=PAGE)
+    a = c.open()
+    c.extend(a, 1)
+    assert c.pages_in_use == 1 and c.pools[0].shape == (c.n_pages * PAGE, 32) and c.pools[3].shape[1] == 64
+    c.extend(a, PAGE + 1)
+    assert c.pages_in_use == 2
+    c.trim(a)  # position PAGE + 1 sees positions 2 .. PAGE + 1: nothing to give back
+    assert c.pages_in_use == 2
+    c.extend(a, 2 * PAGE - 1)
+    c.trim(a)  # the next position, 2 PAGE - 1, sees PAGE .. : the first page is out of every window
+    assert c.pages_in_use == 1 and c.slots[a][0] == -1
+    first = c.host[a, 1]
+    b = c.open()
+    c.extend(b, 3 * PAGE)  # more than was asked for: the pools grow, nothing that is in use moves
+    assert c.host[a, 1] == first and len({*c.slots[b], first}) == 4
+    assert c.rows(b, np.array([0, PAGE, 2 * PAGE + 5])).tolist() == [c.host[b, 0] * PAGE, c.host[b, 1] * PAGE, c.host[b, 2] * PAGE + 5]
+    c.sync()
+    assert torch.equal(c.table, torch.from_numpy(c.host))
+    c.close(a)
+    c.close(b)
+    assert c.pages_in_use == 0 and sorted(c.free) == list(range(c.n_pages)) and c.open() == a
+
+
+def test_cache_contents_survive_growth():
+    c = PagedCache({0: 32}, torch.float32, "cpu", max_tokens=PAGE, max_requests=1)
+    s = c.open()
+    c.extend(s, PAGE)
+    rows = torch.from_numpy(c.rows(s, np.arange(PAGE))).long()
+    c.pools[0][rows] = torch.arange(PAGE, dtype=torch.float32)[:, None].expand(-1, 32)
+    v = c.version
+    c.extend(s, 20 * PAGE)
+    s2 = [c.open() for _ in range(3)]
+    assert c.version > v and len({s, *s2}) == 4
+    assert torch.equal(c.pools[0][torch.from_numpy(c.rows(s, np.arange(PAGE))).long()][:, 0], torch.arange(PAGE, dtype=torch.float32))
+
+
+def test_one_layer_without_a_window_keeps_every_page():
+    cfg = config(64, 32, [(mixer(1, 8, 4, 8, 16, 8), 16), (mixer(1, 8, 4, 8, 16, 8), None)])
+    del cfg["layers"][1]["mixer"]["mask"]
+    m = layered.build_layered_model(LayeredArgs.from_dict(cfg), "cpu", torch.float32)
+    assert m.new_cache(100).window is None
+    cfg["layers"][1]["mixer"]["mask"] = {"size": 9}
+    assert layered.build_layered_model(LayeredArgs.from_dict(cfg), "cpu", torch.float32).new_cache(100).window == 9

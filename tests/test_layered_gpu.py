@@ -1,0 +1,480 @@
+"""GPU: the layered designs against the plain restatement (oracle/layered_oracle.py, float64): whole prompts, token by token, portions,
+unequal batches, reused pages, the fused step and its graphs, sampling, the scheduler, the command line and the trace replay.
+
+32-bit models are held to 2e-5 of the logits' rms per position, which tells every mechanism apart (tests/test_layered.py plants
+mistakes in the oracle); 16-bit models to their rounding."""
+import copy
+import json
+import os
+import subprocess
+import sys
+
+import numpy as np
+import pytest
+import torch
+
+from layered_models import CONFIGS, error, random_tensors, random_tokens, save_checkpoint
+from oracle import layered_oracle as O
+
+pytestmark = pytest.mark.gpu
+DEV = "cuda"
+F32, BF16, F16 = torch.float32, torch.bfloat16, torch.float16
+TOL = {F32: 2e-5, BF16: 0.06, F16: 0.01}
+
+
+def close(e, dtype):
+    """per-position errors within the format's tolerance; in 16 bits a query whose two best keys nearly tie may stand out by rounding
+    alone, so there one position in ten may exceed it, six-fold at most (a wrong key is an error of order 1)"""
+    if dtype == F32:
+        return float(e.max()) < TOL[dtype]
+    return float(e.max()) < 6 * TOL[dtype] and int((e > TOL[dtype]).sum()) <= max(1, len(e) // 10)
+
+
+_cache = {}
+
+
+def setup(name, dtype, tmp_path_factory):
+    """(config, tensors, model on the GPU, {(T, seed): (tokens, oracle logits)}) — built once per session"""
+    from teal_amd import runtime
+    from teal_amd.gpt_fast import registry
+    runtime.init()
+    key = (name, dtype)
+    if key not in _cache:
+        cfg = CONFIGS[name]
+        t = random_tensors(cfg, 1)
+        path = save_checkpoint(tmp_path_factory.mktemp(name), cfg, t)
+        _cache[key] = (cfg, t, registry.load_model(path, DEV, dtype))
+    return _cache[key]
+
+
+def expected(name, cfg, t, n, seed):
+    key = ("want", name, n, seed)
+    if key not in _cache:
+        toks = random_tokens(cfg, n, seed)
+        _cache[key] = (toks, O.forward(cfg, t, toks))
+    return _cache[key]
+
+
+def poison(eng):
+    """NaN in every cache row no live sequence has written: nothing may read it"""
+    used = np.zeros(eng.cache.n_pages * 64, dtype=bool)
+    for s, pages in enumerate(eng.cache.slots):
+        if pages is not None:
+            pos = np.arange(eng.cache.lengths[s])
+            pos = pos[np.asarray([pages[p >> 6] >= 0 for p in pos], dtype=bool)] if len(pos) else pos
+            used[eng.cache.rows(s, pos)] = True
+    rows = torch.from_numpy(np.nonzero(~used)[0]).to(DEV)
+    for layer, pool in eng.cache.pools.items():
+        pool[rows] = float("nan")
+
+
+def engine(model, **kw):
+    from teal_amd.gpt_fast.serving import BatchEngine
+    return BatchEngine(model, **{"max_tokens": 256, "max_requests": 2, **kw})
+
+
+ALL = [(n, d) for n in CONFIGS for d in (F32, BF16)] + [("even", F16), ("heads", F16)]
+
+
+# ---- row kernels -------------------------------------------------------------------------------------------------------
+@pytest.mark.parametrize("dtype", [F32, BF16, F16])
+@pytest.mark.parametrize("D", [64, 70, 2048, 5120])
+def test_residual_norm_rows(dtype, D):
+    from teal_amd.kernels import layered as K
+    T, V, eps = 9, 40, 1e-3
+    r = lambda *s: torch.randn(*s, device=DEV)  # noqa: E731
+    emb, y, bias = r(V, D).to(dtype), (3 * r(T, D)).to(dtype), r(D).to(dtype)
+    post, pre = (1 + 0.2 * r(D)).to(dtype), (1 + 0.2 * r(D)).to(dtype)
+    tok = torch.randint(0, V, (T,), device=DEV, dtype=torch.int32)
+    x = torch.full((T, D), float("nan"), device=DEV)
+    h = K.resid_norm(x, tokens=tok, embed=emb, pre_w=pre, eps=eps)
+    assert torch.equal(x, emb[tok.long()].float())
+    ref = O.rms_norm(x.double(), pre.double(), eps)
+    tol = 1e-5 if dtype == F32 else 2 ** -8 if dtype == BF16 else 2 ** -10
+    assert h.dtype == dtype and ((h.double() - ref).abs() <= tol * (1 + ref.abs())).all()
+    want = x.double() + O.rms_norm(y.double() + bias.double(), post.double(), eps)
+    x2 = x.clone()
+    h = K.resid_norm(x2, y=y, y_bias=bias, post_w=post, pre_w=pre, eps=eps)
+    assert (x2.double() - want).abs().max() < 1e-5
+    ref = O.rms_norm(want, pre.double(), eps)
+    assert ((h.double() - ref).abs() <= tol * (1 + ref.abs())).all()
+    x3, rows = x.clone(), torch.tensor([7, 0, 3], device=DEV, dtype=torch.int32)  # a subset, packed; the other rows stay
+    h3 = K.resid_norm(x3, y=y, y_bias=bias, post_w=post, pre_w=pre, eps=eps, rows=rows)
+    assert torch.equal(h3, h[rows.long()]) and torch.equal(x3[1], x[1]) and torch.equal(x3[7], x2[7])
+    x4 = x.clone()
+    assert K.resid_norm(x4, y=y, dtype=dtype) is None and torch.allclose(x4, x + y.float(), atol=1e-6)  # no norms: a plain add
+
+
+@pytest.mark.parametrize("dtype", [F32, BF16])
+@pytest.mark.parametrize("n,up0", [(128, 128), (77, 90), (4104, 4104)])
+def test_gated_activation_and_soft_cap(dtype, n, up0):
+    from teal_amd.kernels import layered as K
+    gu, b = (2 * torch.randn(5, up0 + n, device=DEV)).to(dtype), torch.randn(up0 + n, device=DEV).to(dtype)
+    g, u = gu[:, :n].double(), gu[:, up0:up0 + n].double()
+    tol = 1e-5 if dtype == F32 else 2 ** -7
+    for act, f in (("gelu_tanh", O.gelu_tanh), ("silu", torch.nn.functional.silu)):
+        ref = f(g + b[:n].double()) * (u + b[up0:up0 + n].double())
+        assert ((K.gated_act(gu, n, up0, act, b).double() - ref).abs() <= tol * (1 + ref.abs())).all()
+        ref = f(g) * u
+        assert ((K.gated_act(gu, n, up0, act).double() - ref).abs() <= tol * (1 + ref.abs())).all()
+    z = (9 * torch.randn(3, n + 8, device=DEV)).to(dtype)
+    assert torch.allclose(K.softcap(z, n, 5.0).double(), 5 * torch.tanh(z[:, :n].double() / 5), atol=1e-5)
+    assert torch.equal(K.softcap(z, n, None), z[:, :n].float())
+
+
+@pytest.mark.parametrize("V", [33, 1000, 32000, 128256])
+def test_sampler_rows(V):
+    from teal_amd.kernels import layered as K
+    B = 4
+    x = 3 * torch.randn(B, V + 3, device=DEV)[:, :V]
+    x[1] = x[1].round()               # ties everywhere
+    x[2] *= 1e-3                      # a flat row
+    x[3, : V // 2] = -50.0
+    rng = torch.tensor([[11 + i, 0] for i in range(B)], device=DEV)
+    pos, hist = torch.zeros(B, dtype=torch.int32, device=DEV), torch.full((B, 6), -1, dtype=torch.int32, device=DEV)
+    assert torch.equal(K.sample_rows(x, rng.clone(), 0.0, None).long(), x.argmax(-1))
+    for k in (1, 2, 7, min(200, V - 1), V):
+        kth = x.topk(k, -1).values[:, -1:]
+        allowed = x >= kth
+        for rep in range(6):
+            t = K.sample_rows(x, rng, 1.5, k, pos=pos, history=hist).long()
+            assert allowed.gather(1, t[:, None]).all(), (V, k)
+    assert (pos == 30).all() and (rng[:, 1] == 30).all() and (hist >= 0).all()
+    # the frequencies of a small distribution
+    p = torch.tensor([[0.5, 0.25, 0.15, 0.1]], device=DEV)
+    rng = torch.tensor([[5, 0]], device=DEV)
+    n = torch.zeros(4)
+    for _ in range(1500):
+        n[int(K.sample_rows(p.log() * 0.7, rng, 0.7, None))] += 1
+    assert (n / 1500 - p[0].cpu()).abs().max() < 0.05
+
+
+# ---- the mixer alone: one key stands out ----------------------------------------------------------------------------------
+@pytest.mark.parametrize("dtype", [F32, BF16])
+@pytest.mark.parametrize("window", [1, 2, 63, 64, 65, 96, 300])
+def test_a_key_at_the_windows_edge(dtype, window):
+    """Query p asks for the key of position j with a score far above all others, j just inside and just outside the window, at page
+    borders and at the start: the answer is j's value inside, anything else's outside.  In the prompt pass and in the step."""
+    from teal_amd import runtime
+    from teal_amd.gpt_fast.layered import LayeredArgs, LayeredTransformer, PromptBatch, StepBatch, _empty
+    from layered_models import config, mixer
+    runtime.init()
+    H, D, R, V, rank, T, W = 2, 16, 8, 16, 64, 200, 64
+    cfg = config(W, 16, [(mixer(H, D, R, V, rank, window, scale=1.0), None)])
+    t = random_tensors(cfg, 9)
+    t["l0.mix.sink"] = torch.tensor([-1.0, 2.0]).to(torch.bfloat16)
+    model = _empty(LayeredArgs.from_dict(cfg), DEV, dtype)
+    model.load_tensors(lambda n: t[n].to(DEV, dtype))
+    mix = model.layers[0].mix
+    Wd = {k: v.double() for k, v in t.items()}
+    h = torch.randn(T, W, dtype=torch.float64).to(torch.bfloat16).double()
+    a = cfg["layers"][0]["mixer"]
+    # the input of query p is built so that W_uk^T W_q h has a large component along j's latent (a least-squares preimage)
+    pairs = [(p, p - d) for p in (40, 63, 64, 65, 127, 128, 130, 199) for d in (0, window - 1, window, window // 2) if p - d >= 0]
+    pairs += [(window - 1, 0), (window, 0)] if window < T else [(150, 0)]
+    h = h.clone()
+    seen = set()
+    plan = []
+    for p, j in pairs:
+        if p in seen or p == j:
+            continue
+        seen.add(p)
+        plan.append((p, j))
+    targets = {j for _, j in plan}
+    plan = [(p, j) for p, j in plan if p not in targets]  # (a target's own input stays as it is)
+    c, kr = O.latents(h, Wd, "l0.mix", a, cfg["norm"]["eps"])
+    M = torch.cat([Wd["l0.mix.uk"][n * D:(n + 1) * D].T @ Wd["l0.mix.q"].view(H, D + R, W)[n, :D] for n in range(H)])  # [H rank, W]
+    for p, j in plan:
+        h[p] = (torch.linalg.lstsq(M, torch.cat([c[j]] * H)[:, None]).solution[:, 0] * 3).to(torch.bfloat16).double()
+    c, kr = O.latents(h, Wd, "l0.mix", a, cfg["norm"]["eps"])
+    want = O.latent_attention(h, c, kr, Wd, "l0.mix", a)
+    wide = O.latent_attention(h, c, kr, Wd, "l0.mix", dict(a, mask={"size": window + 1}))
+    moved = (wide - want).norm(dim=-1) / want.norm(dim=-1)
+    if window < T - 1:
+        assert float(moved.max()) > 0.5  # a window one token wider answers otherwise somewhere
+    tol = 5e-5 if dtype == F32 else 0.1
+    cache = model.new_cache(T, 1)
+    s = cache.open()
+    cache.extend(s, T)
+    cache.sync()
+    hd = h.to(DEV, dtype)
+    got = mix.prompt(hd, PromptBatch(cache, [(s, 0, [0] * T)], DEV))
+    rel = lambda g, w: ((g.double().cpu() - w).norm(dim=-1) / want.norm(dim=-1).mean()).max()  # noqa: E731
+    assert float(rel(got, want)) < tol
+    for pool in cache.pools.values():
+        pool.zero_()
+    out = []
+    for p in range(T):
+        b = StepBatch(cache, torch.zeros(1, dtype=torch.int32, device=DEV), torch.tensor([p], dtype=torch.int32, device=DEV),
+                      torch.tensor([s], dtype=torch.int32, device=DEV), p)
+        out.append(mix.step(hd[p:p + 1], b))
+    assert float(rel(torch.cat(out), want)) < tol
+
+
+def test_no_window_and_no_sink(tmp_path_factory):
+    """the mixer's options: attention over everything before a position, and a softmax without a sink"""
+    from teal_amd.gpt_fast.layered import LayeredArgs, _empty
+    from layered_models import config, mixer
+    cfg = config(64, 50, [(mixer(2, 16, 8, 16, 32, 0), 64)])
+    del cfg["layers"][0]["mixer"]["mask"]
+    t = random_tensors(cfg, 4)
+    toks = random_tokens(cfg, 150, 1)
+    for sink in (True, False):
+        args = LayeredArgs.from_dict(cfg)
+        args.layers[0].mixer.sink = sink
+        model = _empty(args, DEV, F32).load_tensors(lambda n: t[n].to(DEV, F32))
+        tt = t if sink else dict(t, **{"l0.mix.sink": torch.full_like(t["l0.mix.sink"], -1e4)})
+        want = O.forward(cfg, tt, toks)
+        eng = engine(model)
+        assert float(error(eng.step([(0, toks[:90], range(90))]), want[:90]).max()) < TOL[F32]
+        for p in range(90, 150):
+            assert float(error(eng.step([(0, toks[p:p + 1], [0])]), want[p:p + 1]).max()) < TOL[F32] * 3
+
+
+# ---- whole models ---------------------------------------------------------------------------------------------------------
+@pytest.mark.parametrize("name,dtype", ALL)
+def test_whole_prompts(name, dtype, tmp_path_factory):
+    cfg, t, model = setup(name, dtype, tmp_path_factory)
+    eng = engine(model)
+    for n, seed in ((1, 1), (2, 1), (33, 2), (160, 3)):
+        toks, want = expected(name, cfg, t, n, seed)
+        poison(eng)
+        e = error(eng.step([(n, toks, range(n))]), want)
+        assert close(e, dtype), (n, int(e.argmax()), float(e.max()))
+        eng.release(n)
+
+
+@pytest.mark.parametrize("name,dtype", ALL)
+def test_token_by_token_equals_the_prompt(name, dtype, tmp_path_factory):
+    """decoding from the second token on, through several pages and windows, over poisoned memory"""
+    cfg, t, model = setup(name, dtype, tmp_path_factory)
+    toks, want = expected(name, cfg, t, 160, 3)
+    eng = engine(model)
+    got = [eng.step([("a", toks[:1], [0])])]
+    for p in range(1, 160):
+        poison(eng)
+        got.append(eng.step([("a", toks[p:p + 1], [0])]))
+    e = error(torch.cat(got), want)
+    assert close(e, dtype), (int(e.argmax()), float(e.max()))
+    assert eng.cache.pages_in_use <= 1 + -(-max(ly["mixer"]["mask"]["size"] for ly in cfg["layers"]) // 64)
+
+
+@pytest.mark.parametrize("name,dtype", [("ragged", F32), ("even", F32), ("even", BF16), ("heads", BF16)])
+@pytest.mark.parametrize("sizes", [[2], [3, 1], [7, 64], [65, 31], [100, 1, 1, 2]])
+def test_portions_of_a_prompt(name, dtype, sizes, tmp_path_factory):
+    cfg, t, model = setup(name, dtype, tmp_path_factory)
+    toks, want = expected(name, cfg, t, 160, 3)
+    eng, got, at, k = engine(model), [], 0, 0
+    while at < 160:
+        n = min(sizes[k % len(sizes)], 160 - at)
+        poison(eng)
+        got.append(eng.step([("a", toks[at:at + n], range(n))]))
+        at, k = at + n, k + 1
+    assert close(error(torch.cat(got), want), dtype)
+
+
+@pytest.mark.parametrize("name,dtype", [("ragged", F32), ("even", F32), ("even", BF16), ("heads", BF16), ("large", BF16)])
+def test_unequal_batch_and_reused_pages(name, dtype, tmp_path_factory):
+    """requests of different lengths start together, decode together and end one after the other; later requests get their slots and
+    pages; a portion and a running request share a step.  Everything equals each request alone."""
+    cfg, t, model = setup(name, dtype, tmp_path_factory)
+    toks, want = expected(name, cfg, t, 160, 3)
+    other, want2 = expected(name, cfg, t, 33, 2)
+    eng = engine(model, max_tokens=64, max_requests=1)  # (the cache has to grow on the way)
+    check = lambda got, w: close(error(got, w), dtype)  # noqa: E731
+    start = {"a": 1, "b": 33, "c": 64, "d": 100}
+    for rnd in range(2):
+        poison(eng)
+        got = eng.step([(r, toks[:n], [0, n - 1] if n > 1 else [0]) for r, n in start.items()])
+        rows = [i for n in start.values() for i in ([0, n - 1] if n > 1 else [0])]
+        assert check(got, want[rows])
+        live = dict(start)
+        for k in range(40):
+            poison(eng)
+            got = eng.step([(r, toks[p:p + 1], [0]) for r, p in live.items()])
+            assert check(got, want[list(live.values())]), (rnd, k)
+            live = {r: p + 1 for r, p in live.items()}
+            if k % 12 == 11:
+                eng.release(next(iter(live)))
+                live.pop(next(iter(live)))
+        eng.step([("e", other[:20], []), *[(r, toks[p:p + 1], []) for r, p in live.items()]])  # a prompt next to running requests
+        live = {r: p + 1 for r, p in live.items()}
+        poison(eng)
+        got = eng.step([("e", other[20:], [12]), *[(r, toks[p:p + 1], [0]) for r, p in live.items()]])
+        assert check(got, torch.cat([want2[32:33], want[list(live.values())]]))
+        for r in ["e", *live]:
+            eng.release(r)
+        assert eng.cache.pages_in_use == 0
+
+
+def test_bad_steps_are_refused(tmp_path_factory):
+    cfg, t, model = setup("even", F32, tmp_path_factory)
+    eng = engine(model)
+    for entries in ([("a", [], [])], [("a", [256], [])], [("a", [-1], [])], [("a", [1], [1])], [("a", [1], []), ("a", [2], [])]):
+        with pytest.raises(ValueError):
+            eng.step(entries)
+    assert not eng.slot and eng.cache.pages_in_use == 0
+    assert eng.step([("a", [1, 2], [])]) is None and eng.length("a") == 2
+
+
+# ---- the fused step --------------------------------------------------------------------------------------------------------
+@pytest.mark.parametrize("name,dtype", [("even", BF16), ("even", F16), ("heads", BF16), ("large", BF16)])
+def test_fused_step_equals_the_unfused_one(name, dtype, tmp_path_factory):
+    from teal_amd.gpt_fast.layered import StepBatch
+    from teal_amd.gpt_fast.layered_engine import LayeredEngine
+    cfg, t, model = setup(name, dtype, tmp_path_factory)
+    assert LayeredEngine.supports(model, need_caches=False) is None
+    toks, want = expected(name, cfg, t, 160, 3)
+    eng = engine(model)
+    assert eng.fused is not None
+    eng.step([("a", toks[:70], [])])
+    pairs = []
+    for p in range(70, 160):
+        s = eng.slot["a"]
+        eng.cache.extend(s, p + 1)
+        eng.cache.sync()
+        dev = torch.tensor([[toks[p]], [p], [s]], dtype=torch.int32, device=DEV)
+        plain = model.step_pass(StepBatch(eng.cache, dev[0], dev[1], dev[2], p)).clone()
+        fused = eng._decode(dev, p)
+        pairs.append((error(fused, want[p:p + 1]), error(fused, plain.double().cpu())))
+    assert all(close(torch.cat(e), dtype) for e in zip(*pairs))
+
+
+def test_fused_step_needs_whole_chunks(tmp_path_factory):
+    from teal_amd.gpt_fast.engine import pick_engine
+    cfg, t, model = setup("ragged", BF16, tmp_path_factory)  # 72 wide: no fused form, the engine keeps the unfused step
+    cls, why = pick_engine(model, need_caches=False)
+    assert cls is None and "width" in why and engine(model).fused is None
+
+
+@pytest.mark.parametrize("name,dtype,batch", [("even", BF16, 1), ("heads", BF16, 1), ("even", BF16, 3), ("ragged", F32, 2)])
+def test_graph_replays_equal_eager_steps(name, dtype, batch, tmp_path_factory):
+    cfg, t, model = setup(name, dtype, tmp_path_factory)
+    toks, _ = expected(name, cfg, t, 160, 3)
+    a, b = engine(model, max_requests=4, max_tokens=1024), engine(model, max_requests=4, max_tokens=1024, graphs=True)
+    for e in (a, b):
+        e.step([(r, toks[: 50 + r], []) for r in range(batch)])
+    for k in range(60):
+        step = [(r, [toks[50 + r + k]], [0]) for r in range(batch)]
+        x, y = a.step(step), b.step(step)
+        torch.cuda.synchronize()
+        assert float(error(y, x.double().cpu()).max()) < (1e-5 if dtype == F32 else TOL[dtype] / 4), k
+    assert b._graphs
+
+
+def test_sparsity_masks_the_projections(tmp_path_factory):
+    """thresholds of the fused step = the unfused step on masked activations"""
+    from teal_amd.gpt_fast.layered import StepBatch
+    from teal_amd.gpt_fast.layered_engine import LayeredEngine, calibrate_thresholds
+    cfg, t, model = setup("even", BF16, tmp_path_factory)
+    ths = calibrate_thresholds(model, 0.4)
+    toks = random_tokens(cfg, 60, 8)
+    eng = engine(model)
+    eng.step([("a", toks[:40], [])])
+    s = eng.slot["a"]
+    eng.cache.extend(s, 41)
+    eng.cache.sync()
+    dev = torch.tensor([[toks[40]], [40], [s]], dtype=torch.int32, device=DEV)
+    fused = LayeredEngine(model, ths, cache=eng.cache, max_seq=64)
+    fused.slot = dev[2]
+    got = fused(dev[0], dev[1]).view(1, -1).clone()
+    hooks, kept = [], []
+
+    def mask(lin, tau):
+        def pre(_m, args):
+            keep = args[0].float().abs() > tau
+            kept.append(float(keep.float().mean()))
+            return (args[0] * keep,)
+        hooks.append(lin.register_forward_pre_hook(pre))
+
+    for b, th in zip(model.layers, ths):
+        mask(b.mix.proj, th["q"]), mask(b.mix.wo, th["o"]), mask(b.mlp.gate_up, th["gate"]), mask(b.mlp.down, th["down"])
+    plain = model.step_pass(StepBatch(eng.cache, dev[0], dev[1], dev[2], 40)).clone()
+    for h in hooks:
+        h.remove()
+    dense = model.step_pass(StepBatch(eng.cache, dev[0], dev[1], dev[2], 40))
+    assert 0.4 < sum(kept) / len(kept) < 0.8
+    assert float(error(got, plain.double().cpu())) < 0.12 < float(error(dense, plain.double().cpu()))
+
+
+# ---- generation ------------------------------------------------------------------------------------------------------------
+def greedy(cfg, t, prompt, n):
+    seq = list(prompt)
+    for _ in range(n):
+        seq.append(int(O.forward(cfg, t, seq)[-1].argmax()))
+    return seq[len(prompt):]
+
+
+def test_greedy_generation_equals_the_oracle(tmp_path_factory):
+    """32-bit: more requests than run at once, of unequal lengths, whole prompts and portions, eager and from graphs"""
+    from teal_amd.gpt_fast.serving import Request, generate_batch
+    cfg, t, model = setup("even", F32, tmp_path_factory)
+    reqs = [(random_tokens(cfg, n, 20 + n), m) for n, m in ((1, 9), (30, 6), (66, 8), (5, 1), (12, 10))]
+    want = [greedy(cfg, t, p, m) for p, m in reqs]
+    for kw in ({}, {"max_batch": 2}, {"portion": 7}, {"max_batch": 3, "graphs": False}):
+        assert generate_batch(model, [Request(p, m) for p, m in reqs], **kw) == want, kw
+    # sampling: a request's stream depends on its own seed alone
+    r = [Request(p, m) for p, m in reqs]
+    alone = [generate_batch(model, r[i:i + 1], temperature=1.0, top_k=20, seed=50 + i)[0] for i in range(5)]
+    assert generate_batch(model, r, temperature=1.0, top_k=20, seed=50) == alone
+
+
+def test_generate_entry_point_and_command_line(tmp_path_factory):
+    """generate() with the fused engine (bf16: every chosen token is within rounding of the oracle's best) and the CLI's main"""
+    from teal_amd.gpt_fast import generate as G
+    cfg, t, model = setup("even", BF16, tmp_path_factory)
+    path = save_checkpoint(tmp_path_factory.mktemp("cli"), cfg, t)
+    prompt = random_tokens(cfg, 20, 3)
+    base = ["--checkpoint_path", str(path), "--num_samples", "1", "--max_new_tokens", "70", "--temperature", "0", "--compile"]
+    run = lambda *a: G.main(G.build_parser().parse_args([*base, *a]))  # noqa: E731
+    res = run("--precision", "bf16", "--prompt_ids", ",".join(map(str, prompt)))
+    seq = res["sequences"][0]
+    assert res["decoder"] == "EngineDecoder" and seq[:20] == prompt and len(seq) == 90
+    lg = O.forward(cfg, t, seq)
+    gap = (lg.max(-1).values - lg.gather(1, torch.tensor(seq[1:] + [0])[:, None])[:, 0])[19:-1]
+    assert float(gap.max()) < 3 * TOL[BF16] * float(lg.pow(2).mean().sqrt())
+    res = run("--precision", "fp32", "--prompt_ids", "1,2,3;" + " ".join(map(str, prompt)), "--max_new_tokens", "5")
+    assert [s[-5:] for s in res["sequences"]] == [greedy(cfg, t, [1, 2, 3], 5), greedy(cfg, t, prompt, 5)]
+    res = G.main(G.build_parser().parse_args(["--synthetic", "Bolizen-tiny-test", "--precision", "bf16", "--num_samples", "2", "--max_new_tokens", "12", "--compile",
+                                              "--sparsity", "0.3"]))
+    assert len(res["sequences"]) == 2 and res["thresholds"] is not None
+    with pytest.raises(SystemExit):
+        G.main(G.build_parser().parse_args(["--synthetic", "7B", "--precision", "fp32"]))
+
+
+def test_module_contract(tmp_path_factory):
+    """forward(idx, input_pos) as model.Transformer's: prompt of a batch, then a captured single-token step"""
+    from teal_amd.gpt_fast.generate import GraphedDecoder
+    cfg, t, model = setup("even", F32, tmp_path_factory)
+    toks, want = expected("even", cfg, t, 160, 3)
+    model.setup_caches(2, 170)
+    idx = torch.tensor([toks[:50], toks[:50]], device=DEV)
+    lg = model(idx, torch.arange(50, device=DEV))
+    assert lg.shape == (2, 50, 256) and float(error(lg[1], want[:50]).max()) < TOL[F32]
+    dec = GraphedDecoder(model, True, 0.0, None)
+    cur, pos = torch.tensor([[toks[50]]], device=DEV, dtype=torch.int), torch.tensor([50], device=DEV, dtype=torch.int)
+    dec.capture(cur, pos)
+    for p in range(50, 90):
+        got = dec(torch.tensor([[toks[p]]], device=DEV, dtype=torch.int), torch.tensor([p], device=DEV, dtype=torch.int))
+        assert int(got) == int(want[p].argmax()), p
+    model.max_seq_length = model.max_batch_size = -1
+
+
+@pytest.mark.parametrize("dtype", ["bfloat16", "float32"])
+def test_trace_replay(dtype, tmp_path, tmp_path_factory):
+    cfg, t, model = setup("even", F32, tmp_path_factory)
+    toks, want = expected("even", cfg, t, 160, 3)
+    path = save_checkpoint(tmp_path / "m", cfg, t)
+    steps = [{"step": 0, "entries": [{"id": "x", "tokens": toks[:40], "want": [0, 39]}, {"id": "y", "tokens": toks[:1], "want": []}], "end": []},
+             {"step": 1, "entries": [{"id": "x", "tokens": toks[40:41], "want": [0]}, {"id": "y", "tokens": toks[1:2], "want": [0]}], "end": ["y"]},
+             {"step": 2, "entries": [{"id": "x", "tokens": toks[41:42], "want": []}], "end": []},
+             {"step": 3, "entries": [{"id": "x", "tokens": toks[42:43], "want": [0]}], "end": ["x"]}]
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    r = subprocess.run([os.path.join(root, "bin", "trace_run"), "--model", str(path), "--dtype", dtype, "--out", str(tmp_path), "--max-tokens", "64"],
+                       input="".join(json.dumps(s) + "\n" for s in steps), text=True, capture_output=True, timeout=100)
+    assert r.returncode == 0, r.stderr[-2000:]
+    assert [ln for ln in r.stdout.splitlines() if ln.startswith("done")] == [f"done {i}" for i in range(4)]
+    read = lambda i: torch.from_numpy(np.fromfile(tmp_path / f"{i}.f32", dtype="<f4").reshape(-1, 256))  # noqa: E731
+    tol = TOL[getattr(torch, dtype)]
+    assert float(error(read(0), want[[0, 39]]).max()) < tol and float(error(read(1), want[[40, 1]]).max()) < tol
+    assert float(error(read(3), want[[42]]).max()) < tol and not (tmp_path / "2.f32").exists()
