@@ -436,7 +436,8 @@ int teal_latent_step_query(const void* proj, int ldp, int kv0, int batch, const 
                            const float* inv_freq, const void* norm_w, float eps, const void* uk, int heads, int dim, int rot, int rank, void* cache, int ldc, void* qcat,
                            int ldq, int dtype, void* stream);
 /* ... partial attention over the cached rows of the window, split over `splits` workgroups per 16 heads:
- * part fp32 [batch][heads][splits][rank + 2] = {max of the scaled scores in log2 units, sum, weighted latent} */
+ * part fp32 [batch][heads][splits][R4 + 4], R4 = rank rounded up to 4: {weighted latent [R4], max of the scaled scores in log2
+ * units, sum, -, -} */
 int teal_latent_step_attention(const void* qcat, int ldq, const void* cache, int ldc, const int32_t* pos, const int32_t* slot, const int32_t* table, int max_pages,
                                int page_shift, int batch, int heads, int rank, int rot, int window, float scale, int splits, float* part, size_t part_bytes, int dtype,
                                void* stream);

@@ -93,7 +93,6 @@ struct Config {
 struct DeviceCtx {
     int num_cu;       // 0: not initialised yet
     bool gqa_lds_ok;  // the grouped-query attention kernel may take kGqaMaxLds of LDS on this device
-    bool latent_lds_ok;  // ... and the absorbed latent attention kernel kLatentMaxLds (teal_latent.hip)
 };
 DeviceCtx* device_ctx();                   // context of the CURRENT device (nullptr: no device)
 inline int num_cu_or(int dflt) {           // CU count of the current device, or dflt without a device (host-only queries)
@@ -101,7 +100,6 @@ inline int num_cu_or(int dflt) {           // CU count of the current device, or
     return c && c->num_cu > 0 ? c->num_cu : dflt;
 }
 bool attention_device_init();              // teal_attention.hip: per-kernel attributes of the current device
-bool latent_device_init();                 // teal_latent.hip: the same
 // teal_fused_gemv over int4 group-quantised weights (out->weight_bits == 4): teal_gemv_int4.hip
 int fused_gemv_i4(const teal_gemv_in_t* in, const teal_gemv_out_t* out, int Z, int dtype, void* ws, size_t ws_bytes,
                   int* nslabs_out, hipStream_t st);

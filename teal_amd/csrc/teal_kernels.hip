@@ -154,7 +154,6 @@ DeviceCtx* device_ctx() {
         return nullptr;
     }
     c->gqa_lds_ok = attention_device_init();
-    c->latent_lds_ok = latent_device_init();
     c->num_cu = cu;
     return c;
 }

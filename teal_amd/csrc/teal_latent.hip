@@ -21,11 +21,30 @@ namespace teal {
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef _Float16 f16x8 __attribute__((ext_vector_type(8)));
 constexpr float kLog2e = 1.4426950408889634f;
+constexpr int kStepKSteps = 20;  // 32-wide inner-dimension steps of the absorbed score product: cached rows of up to 640 elements
 
 template <bool BF16>
 __device__ __forceinline__ f32x4 mfma16(const u32x4 a, const u32x4 b, const f32x4 c) {
     if constexpr (BF16) return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
     else return __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(f16x8, a), __builtin_bit_cast(f16x8, b), c, 0, 0, 0);
+}
+
+// 2^x of a non-positive x (v_exp_f32: one ulp; results below the normal range are zero)
+__device__ __forceinline__ float exp2_fast(const float x) { return __builtin_amdgcn_exp2f(x); }
+
+// two values as packed high and low 16-bit halves
+template <bool BF16>
+__device__ __forceinline__ void split16x2(const float a, const float b, uint32_t& hi, uint32_t& lo) {
+    if constexpr (BF16) {
+        typedef float f32v2 __attribute__((ext_vector_type(2)));
+        typedef __bf16 bf16v2 __attribute__((ext_vector_type(2)));
+        hi = __builtin_bit_cast(uint32_t, __builtin_convertvector((f32v2{a, b}), bf16v2));
+        lo = __builtin_bit_cast(uint32_t, __builtin_convertvector((f32v2{a - __uint_as_float(hi << 16), b - __uint_as_float(hi & 0xFFFF0000u)}), bf16v2));
+    } else {
+        const uint32_t h0 = float_to_bits<false>(a), h1 = float_to_bits<false>(b);
+        hi = h0 | (h1 << 16);
+        lo = (uint32_t)float_to_bits<false>(a - bits_to_float(h0, false)) | ((uint32_t)float_to_bits<false>(b - bits_to_float(h1, false)) << 16);
+    }
 }
 
 // v as a high and a low 16-bit half
@@ -177,31 +196,52 @@ __global__ __launch_bounds__(256) void latent_prompt_attention_kernel(const Late
     const int last = sq.start + min(q_first + BM, sq.nq) - 1;           // position of the tile's last query
     const int first = max(sq.klo, sq.start + q_first - a.window + 1);   // first position any of its queries sees
     const float sc = a.scale * kLog2e;
-    for (int kt = (first - sq.klo) / BN * BN; sq.klo + kt <= last; kt += BN) {
-        __syncthreads();
-        for (int i = tid; i < BN * (DQP / 8); i += 256) {
-            const int key = i / (DQP / 8), d0 = (i % (DQP / 8)) * 8;
+    // the next tile's keys and values are requested while a tile is worked on
+    constexpr int CK = DQP / 8, CV = BN / 8, NK = (BN * CK + 255) / 256, NV = (DVP * CV + 255) / 256;
+    u32x4 kreg[NK], vreg[NV];
+    auto fetch = [&](const int kt) {
+#pragma unroll
+        for (int i = 0; i < NK; ++i) {
+            const int at = tid + 256 * i, key = at / CK, d0 = (at % CK) * 8;
             const size_t row = (size_t)min(sq.k0 + kt + key, a.S - 1);
-            u32x4 w = {0u, 0u, 0u, 0u};
+            kreg[i] = u32x4{0u, 0u, 0u, 0u};
             if (kvec) {
-                if (d0 < a.dim) w = *reinterpret_cast<const u32x4*>(kp + (row * a.heads + head) * a.dim + d0);
-                else if (d0 < dq) w = *reinterpret_cast<const u32x4*>(krp + row * a.rot + d0 - a.dim);
+                const uint16_t* src = d0 < a.dim ? kp + (row * a.heads + head) * a.dim + d0 : krp + row * a.rot + d0 - a.dim;
+                if (d0 < dq) kreg[i] = *reinterpret_cast<const u32x4*>(src);
             } else {
 #pragma unroll
                 for (int j = 0; j < 8; ++j) {
                     const int d = d0 + j;
-                    if (d < dq) w[j >> 1] |= (uint32_t)(d < a.dim ? kp[(row * a.heads + head) * a.dim + d] : krp[row * a.rot + d - a.dim]) << (16 * (j & 1));
+                    if (d < dq) kreg[i][j >> 1] |= (uint32_t)(d < a.dim ? kp[(row * a.heads + head) * a.dim + d] : krp[row * a.rot + d - a.dim]) << (16 * (j & 1));
                 }
             }
-            *reinterpret_cast<u32x4*>(ks + key * LK + d0) = w;
         }
-        for (int i = tid; i < DVP * (BN / 8); i += 256) {  // (S and every sequence's key base are multiples of 8: 16-byte loads)
-            const int v = i / (BN / 8), c0 = (i % (BN / 8)) * 8;
-            u32x4 w = {0u, 0u, 0u, 0u};
-            if (v < a.vdim && sq.k0 + kt + c0 < a.S) w = *reinterpret_cast<const u32x4*>(vp + (size_t)v * a.S + sq.k0 + kt + c0);
-            *reinterpret_cast<u32x4*>(vs + v * LV + c0) = w;
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {  // (S and every sequence's key base are multiples of 8: 16-byte loads)
+            const int at = tid + 256 * i, v = at / CV, c0 = (at % CV) * 8;
+            vreg[i] = u32x4{0u, 0u, 0u, 0u};
+            if (v < a.vdim && sq.k0 + kt + c0 < a.S) vreg[i] = *reinterpret_cast<const u32x4*>(vp + (size_t)v * a.S + sq.k0 + kt + c0);
+        }
+    };
+    static_assert((BN * CK) % 256 == 0 && (DVP * CV) % 256 == 0, "whole staging rounds");
+    const int wq0 = sq.start + q_first + wave * NQ * 16;  // the wave's first query position
+    const bool whole = q_first + (wave + 1) * NQ * 16 <= sq.nq;
+    int kt = (first - sq.klo) / BN * BN;
+    fetch(kt);
+    for (; sq.klo + kt <= last; kt += BN) {
+        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < NK; ++i) {
+            const int at = tid + 256 * i;
+            *reinterpret_cast<u32x4*>(ks + (at / CK) * LK + (at % CK) * 8) = kreg[i];
+        }
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int at = tid + 256 * i;
+            *reinterpret_cast<u32x4*>(vs + (at / CV) * LV + (at % CV) * 8) = vreg[i];
         }
         __syncthreads();
+        if (sq.klo + kt + BN <= last) fetch(kt + BN);
         f32x4 s[NQ][KT];
 #pragma unroll
         for (int t = 0; t < KT; ++t) {
@@ -214,7 +254,10 @@ __global__ __launch_bounds__(256) void latent_prompt_attention_kernel(const Late
                 for (int n = 0; n < NQ; ++n) s[n][t] = mfma16<BF16>(kf, qf[n][q], s[n][t]);
             }
         }
-        u32x4 ph[NQ][BN / 32], pl[NQ][BN / 32];
+        const int k_first = sq.klo + kt;
+        // every query of the wave sees every key of the tile: no masks
+        const bool open = whole && k_first + BN - 1 <= wq0 && k_first > wq0 + NQ * 16 - 1 - a.window;
+        float ms[NQ];
 #pragma unroll
         for (int n = 0; n < NQ; ++n) {
             float mx = m[n];
@@ -222,35 +265,37 @@ __global__ __launch_bounds__(256) void latent_prompt_attention_kernel(const Late
             for (int t = 0; t < KT; ++t)
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
-                    const int kpos = sq.klo + kt + t * 16 + g * 4 + r;
-                    const bool ok = kpos <= qpos[n] && kpos > qpos[n] - a.window;
-                    s[n][t][r] = ok ? s[n][t][r] * sc : -INFINITY;
-                    mx = fmaxf(mx, s[n][t][r]);
+                    float v = s[n][t][r] * sc;
+                    if (!open) {
+                        const int kpos = k_first + t * 16 + g * 4 + r;
+                        v = kpos <= qpos[n] && kpos > qpos[n] - a.window ? v : -INFINITY;
+                    }
+                    s[n][t][r] = v;
+                    mx = fmaxf(mx, v);
                 }
             mx = fmaxf(mx, __shfl_xor(mx, 16));
             mx = fmaxf(mx, __shfl_xor(mx, 32));
-            const float ms = mx == -INFINITY ? 0.0f : mx;
-            const float al = exp2f(m[n] - ms);
+            ms[n] = mx == -INFINITY ? 0.0f : mx;
+            const float al = exp2_fast(m[n] - ms[n]);
             m[n] = mx;
-            float ls = 0.0f;
-#pragma unroll
-            for (int b = 0; b < BN / 32; ++b)
-#pragma unroll
-                for (int j = 0; j < 4; ++j) {  // word j of the operand: keys 2j, 2j + 1 of the lane's eight (tile 2b, then tile 2b + 1)
-                    const float p0 = exp2f(s[n][2 * b + (j >> 1)][2 * (j & 1)] - ms), p1 = exp2f(s[n][2 * b + (j >> 1)][2 * (j & 1) + 1] - ms);
-                    uint32_t h0, l0, h1, l1;
-                    split16<BF16>(p0, h0, l0);
-                    split16<BF16>(p1, h1, l1);
-                    ph[n][b][j] = h0 | (h1 << 16);
-                    pl[n][b][j] = l0 | (l1 << 16);
-                    ls += p0 + p1;
-                }
-            l[n] = l[n] * al + ls;
+            l[n] *= al;
 #pragma unroll
             for (int v = 0; v < VT; ++v) o[n][v] *= al;
         }
 #pragma unroll
-        for (int b = 0; b < BN / 32; ++b)
+        for (int b = 0; b < BN / 32; ++b) {
+            u32x4 ph[NQ], pl[NQ];
+#pragma unroll
+            for (int n = 0; n < NQ; ++n)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {  // word j of the operand: keys 2j, 2j + 1 of the lane's eight (tile 2b, then tile 2b + 1)
+                    const float p0 = exp2_fast(s[n][2 * b + (j >> 1)][2 * (j & 1)] - ms[n]), p1 = exp2_fast(s[n][2 * b + (j >> 1)][2 * (j & 1) + 1] - ms[n]);
+                    uint32_t hi, lo;
+                    split16x2<BF16>(p0, p1, hi, lo);
+                    ph[n][j] = hi;
+                    pl[n][j] = lo;
+                    l[n] += p0 + p1;
+                }
 #pragma unroll
             for (int v = 0; v < VT; ++v) {
                 const uint16_t* base = vs + (v * 16 + l16) * LV + b * 32 + g * 4;
@@ -258,10 +303,11 @@ __global__ __launch_bounds__(256) void latent_prompt_attention_kernel(const Late
                 const u32x4 vf = {w0[0], w0[1], w1[0], w1[1]};
 #pragma unroll
                 for (int n = 0; n < NQ; ++n) {
-                    o[n][v] = mfma16<BF16>(vf, ph[n][b], o[n][v]);
-                    o[n][v] = mfma16<BF16>(vf, pl[n][b], o[n][v]);
+                    o[n][v] = mfma16<BF16>(vf, ph[n], o[n][v]);
+                    o[n][v] = mfma16<BF16>(vf, pl[n], o[n][v]);
                 }
             }
+        }
     }
 #pragma unroll
     for (int n = 0; n < NQ; ++n) {
@@ -364,8 +410,8 @@ __global__ __launch_bounds__(256) void latent_prompt_attention_scalar_kernel(con
 }
 
 // ------------------------------------------------------------------------------------------------
-// Single tokens, part 1: grid (heads * chunks [+ 1], batch).  Workgroup (head, chunk): 128 columns of the absorbed query
-// W_uk,head^T q (chunk 0 also rotates the query's rotated part); the extra workgroup: the token's cache row.
+// Single tokens, part 1: grid (heads * chunks [+ 1], batch / BT).  Workgroup (head, chunk): 128 columns of the absorbed query
+// W_uk,head^T q of BT tokens (chunk 0 also rotates the query's rotated part); the extra workgroup: the tokens' cache rows.
 // qcat [batch][heads][ldq]: q_abs (rank), rotated part (rot), zeros up to ldq — one fp32 row, or a high and a low 16-bit row.
 // ------------------------------------------------------------------------------------------------
 struct LatentStepArgs {
@@ -377,72 +423,109 @@ struct LatentStepArgs {
     int max_pages, shift, chunks, ldq;
 };
 
-template <int DT>
-__global__ __launch_bounds__(256) void latent_step_query_kernel(const LatentStepArgs a) {
+template <int DT, int BT>
+__global__ __launch_bounds__(256) void latent_step_query_kernel(const LatentStepArgs a, const int batch) {
     using N = Num<DT>;
     using S = typename N::S;
     extern __shared__ __align__(16) unsigned char smem[];
-    float* q = reinterpret_cast<float*>(smem);  // [dim]
+    float* q = reinterpret_cast<float*>(smem);  // [BT][dim]
     __shared__ float red[4], part[16][129];
     const LatentRowArgs& k = a.kv;
-    const int tid = threadIdx.x, b = blockIdx.y, p = k.pos[b];
-    const S* proj = reinterpret_cast<const S*>(k.proj) + (size_t)b * k.ldp;
+    const int tid = threadIdx.x, b0 = blockIdx.y * BT, nb = min(BT, batch - b0);
+    const S* proj = reinterpret_cast<const S*>(k.proj) + (size_t)b0 * k.ldp;
     if ((int)blockIdx.x == k.heads * a.chunks) {
-        const int row = page_row(a.table + (size_t)a.slot[b] * a.max_pages, min(p, (a.max_pages << a.shift) - 1), a.shift);
-        latent_row<DT>(k, proj + k.kv0, p, reinterpret_cast<S*>(k.cache) + (size_t)row * k.ldc, red, tid);
+        for (int i = 0; i < nb; ++i) {
+            const int p = k.pos[b0 + i];
+            const int row = page_row(a.table + (size_t)a.slot[b0 + i] * a.max_pages, min(p, (a.max_pages << a.shift) - 1), a.shift);
+            latent_row<DT>(k, proj + (size_t)i * k.ldp + k.kv0, p, reinterpret_cast<S*>(k.cache) + (size_t)row * k.ldc, red, tid);
+        }
         return;
     }
     const int head = blockIdx.x / a.chunks, r0 = (blockIdx.x % a.chunks) * 128;
     const S* qh = proj + head * (k.dim + k.rot);
-    for (int i = tid; i < k.dim; i += 256) q[i] = N::ld(qh + i);
-    __syncthreads();
     const int c0 = (tid & 15) * 8, dg = tid >> 4;
     const S* w = reinterpret_cast<const S*>(a.uk) + (size_t)head * k.dim * k.rank + r0 + c0;
-    float acc[8];
+    float acc[BT][8];
 #pragma unroll
-    for (int j = 0; j < 8; ++j) acc[j] = 0.0f;
+    for (int t = 0; t < BT; ++t)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) acc[t][j] = 0.0f;
     const int left = k.rank - r0 - c0;
-    if (left >= 8) {
-        const bool vec = !(k.rank & 7);
-#pragma unroll 4
-        for (int d = dg; d < k.dim; d += 16) {
-            float v[8];
-            ld8<DT>(w + (size_t)d * k.rank, v, vec);
+    const bool vec = !(k.rank & 7);
+    constexpr int U = DT == TEAL_F32 ? 4 : 8;  // weight rows in flight; the first ones leave before the query has arrived
+    Raw8<DT> v[U];
+    auto rows = [&](const int d0) {
 #pragma unroll
-            for (int j = 0; j < 8; ++j) acc[j] = fmaf(q[d], v[j], acc[j]);
+        for (int u = 0; u < U; ++u) v[u].load(w + (size_t)min(d0 + 16 * u, k.dim - 1) * k.rank, vec);
+    };
+    if (left >= 8) rows(dg);
+    for (int i = tid; i < BT * k.dim; i += 256) {
+        const int t = BT == 1 ? 0 : i / k.dim, d = i - t * k.dim;
+        q[i] = t < nb ? N::ld(qh + (size_t)t * k.ldp + d) : 0.0f;
+    }
+    __syncthreads();
+    if (left >= 8) {
+        for (int d0 = dg; d0 < k.dim; d0 += 16 * U) {
+            if (d0 != dg) rows(d0);
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const int d = min(d0 + 16 * u, k.dim - 1);
+                float x[BT];
+#pragma unroll
+                for (int t = 0; t < BT; ++t) x[t] = d0 + 16 * u < k.dim ? q[t * k.dim + d] : 0.0f;
+#pragma unroll
+                for (int j = 0; j < 8; ++j) {
+                    const float wj = v[u].get(j);
+#pragma unroll
+                    for (int t = 0; t < BT; ++t) acc[t][j] = fmaf(x[t], wj, acc[t][j]);
+                }
+            }
         }
     } else if (left > 0) {
         for (int d = dg; d < k.dim; d += 16)
-            for (int j = 0; j < left; ++j) acc[j] = fmaf(q[d], N::ld(w + (size_t)d * k.rank + j), acc[j]);
+#pragma unroll
+            for (int j = 0; j < 8; ++j)
+                if (j < left) {
+                    const float wj = N::ld(w + (size_t)d * k.rank + j);
+#pragma unroll
+                    for (int t = 0; t < BT; ++t) acc[t][j] = fmaf(q[t * k.dim + d], wj, acc[t][j]);
+                }
     }
 #pragma unroll
-    for (int j = 0; j < 8; ++j) part[dg][c0 + j] = acc[j];
-    __syncthreads();
-    auto put = [&](const int i, const float v) {  // element i of this head's row
-        const size_t at = (size_t)b * k.heads + head;
-        if constexpr (DT == TEAL_F32) {
-            reinterpret_cast<float*>(a.qcat)[at * a.ldq + i] = v;
-        } else {
-            uint32_t hi, lo;
-            split16<DT == TEAL_BF16>(v, hi, lo);
-            reinterpret_cast<uint16_t*>(a.qcat)[at * 2 * a.ldq + i] = (uint16_t)hi;
-            reinterpret_cast<uint16_t*>(a.qcat)[(at * 2 + 1) * a.ldq + i] = (uint16_t)lo;
-        }
-    };
-    if (tid < 128 && r0 + tid < k.rank) {
-        float t = 0.0f;
+    for (int t = 0; t < BT; ++t) {
+        if (t >= nb) break;
+        auto put = [&](const int i, const float x) {  // element i of this head's row
+            const size_t at = (size_t)(b0 + t) * k.heads + head;
+            if constexpr (DT == TEAL_F32) {
+                reinterpret_cast<float*>(a.qcat)[at * a.ldq + i] = x;
+            } else {
+                uint32_t hi, lo;
+                split16<DT == TEAL_BF16>(x, hi, lo);
+                reinterpret_cast<uint16_t*>(a.qcat)[at * 2 * a.ldq + i] = (uint16_t)hi;
+                reinterpret_cast<uint16_t*>(a.qcat)[(at * 2 + 1) * a.ldq + i] = (uint16_t)lo;
+            }
+        };
+        if (t) __syncthreads();
 #pragma unroll
-        for (int i = 0; i < 16; ++i) t += part[i][tid];
-        put(r0 + tid, t);
-    }
-    if (r0 == 0) {
-        for (int i = tid; i < k.rot / 2; i += 256) {
-            float x, y;
-            rotate_pair(N::ld(qh + k.dim + 2 * i), N::ld(qh + k.dim + 2 * i + 1), p, k.inv_freq[i], x, y);
-            put(k.rank + 2 * i, x);
-            put(k.rank + 2 * i + 1, y);
+        for (int j = 0; j < 8; ++j) part[dg][c0 + j] = acc[t][j];
+        __syncthreads();
+        if (tid < 128 && r0 + tid < k.rank) {
+            float x = 0.0f;
+#pragma unroll
+            for (int i = 0; i < 16; ++i) x += part[i][tid];
+            put(r0 + tid, x);
         }
-        for (int i = k.rank + k.rot + tid; i < a.ldq; i += 256) put(i, 0.0f);
+        if (r0 == 0) {
+            const S* qr = qh + (size_t)t * k.ldp + k.dim;
+            const int p = k.pos[b0 + t];
+            for (int i = tid; i < k.rot / 2; i += 256) {
+                float x, y;
+                rotate_pair(N::ld(qr + 2 * i), N::ld(qr + 2 * i + 1), p, k.inv_freq[i], x, y);
+                put(k.rank + 2 * i, x);
+                put(k.rank + 2 * i + 1, y);
+            }
+            for (int i = k.rank + k.rot + tid; i < a.ldq; i += 256) put(i, 0.0f);
+        }
     }
 }
 
@@ -451,8 +534,10 @@ __global__ __launch_bounds__(256) void latent_step_query_kernel(const LatentStep
 // 32-key tiles of the window.  Per tile: the waves share the score product by its inner dimension (both 16-key tiles, K steps
 // wave, wave + 4, ...; partial scores through LDS), then each wave owns a quarter of the latent's columns in the value product.
 // The tile's rows are staged transposed ([column][key]) for that product; the score product's operand comes straight from memory.
-// part [batch][heads][splits][rank + 2] = {max (log2 units), sum, weighted latent}.
+// part [batch][heads][splits][part_stride(rank)] = {weighted latent (rank, padded to 4), max (log2 units), sum, -, -}.
 // ------------------------------------------------------------------------------------------------
+__host__ __device__ constexpr int part_stride(const int rank) { return ((rank + 3) & ~3) + 4; }
+
 struct LatentDecodeArgs {
     const void* qcat;
     const void* cache;
@@ -479,70 +564,96 @@ __device__ __forceinline__ KeyRange split_range(const int p, const int window, c
 
 template <bool BF16, int RT>
 __global__ __launch_bounds__(256) void latent_decode_attention_kernel(const LatentDecodeArgs a) {
-    constexpr int RPW = RT / 4, LT = 36;  // 16-column tiles per wave; row stride (keys) of the transposed tile
-    extern __shared__ __align__(16) unsigned char smem[];
-    const int LQ = a.ldq + 8;
-    uint16_t* qs = reinterpret_cast<uint16_t*>(smem);          // [2][16][LQ] high, low
-    uint16_t* ct = qs + 2 * 16 * LQ;                           // [RT * 16][LT]
-    float* sp = reinterpret_cast<float*>(ct + RT * 16 * LT);   // [4][2][64][4] partial scores (lane-major)
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, g = lane >> 4;
+    constexpr int RPW = RT / 4, LT = 36;    // 16-column tiles per wave; row stride (keys) of the transposed tile
+    constexpr int KSW = kStepKSteps / 4, NI = (RT + 7) / 8;  // inner-dimension steps per wave; staging rounds
+    __shared__ __align__(16) uint16_t ct[RT * 16 * LT];
+    __shared__ __align__(16) float sp[4 * 2 * 64 * 4];       // partial scores, lane-major
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), l16 = lane & 15, g = lane >> 4;
     const int split = blockIdx.x, h0 = blockIdx.y * 16, b = blockIdx.z;
     const int nh = min(16, a.heads - h0);
-    const int p = a.pos[b];
+    const int p = min(a.pos[b], (a.max_pages << a.shift) - 1);  // (a position past the table would read past it)
     const int* table = a.table + (size_t)a.slot[b] * a.max_pages;
-    const int plast = (a.max_pages << a.shift) - 1;  // (a position past the table would read past it: clamp)
-    const KeyRange kr = split_range(min(p, plast), a.window, split, a.splits, 32);
-    for (int i = tid; i < 2 * 16 * (a.ldq / 8); i += 256) {
-        const int half = i / (16 * (a.ldq / 8)), rest = i % (16 * (a.ldq / 8)), h = rest / (a.ldq / 8), d0 = (rest % (a.ldq / 8)) * 8;
-        u32x4 w = {0u, 0u, 0u, 0u};
-        if (h < nh) w = *reinterpret_cast<const u32x4*>(reinterpret_cast<const uint16_t*>(a.qcat) + (((size_t)b * a.heads + h0 + h) * 2 + half) * a.ldq + d0);
-        *reinterpret_cast<u32x4*>(qs + (half * 16 + h) * LQ + d0) = w;
+    const int ksteps = a.ldq / 32;
+    // this wave's part of the absorbed query, high and low halves: operand rows of sixteen heads
+    u32x4 qf[KSW][2];
+    {
+        const uint16_t* q = reinterpret_cast<const uint16_t*>(a.qcat) + ((size_t)b * a.heads + h0 + min(l16, nh - 1)) * 2 * a.ldq + g * 8;
+#pragma unroll
+        for (int s = 0; s < KSW; ++s)
+#pragma unroll
+            for (int h = 0; h < 2; ++h) {
+                qf[s][h] = u32x4{0u, 0u, 0u, 0u};
+                if (wave + 4 * s < ksteps) qf[s][h] = *reinterpret_cast<const u32x4*>(q + h * a.ldq + (wave + 4 * s) * 32);
+            }
     }
-    __syncthreads();
+    const KeyRange kr = split_range(p, a.window, split, a.splits, 32);
     const uint16_t* cache = reinterpret_cast<const uint16_t*>(a.cache);
     const float sc = a.scale * kLog2e;
-    const int ksteps = a.ldq / 32;
     float m = -INFINITY, l = 0.0f;
     f32x4 o[RPW];
 #pragma unroll
     for (int r = 0; r < RPW; ++r) o[r] = f32x4{0.f, 0.f, 0.f, 0.f};
     const int kp = tid & 15, cg = tid >> 4;  // staging: key pair, column group (8 columns, then every 128th)
-    for (int j0 = kr.lo / 32 * 32; j0 < kr.hi; j0 += 32) {
-        const int base = page_row(table, j0, a.shift);  // (a tile of 32 keys never crosses a page: pages hold 2^shift >= 32)
-        {   // rows of keys 2 kp, 2 kp + 1, transposed; keys outside the share read as zero (their rows may be another sequence's leftovers)
-            const bool in0 = j0 + 2 * kp >= kr.lo && j0 + 2 * kp < kr.hi, in1 = j0 + 2 * kp + 1 >= kr.lo && j0 + 2 * kp + 1 < kr.hi;
-            const uint16_t* r0 = cache + (size_t)(base + 2 * kp) * a.ldc;
+    u32x4 sx[NI], sy[NI], kf[KSW][2];        // the next tile: rows of keys 2 kp and 2 kp + 1; score operands
+    auto fetch = [&](const int j0, const int base) {
+        // keys outside the share read as zero in the value product (their rows may be another sequence's leftovers)
+        const bool in0 = j0 + 2 * kp >= kr.lo && j0 + 2 * kp < kr.hi, in1 = j0 + 2 * kp + 1 >= kr.lo && j0 + 2 * kp + 1 < kr.hi;
+        const uint16_t* k0 = cache + (size_t)(base + l16) * a.ldc + g * 8;
 #pragma unroll
-            for (int i = 0; i < (RT + 7) / 8; ++i) {
-                const int c0 = (cg + 16 * i) * 8;
-                if (c0 < RT * 16) {
-                    u32x4 x = {0u, 0u, 0u, 0u}, y = {0u, 0u, 0u, 0u};
-                    if (c0 < a.ldc) {
-                        if (in0) x = *reinterpret_cast<const u32x4*>(r0 + c0);
-                        if (in1) y = *reinterpret_cast<const u32x4*>(r0 + a.ldc + c0);
-                    }
+        for (int s = 0; s < KSW; ++s)
 #pragma unroll
-                    for (int j = 0; j < 4; ++j) {
-                        *reinterpret_cast<uint32_t*>(ct + (c0 + 2 * j) * LT + 2 * kp) = (x[j] & 0xFFFFu) | (y[j] << 16);
-                        *reinterpret_cast<uint32_t*>(ct + (c0 + 2 * j + 1) * LT + 2 * kp) = (x[j] >> 16) | (y[j] & 0xFFFF0000u);
-                    }
+            for (int t = 0; t < 2; ++t) {
+                kf[s][t] = u32x4{0u, 0u, 0u, 0u};
+                if (wave + 4 * s < ksteps) kf[s][t] = *reinterpret_cast<const u32x4*>(k0 + (size_t)t * 16 * a.ldc + (wave + 4 * s) * 32);
+            }
+        const uint16_t* r0 = cache + (size_t)(base + 2 * kp) * a.ldc;
+#pragma unroll
+        for (int i = 0; i < NI; ++i) {
+            const int c0 = (cg + 16 * i) * 8;
+            sx[i] = sy[i] = u32x4{0u, 0u, 0u, 0u};
+            if (c0 < RT * 16 && c0 < a.ldc) {
+                if (in0) sx[i] = *reinterpret_cast<const u32x4*>(r0 + c0);
+                if (in1) sy[i] = *reinterpret_cast<const u32x4*>(r0 + a.ldc + c0);
+            }
+        }
+    };
+    const int jend = (kr.hi - 1) / 32 * 32;  // (a tile of 32 keys never crosses a page: pages hold 2^shift >= 32)
+    int j0 = kr.lo / 32 * 32;
+    int next = 0;
+    if (kr.lo < kr.hi) {
+        fetch(j0, page_row(table, j0, a.shift));
+        next = page_row(table, min(j0 + 32, jend), a.shift);
+    }
+    for (; j0 < kr.hi && kr.lo < kr.hi; j0 += 32) {
+#pragma unroll
+        for (int i = 0; i < NI; ++i) {
+            const int c0 = (cg + 16 * i) * 8;
+            if (c0 < RT * 16) {
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    *reinterpret_cast<uint32_t*>(ct + (c0 + 2 * j) * LT + 2 * kp) = (sx[i][j] & 0xFFFFu) | (sy[i][j] << 16);
+                    *reinterpret_cast<uint32_t*>(ct + (c0 + 2 * j + 1) * LT + 2 * kp) = (sx[i][j] >> 16) | (sy[i][j] & 0xFFFF0000u);
                 }
             }
         }
         f32x4 s[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
-        for (int q = wave; q < ksteps; q += 4) {
-            const u32x4 qh = *reinterpret_cast<const u32x4*>(qs + l16 * LQ + q * 32 + g * 8);
-            const u32x4 ql = *reinterpret_cast<const u32x4*>(qs + (16 + l16) * LQ + q * 32 + g * 8);
 #pragma unroll
-            for (int t = 0; t < 2; ++t) {
-                const u32x4 kf = *reinterpret_cast<const u32x4*>(cache + (size_t)(base + t * 16 + l16) * a.ldc + q * 32 + g * 8);
-                s[t] = mfma16<BF16>(kf, qh, s[t]);
-                s[t] = mfma16<BF16>(kf, ql, s[t]);
+        for (int q = 0; q < KSW; ++q)
+            if (wave + 4 * q < ksteps) {
+#pragma unroll
+                for (int t = 0; t < 2; ++t) {
+                    s[t] = mfma16<BF16>(kf[q][t], qf[q][0], s[t]);
+                    s[t] = mfma16<BF16>(kf[q][t], qf[q][1], s[t]);
+                }
             }
-        }
 #pragma unroll
         for (int t = 0; t < 2; ++t) *reinterpret_cast<f32x4*>(sp + ((wave * 2 + t) * 64 + lane) * 4) = s[t];
         __syncthreads();
+        if (j0 + 32 < kr.hi) {
+            const int base = next;
+            next = page_row(table, min(j0 + 64, jend), a.shift);
+            fetch(j0 + 32, base);
+        }
         float mx = m;
 #pragma unroll
         for (int t = 0; t < 2; ++t) {
@@ -559,18 +670,17 @@ __global__ __launch_bounds__(256) void latent_decode_attention_kernel(const Late
         mx = fmaxf(mx, __shfl_xor(mx, 16));
         mx = fmaxf(mx, __shfl_xor(mx, 32));
         const float ms = mx == -INFINITY ? 0.0f : mx;
-        const float al = exp2f(m - ms);
+        const float al = exp2_fast(m - ms);
         m = mx;
         u32x4 ph, pl;
         float ls = 0.0f;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-            const float p0 = exp2f(s[j >> 1][2 * (j & 1)] - ms), p1 = exp2f(s[j >> 1][2 * (j & 1) + 1] - ms);
-            uint32_t a0, b0, a1, b1;
-            split16<BF16>(p0, a0, b0);
-            split16<BF16>(p1, a1, b1);
-            ph[j] = a0 | (a1 << 16);
-            pl[j] = b0 | (b1 << 16);
+            const float p0 = exp2_fast(s[j >> 1][2 * (j & 1)] - ms), p1 = exp2_fast(s[j >> 1][2 * (j & 1) + 1] - ms);
+            uint32_t hi, lo;
+            split16x2<BF16>(p0, p1, hi, lo);
+            ph[j] = hi;
+            pl[j] = lo;
             ls += p0 + p1;
         }
         l = l * al + ls;
@@ -588,15 +698,14 @@ __global__ __launch_bounds__(256) void latent_decode_attention_kernel(const Late
     l += __shfl_xor(l, 16);
     l += __shfl_xor(l, 32);
     if (l16 < nh) {
-        float* out = a.part + (((size_t)b * a.heads + h0 + l16) * a.splits + split) * (a.rank + 2);
-        if (wave == 0 && g == 0) { out[0] = m; out[1] = l; }
+        const int r4 = part_stride(a.rank) - 4;
+        float* out = a.part + (((size_t)b * a.heads + h0 + l16) * a.splits + split) * (r4 + 4);
+        if (wave == 0 && g == 0) { out[r4] = m; out[r4 + 1] = l; }
 #pragma unroll
-        for (int r = 0; r < RPW; ++r)
-#pragma unroll
-            for (int j = 0; j < 4; ++j) {
-                const int c = (wave * RPW + r) * 16 + g * 4 + j;
-                if (c < a.rank) out[2 + c] = o[r][j];
-            }
+        for (int r = 0; r < RPW; ++r) {
+            const int c = (wave * RPW + r) * 16 + g * 4;
+            if (c < r4) *reinterpret_cast<f32x4*>(out + c) = o[r];  // (columns past the rank: other parts of the rows, never read)
+        }
     }
 }
 
@@ -645,9 +754,10 @@ __global__ __launch_bounds__(256) void latent_decode_attention_scalar_kernel(con
         }
         __syncthreads();
     }
-    float* out = a.part + (at * a.splits + split) * (a.rank + 2);
-    if (tid == 0) { out[0] = m; out[1] = l; }
-    for (int r = tid; r < a.rank; r += 256) out[2 + r] = o[r];
+    const int r4 = part_stride(a.rank) - 4;
+    float* out = a.part + (at * a.splits + split) * (r4 + 4);
+    if (tid == 0) { out[r4] = m; out[r4 + 1] = l; }
+    for (int r = tid; r < r4; r += 256) out[r] = r < a.rank ? o[r] : 0.0f;
 }
 
 // ------------------------------------------------------------------------------------------------
@@ -662,77 +772,127 @@ struct LatentMergeArgs {
     int heads, rank, vdim, splits, ldg, ldy;
 };
 
-template <int DT>
-__global__ __launch_bounds__(256) void latent_decode_merge_kernel(const LatentMergeArgs a) {
+template <int DT, int BT>
+__global__ __launch_bounds__(256) void latent_decode_merge_kernel(const LatentMergeArgs a, const int batch) {
     using N = Num<DT>;
     using S = typename N::S;
     extern __shared__ __align__(16) unsigned char smem[];
-    float* o = reinterpret_cast<float*>(smem);  // [rank rounded up to 8]
-    float* f = o + ((a.rank + 7) & ~7);         // [splits]
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, head = blockIdx.y, b = blockIdx.z;
-    const float* part = a.part + ((size_t)b * a.heads + head) * a.splits * (a.rank + 2);
+    const int lo = (a.rank + 7) & ~7;
+    float* o = reinterpret_cast<float*>(smem);  // [BT][rank rounded up to 8]
+    float* f = o + BT * lo;                     // [256]
+    float* sum = f + 256;                       // [1024] partial sums of groups of splits
+    __shared__ float red[4];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, head = blockIdx.y, b0 = blockIdx.z * BT, nb = min(BT, batch - b0);
+    const int stride = part_stride(a.rank), r4 = stride - 4;
+    // what does not depend on the weights of the splits leaves first: this wave's eight rows of W_uv (lane: eight of the latent's
+    // columns, the first 512 of them), the gate and the sink
+    const int v0 = blockIdx.x * 32 + wave * 8, nv = min(8, a.vdim - v0);
+    const S* w = reinterpret_cast<const S*>(a.uv) + (size_t)(head * a.vdim + min(v0, a.vdim - 1)) * a.rank;
+    const bool vec = !(a.rank & 7);
+    auto full = [&](const int c0) { return c0 + 8 <= a.rank && nv > 0; };
+    Raw8<DT> wv[8];
+    auto weights = [&](const int c0) {
+#pragma unroll
+        for (int i = 0; i < 8; ++i) wv[i].load(w + (size_t)min(i, nv - 1) * a.rank + c0, vec);
+    };
+    if (full(lane * 8)) weights(lane * 8);
+    const int col = head * a.vdim + min(v0 + min(lane, 7), a.vdim - 1);  // (lanes 0 .. nv - 1: their own output column)
+    float gt[BT];
+#pragma unroll
+    for (int t = 0; t < BT; ++t) gt[t] = a.gate ? N::ld(reinterpret_cast<const S*>(a.gate) + (size_t)(b0 + min(t, nb - 1)) * a.ldg + col) : 0.0f;
     const float sink2 = a.sink ? N::ld(reinterpret_cast<const S*>(a.sink) + head) * kLog2e : -INFINITY;
-    float M = sink2;
-    for (int s = 0; s < a.splits; ++s) M = fmaxf(M, part[(size_t)s * (a.rank + 2)]);
-    if (tid < a.splits) f[tid] = exp2f(part[(size_t)tid * (a.rank + 2)] - M);
-    __syncthreads();
-    float L = a.sink ? exp2f(sink2 - M) : 0.0f;
-    for (int s = 0; s < a.splits; ++s) L = fmaf(part[(size_t)s * (a.rank + 2) + 1], f[s], L);
-    const float inv = 1.0f / L;
-    for (int r = tid; r < ((a.rank + 7) & ~7); r += 256) {
-        float t = 0.0f;
-        if (r < a.rank)
-            for (int s = 0; s < a.splits; ++s) t = fmaf(part[(size_t)s * (a.rank + 2) + 2 + r], f[s], t);
-        o[r] = t * inv;
+#pragma unroll 1
+    for (int t = 0; t < nb; ++t) {
+        const float* part = a.part + ((size_t)(b0 + t) * a.heads + head) * a.splits * stride;
+        // thread: four columns of the latent, every `groups`-th split; the first eight partials leave before the factors are known
+        const int quads = r4 / 4, groups = quads >= 256 ? 1 : 256 / quads;
+        const int grp = quads >= 256 ? 0 : tid / quads, quad0 = quads >= 256 ? tid : tid % quads;
+        const bool act = grp < groups;
+        auto at = [&](const int s, const int quad) { return *reinterpret_cast<const f32x4*>(part + (size_t)min(s, a.splits - 1) * stride + 4 * quad); };
+        f32x4 y[8];
+        if (act) {
+#pragma unroll
+            for (int u = 0; u < 8; ++u) y[u] = at(grp + groups * u, min(quad0, quads - 1));
+        }
+        const float pm = tid < a.splits ? part[(size_t)tid * stride + r4] : -INFINITY, pl = tid < a.splits ? part[(size_t)tid * stride + r4 + 1] : 0.0f;
+        const float M = fmaxf(sink2, block_max<256>(pm, red, tid));
+        const float pf = exp2f(pm - M);
+        f[tid] = tid < a.splits ? pf : 0.0f;
+        const float inv = 1.0f / (block_sum<256>(pl * pf, red, tid) + (a.sink ? exp2f(sink2 - M) : 0.0f));
+        for (int quad = quad0; quad < quads; quad += 256) {
+            f32x4 x = {0.f, 0.f, 0.f, 0.f};
+            if (act) {
+                for (int s = grp; s < a.splits; s += 8 * groups) {
+                    if (s != grp || quad != quad0) {
+#pragma unroll
+                        for (int u = 0; u < 8; ++u) y[u] = at(s + groups * u, quad);
+                    }
+#pragma unroll
+                    for (int u = 0; u < 8; ++u) x += y[u] * (s + groups * u < a.splits ? f[s + groups * u] : 0.0f);
+                }
+            }
+            if (groups == 1) {
+#pragma unroll
+                for (int j = 0; j < 4; ++j) if (act && 4 * quad + j < lo) o[t * lo + 4 * quad + j] = 4 * quad + j < a.rank ? x[j] * inv : 0.0f;
+            } else if (act) {
+                *reinterpret_cast<f32x4*>(sum + (grp * quads + quad) * 4) = x;
+            }
+        }
+        if (groups > 1) {
+            __syncthreads();
+            for (int r = tid; r < lo; r += 256) {
+                float x = 0.0f;
+                for (int g = 0; g < groups; ++g) x += r < r4 ? sum[g * r4 + r] : 0.0f;
+                o[t * lo + r] = r < a.rank ? x * inv : 0.0f;
+            }
+        } else {
+            for (int r = r4 + tid; r < lo; r += 256) o[t * lo + r] = 0.0f;
+        }
     }
     __syncthreads();
-    const int v0 = blockIdx.x * 32 + wave * 8, nv = min(8, a.vdim - v0);
     if (nv <= 0) return;
-    const S* w = reinterpret_cast<const S*>(a.uv) + (size_t)(head * a.vdim + v0) * a.rank;
-    float acc[8];
+    float acc[BT][8];
 #pragma unroll
-    for (int i = 0; i < 8; ++i) acc[i] = 0.0f;
-    const bool vec = !(a.rank & 7);
+    for (int t = 0; t < BT; ++t)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) acc[t][i] = 0.0f;
     for (int c0 = lane * 8; c0 < a.rank; c0 += 512) {
-        const int m = min(8, a.rank - c0);
+        if (full(c0)) {
+            if (c0 != lane * 8) weights(c0);
 #pragma unroll
-        for (int i = 0; i < 8; ++i) {
-            const S* wr = w + (size_t)min(i, nv - 1) * a.rank + c0;
-            if (m == 8) {
-                float v[8];
-                ld8<DT>(wr, v, vec);
+            for (int t = 0; t < BT; ++t) {
+                if (t >= nb) break;
+                float x[8];
 #pragma unroll
-                for (int j = 0; j < 8; ++j) acc[i] = fmaf(v[j], o[c0 + j], acc[i]);
-            } else {
-                for (int j = 0; j < m; ++j) acc[i] = fmaf(N::ld(wr + j), o[c0 + j], acc[i]);
+                for (int j = 0; j < 8; ++j) x[j] = o[t * lo + c0 + j];
+#pragma unroll
+                for (int i = 0; i < 8; ++i)
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) acc[t][i] = fmaf(wv[i].get(j), x[j], acc[t][i]);
             }
+        } else {
+#pragma unroll
+            for (int i = 0; i < 8; ++i)
+                if (i < nv)
+                    for (int j = c0; j < a.rank; ++j) {
+                        const float x = N::ld(w + (size_t)i * a.rank + j);
+#pragma unroll
+                        for (int t = 0; t < BT; ++t) acc[t][i] = t < nb ? fmaf(x, o[t * lo + j], acc[t][i]) : 0.0f;
+                    }
         }
     }
 #pragma unroll
-    for (int i = 0; i < 8; ++i) acc[i] = wave_sum_f(acc[i]);
-    if (lane < nv) {
-        float t = acc[0];
+    for (int t = 0; t < BT; ++t) {
+        if (t >= nb) break;
 #pragma unroll
-        for (int i = 1; i < 8; ++i) t = lane == i ? acc[i] : t;
-        const int col = head * a.vdim + v0 + lane;
-        if (a.gate) t *= sigmoid_f(N::ld(reinterpret_cast<const S*>(a.gate) + (size_t)b * a.ldg + col));
-        reinterpret_cast<S*>(a.y)[(size_t)b * a.ldy + col] = N::cvt(t);
+        for (int i = 0; i < 8; ++i) acc[t][i] = wave_sum_f(acc[t][i]);
+        float x = acc[t][0];
+#pragma unroll
+        for (int i = 1; i < 8; ++i) x = lane == i ? acc[t][i] : x;
+        if (a.gate) x *= sigmoid_f(gt[t]);
+        if (lane < nv) reinterpret_cast<S*>(a.y)[(size_t)(b0 + t) * a.ldy + col] = N::cvt(x);
     }
 }
-
-constexpr size_t kLatentMaxLds = 128 * 1024;
-
-// first use of a device (device_ctx()): the absorbed attention may take more than the default 64 KB of a CU's LDS
-bool latent_device_init() {
-    bool ok = true;
-#define TEAL_OPT(BF, RT) ok = ok && hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_decode_attention_kernel<BF, RT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)kLatentMaxLds) == hipSuccess
-    TEAL_OPT(false, 8); TEAL_OPT(false, 16); TEAL_OPT(false, 32); TEAL_OPT(true, 8); TEAL_OPT(true, 16); TEAL_OPT(true, 32);
-#undef TEAL_OPT
-    if (!ok) (void)hipGetLastError();
-    return ok;
-}
-
-inline size_t decode_lds(const int ldq, const int rt) { return (size_t)2 * 16 * (ldq + 8) * 2 + (size_t)rt * 16 * 36 * 2 + (size_t)4 * 2 * 64 * 4 * sizeof(float); }
 
 template <bool BF16, int NQ>
 int launch_prompt(const LatentPromptArgs& a, const int n_tiles, hipStream_t st) {
@@ -820,7 +980,11 @@ int teal_latent_step_query(const void* proj, int ldp, int kv0, int batch, const 
     const LatentStepArgs a = {{const_cast<void*>(proj), pos, nullptr, inv_freq, norm_w, cache, ldp, kv0, heads, dim, rot, rank, ldc, eps}, slot, table, uk, qcat, max_pages, page_shift, chunks, ldq};
     hipStream_t st = reinterpret_cast<hipStream_t>(stream);
     return with_dtype(dtype, [&](auto dt) {
-        hipLaunchKernelGGL((latent_step_query_kernel<decltype(dt)::value>), dim3(heads * chunks + (kv0 >= 0 ? 1 : 0), batch), dim3(256), (size_t)dim * sizeof(float), st, a);
+        constexpr int DT = decltype(dt)::value;
+        const int nx = heads * chunks + (kv0 >= 0 ? 1 : 0);
+        // (from eight tokens on a workgroup reads its weights once for four of them)
+        if (batch >= 8 && dim <= 2048) hipLaunchKernelGGL((latent_step_query_kernel<DT, 4>), dim3(nx, (batch + 3) / 4), dim3(256), (size_t)4 * dim * sizeof(float), st, a, batch);
+        else hipLaunchKernelGGL((latent_step_query_kernel<DT, 1>), dim3(nx, batch), dim3(256), (size_t)dim * sizeof(float), st, a, batch);
         return launched();
     });
 }
@@ -832,16 +996,14 @@ int teal_latent_step_attention(const void* qcat, int ldq, const void* cache, int
     if (splits < 1 || splits > 256 || batch > 65535 || heads > 65535 || page_shift < 5 || page_shift > 20 || (ldq & 31) || ldq < rank + rot || (ldc & 31) || ldc < rank + rot || rank + rot > 6144)
         return TEAL_ERR_SHAPE;
     if (!aligned16(qcat) || !aligned16(cache)) return TEAL_ERR_ALIGN;
-    if (part_bytes < (size_t)batch * heads * splits * (rank + 2) * sizeof(float)) return TEAL_ERR_WORKSPACE;
-    DeviceCtx* ctx = device_ctx();
-    if (!ctx) return TEAL_ERR_NO_DEVICE;
+    if (!aligned16(part)) return TEAL_ERR_ALIGN;
+    if (part_bytes < (size_t)batch * heads * splits * part_stride(rank) * sizeof(float)) return TEAL_ERR_WORKSPACE;
     const LatentDecodeArgs a = {qcat, cache, pos, slot, table, part, max_pages, page_shift, ldq, ldc, heads, rank, rot, window, splits, scale};
     hipStream_t st = reinterpret_cast<hipStream_t>(stream);
     const int rt = rank <= 128 ? 8 : (rank <= 256 ? 16 : 32);
-    const size_t lds = decode_lds(ldq, rt);
-    if (dtype != TEAL_F32 && rank <= 512 && ldq == ldc && lds <= kLatentMaxLds && (lds <= 64 * 1024 || ctx->latent_lds_ok)) {
+    if (dtype != TEAL_F32 && rank <= 512 && ldq == ldc && ldq <= 32 * kStepKSteps) {
         const dim3 grid(splits, (heads + 15) / 16, batch), block(256);
-#define TEAL_LD(BF, RT) hipLaunchKernelGGL((latent_decode_attention_kernel<BF, RT>), grid, block, lds, st, a)
+#define TEAL_LD(BF, RT) hipLaunchKernelGGL((latent_decode_attention_kernel<BF, RT>), grid, block, 0, st, a)
         if (dtype == TEAL_BF16) { if (rt == 8) TEAL_LD(true, 8); else if (rt == 16) TEAL_LD(true, 16); else TEAL_LD(true, 32); }
         else if (dtype == TEAL_F16) { if (rt == 8) TEAL_LD(false, 8); else if (rt == 16) TEAL_LD(false, 16); else TEAL_LD(false, 32); }
         else return TEAL_ERR_DTYPE;
@@ -858,11 +1020,14 @@ int teal_latent_step_merge(const float* part, int splits, const void* uv, const 
                            int vdim, int dtype, void* stream) {
     if (!part || !uv || !y || batch <= 0 || heads <= 0 || rank <= 0 || vdim <= 0 || splits < 1) return TEAL_ERR_ARG;
     if (splits > 256 || rank > 8192 || batch > 65535 || heads > 65535 || ldy < heads * vdim || (gate && ldg < heads * vdim)) return TEAL_ERR_SHAPE;
-    if (!aligned16(uv)) return TEAL_ERR_ALIGN;
+    if (!aligned16(uv) || !aligned16(part)) return TEAL_ERR_ALIGN;
     const LatentMergeArgs a = {part, uv, sink, gate, y, heads, rank, vdim, splits, ldg, ldy};
     hipStream_t st = reinterpret_cast<hipStream_t>(stream);
     return with_dtype(dtype, [&](auto dt) {
-        hipLaunchKernelGGL((latent_decode_merge_kernel<decltype(dt)::value>), dim3((vdim + 31) / 32, heads, batch), dim3(256), (size_t)(rank + 8 + splits) * sizeof(float), st, a);
+        constexpr int DT = decltype(dt)::value;
+        const int nx = (vdim + 31) / 32;
+        if (batch >= 8 && rank <= 2048) hipLaunchKernelGGL((latent_decode_merge_kernel<DT, 4>), dim3(nx, heads, (batch + 3) / 4), dim3(256), (size_t)(4 * ((rank + 7) & ~7) + 1280) * sizeof(float), st, a, batch);
+        else hipLaunchKernelGGL((latent_decode_merge_kernel<DT, 1>), dim3(nx, heads, batch), dim3(256), (size_t)(((rank + 7) & ~7) + 1280) * sizeof(float), st, a, batch);
         return launched();
     });
 }

@@ -40,6 +40,28 @@ __device__ __forceinline__ void ld8(const typename Num<DT>::S* __restrict__ p, f
     }
 }
 
+// eight consecutive elements as loaded: request early, convert where they are used
+template <int DT>
+struct Raw8 {
+    u32x4 w[DT == TEAL_F32 ? 2 : 1];
+    __device__ __forceinline__ void load(const typename Num<DT>::S* __restrict__ p, const bool vec) {
+        if (vec) {
+            w[0] = *reinterpret_cast<const u32x4*>(p);
+            if constexpr (DT == TEAL_F32) w[1] = *reinterpret_cast<const u32x4*>(p + 4);
+        } else {
+#pragma unroll
+            for (int j = 0; j < 8; ++j) {
+                if constexpr (DT == TEAL_F32) w[j >> 2][j & 3] = __float_as_uint(p[j]);
+                else w[0][j >> 1] = (j & 1) ? w[0][j >> 1] | ((uint32_t)p[j] << 16) : (uint32_t)p[j];
+            }
+        }
+    }
+    __device__ __forceinline__ float get(const int j) const {
+        if constexpr (DT == TEAL_F32) return __uint_as_float(w[j >> 2][j & 3]);
+        else return bits_to_float((j & 1) ? w[0][j >> 1] >> 16 : w[0][j >> 1] & 0xFFFFu, DT == TEAL_BF16);
+    }
+};
+
 // sum over the NT threads of a workgroup (red: NT / 64 floats of LDS, free on entry after a barrier); every thread gets it
 template <int NT>
 __device__ __forceinline__ float block_sum(float v, float* red, const int tid) {

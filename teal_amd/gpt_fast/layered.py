@@ -234,6 +234,7 @@ class LatentAttention(nn.Module):
     padded with zero rows to whole 64-column tiles; `wo` reads the padded concatenation of the heads."""
 
     args = LatentAttentionArgs
+    MAX_SPLITS = 64
 
     def __init__(self, cfg: LayeredArgs, index: int, a: LatentAttentionArgs):
         super().__init__()
@@ -313,10 +314,10 @@ class LatentAttention(nn.Module):
         return self.wo(y)
 
     def splits(self, batch: int, max_pos: int, dtype: torch.dtype) -> int:
-        """workgroups the cached rows of one sequence are split over: about one per CU, two 32-key tiles each at least"""
+        """workgroups the cached rows of one sequence are split over: two per CU in all, one 32-key tile each at least"""
         groups = self.a.heads if dtype == torch.float32 else -(-self.a.heads // 16)
         tiles = min(self.window, max_pos + 1) // 32 + 1
-        return max(1, min(-(-tiles // 2), -(-256 // (batch * groups)), 32))
+        return max(1, min(tiles, 512 // (batch * groups), self.MAX_SPLITS))
 
     def attend(self, proj: torch.Tensor, b: StepBatch, y: Optional[torch.Tensor] = None, buffers=None) -> torch.Tensor:
         """the step's attention on a computed projection: append the cache row, attend, merge -> the wo projection's input"""
@@ -325,7 +326,7 @@ class LatentAttention(nn.Module):
         splits = self.splits(n, b.max_pos, proj.dtype)
         if buffers is None:
             qcat = K.latent_qcat(n, a.heads, pool.shape[-1], proj.dtype, proj.device)
-            part = torch.empty(n * a.heads * splits * (a.kv_rank + 2), device=proj.device, dtype=torch.float32)
+            part = K.latent_part(n, a.heads, splits, a.kv_rank, proj.device)
         else:
             qcat, part = buffers
         K.latent_step_query(proj, self.kv0 if own else -1, b.pos, b.slot, b.cache.table, PAGE_SHIFT, self.inv_freq, self.kv_norm, self.eps, self.uk, a.heads,

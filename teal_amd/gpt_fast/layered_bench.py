@@ -1,0 +1,131 @@
+"""Throughput of a layered design next to the Llama stack at equal sizes (bench.py --layered): random weights, bf16.
+
+Per size: prompt passes (tokens/s), dense decoding at batch 1 through both fused engines (tokens/s and microseconds per stage), and
+batched decode steps (the layered design's paged step against the Llama stack's module path, both replayed from a hipGraph)."""
+from __future__ import annotations
+
+import time
+from typing import Dict, List
+
+import torch
+
+from .. import runtime
+from . import layered
+from .engine import DecodeEngine
+from .generate import relayout_for_engine
+from .layered_engine import LayeredEngine
+from .model import ModelArgs, Transformer
+from .serving import BatchEngine
+
+DEV = "cuda"
+
+
+def _median_ms(fn, reps: int, warm: int = 3) -> float:
+    """median time of one call, device work included"""
+    for _ in range(warm):
+        fn()
+    ts = []
+    for _ in range(reps):
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        fn()
+        torch.cuda.synchronize()
+        ts.append((time.perf_counter() - t0) * 1e3)
+    return sorted(ts)[len(ts) // 2]
+
+
+def _graphed(fn):
+    s = torch.cuda.Stream()
+    s.wait_stream(torch.cuda.current_stream())
+    with torch.cuda.stream(s):
+        fn()
+        fn()
+    torch.cuda.current_stream().wait_stream(s)
+    torch.cuda.synchronize()
+    g = torch.cuda.CUDAGraph()
+    with runtime.graph_capture(g):
+        fn()
+    return g.replay
+
+
+def llama_like(cfg: layered.LayeredArgs, dtype, max_seq: int) -> Transformer:
+    """the Llama stack at the layered model's width, depth, heads, feed-forward and vocabulary"""
+    mx = cfg.layers[0].mixer
+    args = ModelArgs(block_size=max_seq, vocab_size=cfg.vocab_size, n_layer=cfg.n_layer, n_head=mx.heads, dim=cfg.dim, intermediate_size=cfg.layers[0].mlp.ff)
+    with torch.device("meta"):
+        model = Transformer(args).to(dtype)
+    model = model.to_empty(device=DEV)
+    g = torch.Generator(device=DEV).manual_seed(5)
+    with torch.no_grad():
+        for n, p in model.named_parameters():
+            p.requires_grad_(False)
+            if n.endswith("norm.weight"):
+                p.fill_(1.0)
+            else:
+                p.copy_(torch.randn(p.shape, device=DEV, generator=g) * 0.02)
+    model.eval()
+    relayout_for_engine(model)
+    return model
+
+
+@torch.no_grad()
+def run(name: str, n_layer: int, prompts: List[int], contexts: List[int], batches: List[int], reps: int = 20, log=print) -> Dict:
+    dtype = torch.bfloat16
+    runtime.init()
+    cfg = layered.LayeredArgs.from_name(name, n_layer)
+    model = layered.build_layered_model(cfg, DEV, dtype)
+    max_seq = max(prompts + contexts) + 64
+    base = llama_like(cfg, dtype, max_seq)
+    out: Dict = {"model": name, "n_layer": n_layer, "dtype": "bf16", "prompt": {}, "decode": {}, "batch": {}, "stages": {}}
+    tok = torch.randint(0, cfg.vocab_size, (max_seq,), generator=torch.Generator().manual_seed(1))
+
+    base.setup_caches(1, max_seq)
+    eng = BatchEngine(model, max_tokens=max_seq, max_requests=2)
+    for T in prompts:
+        ids = tok[:T].tolist()
+
+        def ours():
+            eng.step([("p", ids, [T - 1])])
+            eng.release("p")
+
+        idx, pos = tok[:T].view(1, -1).to(DEV), torch.arange(T, device=DEV)
+        a, b = _median_ms(ours, 7), _median_ms(lambda: base(idx, pos), 7)
+        out["prompt"][T] = {"tokens_per_s": T / a * 1e3, "llama_tokens_per_s": T / b * 1e3}
+        log(f"[{name}] prompt {T}: {out['prompt'][T]}")
+    del eng
+
+    model.setup_caches(1, max_seq)
+    fused = LayeredEngine(model)
+    lead = DecodeEngine(base, [dict.fromkeys(("q", "k", "v", "o", "gate", "up", "down"), -1.0) for _ in base.layers])
+    for ctx in contexts:
+        row = {}
+        for key, e in (("tokens_per_s", fused), ("llama_tokens_per_s", lead)):
+            e.tok_buf.fill_(7)
+            e.pos_buf.fill_(ctx)
+            step = _graphed(lambda e=e: e(e.tok_buf, e.pos_buf))
+            row[key] = 1e3 / (_median_ms(lambda: [step() for _ in range(10)], reps) / 10)
+        out["decode"][ctx] = row
+        log(f"[{name}] decode, context {ctx}: {row}")
+    fused.pos_buf.fill_(contexts[0])
+    out["stages"]["ours"] = fused.stage_times()
+    lead.pos_buf.fill_(contexts[0])
+    if lead.att_split and lead.att_fused_merge:
+        lt = lead.stage_times()
+        out["stages"]["llama"] = {k: {"us": lt[k], "bytes": lt["bytes"][k]} for k in lt["bytes"]}
+    for who, st in out["stages"].items():
+        log(f"[{name}] stages {who}: " + ", ".join(f"{k} {v['us']:.1f} us ({v['bytes'] / v['us'] / 8e6:.2f} of 8 TB/s)" for k, v in st.items()))
+    del fused, lead
+
+    for B in batches:
+        ctx = contexts[-1]
+        model.max_seq_length = base.max_seq_length = -1
+        model.setup_caches(B, ctx + 8)
+        base.setup_caches(B, ctx + 8)
+        idx, pos = tok[:B].view(B, 1).to(DEV, torch.int32), torch.tensor([ctx], device=DEV, dtype=torch.int32)
+        row = {}
+        for key, m in (("tokens_per_s", model), ("llama_tokens_per_s", base)):
+            step = _graphed(lambda m=m: m(idx, pos))
+            row[key] = B * 1e3 / (_median_ms(lambda: [step() for _ in range(4)], reps) / 4)
+        out["batch"][B] = row
+        log(f"[{name}] batch {B}, context {ctx}: {row}")
+    return out

@@ -83,7 +83,7 @@ class LayeredEngine(DecodeLoop):
         for m in mixes:
             key = (m.a.heads, self.cache.pools[m.owner].shape[-1])
             self.qcat[key] = K.latent_qcat(1, *key, dt, dev)
-        self.part = z(max(m.a.heads * 32 * (m.a.kv_rank + 2) for m in mixes), dtype=torch.float32)
+        self.part = max((K.latent_part(1, m.a.heads, m.MAX_SPLITS, m.a.kv_rank, dev) for m in mixes), key=torch.numel)
         self.vocab_pad = model.output.weight.shape[0]
         self.logits_pad = z(self.vocab_pad, dtype=torch.float32)
         self.logits = self.logits_pad[: self.cfg.vocab_size].view(1, 1, -1)
@@ -152,36 +152,75 @@ class LayeredEngine(DecodeLoop):
             _lib.check(rc, "teal_fused_gemv")
         return self._n.value
 
-    def __call__(self, idx: torch.Tensor, input_pos: torch.Tensor, hook=None) -> torch.Tensor:
+    STAGES = ("proj", "attend", "wo", "gate_up", "down", "head")
+
+    def __call__(self, idx: torch.Tensor, input_pos: torch.Tensor, only=STAGES) -> torch.Tensor:
         """idx: int32 [1, 1] token id, input_pos: int32 [1] position -> logits [1, 1, vocab] (fp32; the next call overwrites them).
-        hook(stage, layer): called before every launch group ("proj", "attend", "wo", "gate_up", "down", "head"); measurements only."""
+        `only` (measurements: stage_times): launch just these stages, on whatever the buffers hold from the last full step."""
         assert idx.dtype == torch.int32 and input_pos.dtype == torch.int32 and idx.numel() == 1
         self._stream = runtime.stream_ptr()
-        cb = hook or (lambda *a: None)
         b = StepBatch(self.cache, idx, input_pos, self.slot, self.max_pos)
         slabs = 0
         for i, (mix, gin, gout, y, win, wout, ff) in enumerate(self.launches):
             if i == 0:
                 gin.row_index = idx.data_ptr()
-            gin.nslabs = slabs
-            cb("proj", i)
-            self._gemv(gin, gout, self.dim)
-            cb("attend", i)
-            mix.attend(self.proj[:, : mix.proj.out_features], b, y, (self.qcat[(mix.a.heads, self.cache.pools[mix.owner].shape[-1])], self.part))
-            cb("wo", i)
-            slabs = self._gemv(win, wout, mix.wo.in_features)
+            if "proj" in only:
+                gin.nslabs = slabs
+                self._gemv(gin, gout, self.dim)
+            if "attend" in only:
+                mix.attend(self.proj[:, : mix.proj.out_features], b, y, (self.qcat[(mix.a.heads, self.cache.pools[mix.owner].shape[-1])], self.part))
+            if "wo" in only:
+                slabs = self._gemv(win, wout, mix.wo.in_features)
             if ff is not None:
                 fin, fout, din, dout, Z = ff
-                fin.nslabs = slabs
-                cb("gate_up", i)
-                self._gemv(fin, fout, self.dim)
-                cb("down", i)
-                slabs = self._gemv(din, dout, Z)
-        hin, hout = self.head
-        hin.nslabs = slabs
-        cb("head", -1)
-        self._gemv(hin, hout, self.dim)
+                if "gate_up" in only:
+                    fin.nslabs = slabs
+                    self._gemv(fin, fout, self.dim)
+                if "down" in only:
+                    slabs = self._gemv(din, dout, Z)
+        if "head" in only:
+            hin, hout = self.head
+            hin.nslabs = slabs
+            self._gemv(hin, hout, self.dim)
         return self.logits
+
+    @torch.no_grad()
+    def stage_times(self, reps: int = 20) -> Dict[str, Dict[str, float]]:
+        """Microseconds per launch group and layer — a hipGraph of that one stage over every layer, its launch boundaries included — and
+        the bytes a dense step has to move for it.  Run after a full step: a stage works on what the buffers hold."""
+        m, out, el = self.model, {}, 2
+        pos = int(self.pos_buf.item())
+        mean = lambda f: sum(f(b) for b in m.layers) / len(m.layers)  # noqa: E731
+
+        def attention_bytes(b):
+            a = b.mix.a
+            keys = min(pos + 1, b.mix.window)
+            return el * (b.mix.uk.numel() + b.mix.uv.numel() + keys * (a.kv_rank + a.rot_dim) + b.mix.proj.out_features + b.mix.nv)
+
+        size = {"proj": mean(lambda b: el * b.mix.proj.weight.numel()), "attend": mean(attention_bytes), "wo": mean(lambda b: el * b.mix.wo.weight.numel()),
+                "gate_up": mean(lambda b: el * b.mlp.gate_up.weight.numel() if b.mlp is not None else 0),
+                "down": mean(lambda b: el * b.mlp.down.weight.numel() if b.mlp is not None else 0), "head": el * m.output.weight.numel()}
+        for stage in self.STAGES:
+            s = torch.cuda.Stream()
+            s.wait_stream(torch.cuda.current_stream())
+            with torch.cuda.stream(s):
+                self(self.tok_buf, self.pos_buf, only=(stage,))
+            torch.cuda.current_stream().wait_stream(s)
+            torch.cuda.synchronize()
+            g = torch.cuda.CUDAGraph()
+            with runtime.graph_capture(g):
+                self(self.tok_buf, self.pos_buf, only=(stage,))
+            ts = []
+            for r in range(reps + 3):
+                e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+                e0.record()
+                g.replay()
+                e1.record()
+                e1.synchronize()
+                if r >= 3:
+                    ts.append(e0.elapsed_time(e1) * 1e3 / (1 if stage == "head" else len(m.layers)))
+            out[stage] = {"us": sorted(ts)[len(ts) // 2], "bytes": size[stage]}
+        return out
 
     def sample_fused(self, logits: torch.Tensor, temperature: float = 1.0, top_k: Optional[int] = None, feed: bool = False) -> torch.Tensor:
         tok = self.tok_buf if feed else self.token

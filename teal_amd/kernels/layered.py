@@ -107,6 +107,11 @@ def latent_qcat(batch, heads, ldq, dtype, device):
     return torch.empty(batch, heads, *(() if dtype == torch.float32 else (2,)), ldq, device=device, dtype=dtype)
 
 
+def latent_part(batch, heads, splits, rank, device):
+    """the splits' partial results: weighted latent (padded to 4), max, sum"""
+    return torch.empty(batch * heads * splits * (-(-rank // 4) * 4 + 4), device=device, dtype=torch.float32)
+
+
 def latent_step_query(proj, kv0, pos, slot, table, page_shift, inv_freq, norm_w, eps, uk, heads, dim, rot, rank, pool, qcat):
     assert uk.is_contiguous() and table.is_contiguous() and pos.dtype == slot.dtype == table.dtype == torch.int32
     _run("teal_latent_step_query", _p(proj), _rows(proj), kv0, proj.shape[0], _p(pos), _p(slot), _p(table), table.shape[1], page_shift, _p(inv_freq), _p(norm_w),
