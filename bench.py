@@ -88,7 +88,21 @@ def parse():
     ap.add_argument("--profile-markers", action="store_true",
                     help="bracket the timed region with one marker dispatch each (compact_kernel on 64 elements) so that "
                          "scripts/summarize_prof.py can restrict a rocprofv3 trace / counter pass to the timed hipGraph replays")
+    ap.add_argument("--layered", nargs="*", default=None, metavar="NAME",
+                    help="instead of the decode workload: prompt, decode and batched-decode throughput of layered designs (names of "
+                         "layered.layered_configs; none given: Bolizen-1B Bolizen-7B) next to the Llama stack at equal sizes, one JSON line each")
     return ap.parse_args()
+
+
+def run_layered(names, n_layer):
+    """bench.py --layered: a few layers of each size are enough (every layer is the same work)"""
+    from teal_amd.gpt_fast import layered_bench
+    assert torch.cuda.is_available(), "--layered needs a GPU"
+    for name in names or ["Bolizen-1B", "Bolizen-7B"]:
+        res = layered_bench.run(name, n_layer or 4, prompts=[128, 512, 2048, 8192], contexts=[500, 4000], batches=[4, 16, 64],
+                                log=lambda *x: print(*x, file=sys.stderr, flush=True))
+        print(json.dumps(res), flush=True)
+        torch.cuda.empty_cache()
 
 
 def _dist_on():
@@ -597,6 +611,8 @@ def cpu_baseline(model, a, budget_s=14.0, n_layers_sampled=4):
 
 def main():
     a = parse()
+    if a.layered is not None:
+        return run_layered(a.layered, a.n_layer)
     if a.tuning:  # a forced launch geometry is a switch of the diagnostics build (libteal_hip_diag.so): the whole run goes through it
         os.environ["TEAL_LIB_FLAVOR"] = "diag"
     rank, world, local = dist_setup(a.gpus)

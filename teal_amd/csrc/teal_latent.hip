@@ -21,6 +21,7 @@ namespace teal {
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef _Float16 f16x8 __attribute__((ext_vector_type(8)));
 constexpr float kLog2e = 1.4426950408889634f;
+constexpr int kMaxStepSplits = 64;  // workgroups a sequence's cached rows may be split over
 constexpr int kStepKSteps = 20;  // 32-wide inner-dimension steps of the absorbed score product: cached rows of up to 640 elements
 
 template <bool BF16>
@@ -146,9 +147,9 @@ struct LatentPromptArgs {
 
 // S^T = K Q^T per tile: a lane then holds four consecutive keys of ONE query, which is the layout the second product's operand
 // needs when the keys of two 16-key tiles are interleaved per lane group — the weights never cross lanes.  O^T = V^T P^T.
-template <bool BF16, int DQP, int DVP, int NQ, int BN>
-__global__ __launch_bounds__(256) void latent_prompt_attention_kernel(const LatentPromptArgs a) {
-    constexpr int KS = DQP / 32, KT = BN / 16, VT = DVP / 16, LK = DQP + 8, LV = BN + 8, BM = 64 * NQ;
+template <bool BF16, int DQP, int DVP, int NQ, int BN, int NT>
+__global__ __launch_bounds__(NT) void latent_prompt_attention_kernel(const LatentPromptArgs a) {
+    constexpr int KS = DQP / 32, KT = BN / 16, VT = DVP / 16, LK = DQP + 8, LV = BN + 8, BM = NT / 4 * NQ;
     __shared__ __align__(16) uint16_t ks[BN * LK];
     __shared__ __align__(16) uint16_t vs[DVP * LV];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, g = lane >> 4;
@@ -197,12 +198,12 @@ __global__ __launch_bounds__(256) void latent_prompt_attention_kernel(const Late
     const int first = max(sq.klo, sq.start + q_first - a.window + 1);   // first position any of its queries sees
     const float sc = a.scale * kLog2e;
     // the next tile's keys and values are requested while a tile is worked on
-    constexpr int CK = DQP / 8, CV = BN / 8, NK = (BN * CK + 255) / 256, NV = (DVP * CV + 255) / 256;
+    constexpr int CK = DQP / 8, CV = BN / 8, NK = BN * CK / NT, NV = DVP * CV / NT;
     u32x4 kreg[NK], vreg[NV];
     auto fetch = [&](const int kt) {
 #pragma unroll
         for (int i = 0; i < NK; ++i) {
-            const int at = tid + 256 * i, key = at / CK, d0 = (at % CK) * 8;
+            const int at = tid + NT * i, key = at / CK, d0 = (at % CK) * 8;
             const size_t row = (size_t)min(sq.k0 + kt + key, a.S - 1);
             kreg[i] = u32x4{0u, 0u, 0u, 0u};
             if (kvec) {
@@ -218,12 +219,12 @@ __global__ __launch_bounds__(256) void latent_prompt_attention_kernel(const Late
         }
 #pragma unroll
         for (int i = 0; i < NV; ++i) {  // (S and every sequence's key base are multiples of 8: 16-byte loads)
-            const int at = tid + 256 * i, v = at / CV, c0 = (at % CV) * 8;
+            const int at = tid + NT * i, v = at / CV, c0 = (at % CV) * 8;
             vreg[i] = u32x4{0u, 0u, 0u, 0u};
             if (v < a.vdim && sq.k0 + kt + c0 < a.S) vreg[i] = *reinterpret_cast<const u32x4*>(vp + (size_t)v * a.S + sq.k0 + kt + c0);
         }
     };
-    static_assert((BN * CK) % 256 == 0 && (DVP * CV) % 256 == 0, "whole staging rounds");
+    static_assert((BN * CK) % NT == 0 && (DVP * CV) % NT == 0, "whole staging rounds");
     const int wq0 = sq.start + q_first + wave * NQ * 16;  // the wave's first query position
     const bool whole = q_first + (wave + 1) * NQ * 16 <= sq.nq;
     int kt = (first - sq.klo) / BN * BN;
@@ -232,12 +233,12 @@ __global__ __launch_bounds__(256) void latent_prompt_attention_kernel(const Late
         __syncthreads();
 #pragma unroll
         for (int i = 0; i < NK; ++i) {
-            const int at = tid + 256 * i;
+            const int at = tid + NT * i;
             *reinterpret_cast<u32x4*>(ks + (at / CK) * LK + (at % CK) * 8) = kreg[i];
         }
 #pragma unroll
         for (int i = 0; i < NV; ++i) {
-            const int at = tid + 256 * i;
+            const int at = tid + NT * i;
             *reinterpret_cast<u32x4*>(vs + (at / CV) * LV + (at % CV) * 8) = vreg[i];
         }
         __syncthreads();
@@ -779,9 +780,7 @@ __global__ __launch_bounds__(256) void latent_decode_merge_kernel(const LatentMe
     extern __shared__ __align__(16) unsigned char smem[];
     const int lo = (a.rank + 7) & ~7;
     float* o = reinterpret_cast<float*>(smem);  // [BT][rank rounded up to 8]
-    float* f = o + BT * lo;                     // [256]
-    float* sum = f + 256;                       // [1024] partial sums of groups of splits
-    __shared__ float red[4];
+    float* sum = o + BT * lo;                   // [1024] partial sums of groups of splits
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, head = blockIdx.y, b0 = blockIdx.z * BT, nb = min(BT, batch - b0);
     const int stride = part_stride(a.rank), r4 = stride - 4;
     // what does not depend on the weights of the splits leaves first: this wave's eight rows of W_uv (lane: eight of the latent's
@@ -810,41 +809,44 @@ __global__ __launch_bounds__(256) void latent_decode_merge_kernel(const LatentMe
         const bool act = grp < groups;
         auto at = [&](const int s, const int quad) { return *reinterpret_cast<const f32x4*>(part + (size_t)min(s, a.splits - 1) * stride + 4 * quad); };
         f32x4 y[8];
-        if (act) {
 #pragma unroll
-            for (int u = 0; u < 8; ++u) y[u] = at(grp + groups * u, min(quad0, quads - 1));
-        }
-        const float pm = tid < a.splits ? part[(size_t)tid * stride + r4] : -INFINITY, pl = tid < a.splits ? part[(size_t)tid * stride + r4 + 1] : 0.0f;
-        const float M = fmaxf(sink2, block_max<256>(pm, red, tid));
-        const float pf = exp2f(pm - M);
-        f[tid] = tid < a.splits ? pf : 0.0f;
-        const float inv = 1.0f / (block_sum<256>(pl * pf, red, tid) + (a.sink ? exp2f(sink2 - M) : 0.0f));
-        for (int quad = quad0; quad < quads; quad += 256) {
+        for (int u = 0; u < 8; ++u) y[u] = at((act ? grp : 0) + groups * u, min(quad0, quads - 1));
+        // every wave for itself: lane = split (kMaxStepSplits of them), no barriers
+        const float pm = lane < a.splits ? part[(size_t)lane * stride + r4] : -INFINITY, pl = lane < a.splits ? part[(size_t)lane * stride + r4 + 1] : 0.0f;
+        const float M = fmaxf(sink2, wave_max_f(pm));
+        const float pf = lane < a.splits ? exp2f(pm - M) : 0.0f;
+        const float inv = 1.0f / (wave_sum_f(pl * pf) + (a.sink ? exp2f(sink2 - M) : 0.0f));
+        for (int q0 = 0; q0 < quads; q0 += 256) {  // (uniform trip counts: the factors come from other lanes)
+            const int quad = min(q0 + quad0, quads - 1);
+            const bool mine = act && q0 + quad0 < quads;
             f32x4 x = {0.f, 0.f, 0.f, 0.f};
-            if (act) {
-                for (int s = grp; s < a.splits; s += 8 * groups) {
-                    if (s != grp || quad != quad0) {
+            for (int s0 = 0; s0 < a.splits; s0 += 8 * groups) {
+                const int s = s0 + (act ? grp : 0);
+                if (s0 != 0 || q0 != 0) {
 #pragma unroll
-                        for (int u = 0; u < 8; ++u) y[u] = at(s + groups * u, quad);
-                    }
+                    for (int u = 0; u < 8; ++u) y[u] = at(s + groups * u, quad);
+                }
 #pragma unroll
-                    for (int u = 0; u < 8; ++u) x += y[u] * (s + groups * u < a.splits ? f[s + groups * u] : 0.0f);
+                for (int u = 0; u < 8; ++u) {
+                    const float fs = __shfl(pf, min(s + groups * u, 63));
+                    if (s + groups * u < a.splits) x += y[u] * fs;
                 }
             }
-            if (groups == 1) {
-#pragma unroll
-                for (int j = 0; j < 4; ++j) if (act && 4 * quad + j < lo) o[t * lo + 4 * quad + j] = 4 * quad + j < a.rank ? x[j] * inv : 0.0f;
-            } else if (act) {
+            if (mine && groups > 1) {
                 *reinterpret_cast<f32x4*>(sum + (grp * quads + quad) * 4) = x;
+            } else if (mine) {
+#pragma unroll
+                for (int j = 0; j < 4; ++j) if (4 * quad + j < lo) o[t * lo + 4 * quad + j] = 4 * quad + j < a.rank ? x[j] * inv : 0.0f;
             }
         }
         if (groups > 1) {
-            __syncthreads();
+            __syncthreads();  // (the next token's writes wait behind the barrier below)
             for (int r = tid; r < lo; r += 256) {
                 float x = 0.0f;
                 for (int g = 0; g < groups; ++g) x += r < r4 ? sum[g * r4 + r] : 0.0f;
                 o[t * lo + r] = r < a.rank ? x * inv : 0.0f;
             }
+            if (t + 1 < nb) __syncthreads();
         } else {
             for (int r = r4 + tid; r < lo; r += 256) o[t * lo + r] = 0.0f;
         }
@@ -894,12 +896,12 @@ __global__ __launch_bounds__(256) void latent_decode_merge_kernel(const LatentMe
     }
 }
 
-template <bool BF16, int NQ>
+template <bool BF16, int NQ, int NT>
 int launch_prompt(const LatentPromptArgs& a, const int n_tiles, hipStream_t st) {
     const int dq = a.dim + a.rot;
-    const dim3 grid(n_tiles, a.heads), block(256);
-#define TEAL_LP(DQ, DV, BN) do { hipLaunchKernelGGL((latent_prompt_attention_kernel<BF16, DQ, DV, NQ, BN>), grid, block, 0, st, a); return launched(); } while (0)
-#define TEAL_LP_V(DQ) do { if (a.vdim <= 64) TEAL_LP(DQ, 64, 64); if (a.vdim <= 128) TEAL_LP(DQ, 128, 64); if constexpr (NQ == 1) TEAL_LP(DQ, 256, 32); } while (0)
+    const dim3 grid(n_tiles, a.heads), block(NT);
+#define TEAL_LP(DQ, DV, BN) do { hipLaunchKernelGGL((latent_prompt_attention_kernel<BF16, DQ, DV, NQ, BN, NT>), grid, block, 0, st, a); return launched(); } while (0)
+#define TEAL_LP_V(DQ) do { if (a.vdim <= 64) TEAL_LP(DQ, 64, 64); if (a.vdim <= 128) TEAL_LP(DQ, 128, 64); if constexpr (NT == 256) TEAL_LP(DQ, 256, 32); return TEAL_ERR_SHAPE; } while (0)
     if (dq <= 64) TEAL_LP_V(64);
     else if (dq <= 128) TEAL_LP_V(128);
     else if (dq <= 192) TEAL_LP_V(192);
@@ -962,8 +964,8 @@ int teal_latent_prompt_attention(const void* q, int ldq, const void* k, const vo
             hipLaunchKernelGGL((latent_prompt_attention_scalar_kernel<decltype(dt)::value>), dim3(n_tiles, heads), dim3(256), (size_t)(dim + rot + 512) * sizeof(float), st, a);
             return launched();
         });
-    if (dtype == TEAL_BF16) return tile == 128 ? launch_prompt<true, 2>(a, n_tiles, st) : launch_prompt<true, 1>(a, n_tiles, st);
-    if (dtype == TEAL_F16) return tile == 128 ? launch_prompt<false, 2>(a, n_tiles, st) : launch_prompt<false, 1>(a, n_tiles, st);
+    if (dtype == TEAL_BF16) return tile == 128 ? launch_prompt<true, 1, 512>(a, n_tiles, st) : launch_prompt<true, 1, 256>(a, n_tiles, st);
+    if (dtype == TEAL_F16) return tile == 128 ? launch_prompt<false, 1, 512>(a, n_tiles, st) : launch_prompt<false, 1, 256>(a, n_tiles, st);
     return TEAL_ERR_DTYPE;
 }
 
@@ -993,7 +995,7 @@ int teal_latent_step_attention(const void* qcat, int ldq, const void* cache, int
                                int page_shift, int batch, int heads, int rank, int rot, int window, float scale, int splits, float* part, size_t part_bytes, int dtype,
                                void* stream) {
     if (!qcat || !cache || !pos || !slot || !table || !part || batch <= 0 || heads <= 0 || rank <= 0 || rot < 0 || window <= 0 || max_pages <= 0) return TEAL_ERR_ARG;
-    if (splits < 1 || splits > 256 || batch > 65535 || heads > 65535 || page_shift < 5 || page_shift > 20 || (ldq & 31) || ldq < rank + rot || (ldc & 31) || ldc < rank + rot || rank + rot > 6144)
+    if (splits < 1 || splits > kMaxStepSplits || batch > 65535 || heads > 65535 || page_shift < 5 || page_shift > 20 || (ldq & 31) || ldq < rank + rot || (ldc & 31) || ldc < rank + rot || rank + rot > 6144)
         return TEAL_ERR_SHAPE;
     if (!aligned16(qcat) || !aligned16(cache)) return TEAL_ERR_ALIGN;
     if (!aligned16(part)) return TEAL_ERR_ALIGN;
@@ -1019,15 +1021,15 @@ int teal_latent_step_attention(const void* qcat, int ldq, const void* cache, int
 int teal_latent_step_merge(const float* part, int splits, const void* uv, const void* sink, const void* gate, int ldg, void* y, int ldy, int batch, int heads, int rank,
                            int vdim, int dtype, void* stream) {
     if (!part || !uv || !y || batch <= 0 || heads <= 0 || rank <= 0 || vdim <= 0 || splits < 1) return TEAL_ERR_ARG;
-    if (splits > 256 || rank > 8192 || batch > 65535 || heads > 65535 || ldy < heads * vdim || (gate && ldg < heads * vdim)) return TEAL_ERR_SHAPE;
+    if (splits > kMaxStepSplits || rank > 8192 || batch > 65535 || heads > 65535 || ldy < heads * vdim || (gate && ldg < heads * vdim)) return TEAL_ERR_SHAPE;
     if (!aligned16(uv) || !aligned16(part)) return TEAL_ERR_ALIGN;
     const LatentMergeArgs a = {part, uv, sink, gate, y, heads, rank, vdim, splits, ldg, ldy};
     hipStream_t st = reinterpret_cast<hipStream_t>(stream);
     return with_dtype(dtype, [&](auto dt) {
         constexpr int DT = decltype(dt)::value;
         const int nx = (vdim + 31) / 32;
-        if (batch >= 8 && rank <= 2048) hipLaunchKernelGGL((latent_decode_merge_kernel<DT, 4>), dim3(nx, heads, (batch + 3) / 4), dim3(256), (size_t)(4 * ((rank + 7) & ~7) + 1280) * sizeof(float), st, a, batch);
-        else hipLaunchKernelGGL((latent_decode_merge_kernel<DT, 1>), dim3(nx, heads, batch), dim3(256), (size_t)(((rank + 7) & ~7) + 1280) * sizeof(float), st, a, batch);
+        if (batch >= 8 && rank <= 2048) hipLaunchKernelGGL((latent_decode_merge_kernel<DT, 4>), dim3(nx, heads, (batch + 3) / 4), dim3(256), (size_t)(4 * ((rank + 7) & ~7) + 1024) * sizeof(float), st, a, batch);
+        else hipLaunchKernelGGL((latent_decode_merge_kernel<DT, 1>), dim3(nx, heads, batch), dim3(256), (size_t)(((rank + 7) & ~7) + 1024) * sizeof(float), st, a, batch);
         return launched();
     });
 }

@@ -29,8 +29,9 @@ CONFIGS = {
     "even": config(128, 256, [(mixer(4, 32, 16, 32, 64, 64), 192), (mixer(2, 48, 16, 64, 64, 65, kv_from=0), 128), (mixer(4, 16, 32, 16, 96, 20, base=2000.0), 256)], cap=12.0),
     # more than sixteen heads, a latent that is no multiple of 16 and one larger than 256
     "heads": config(192, 320, [(mixer(20, 24, 8, 16, 200, 40), 128), (mixer(17, 16, 8, 24, 200, 100, kv_from=0), None), (mixer(3, 64, 32, 80, 320, 96), 320)]),
-    # head sizes at the far end of the matrix-core tiles, and (second layer) beyond them
-    "large": config(256, 200, [(mixer(2, 160, 96, 144, 512, 50), 96), (mixer(1, 200, 64, 264, 520, 45), 64)]),
+    # head sizes and latents at the far end of the matrix-core tiles, and (second and third layer) beyond them
+    "large": config(256, 200, [(mixer(2, 160, 96, 144, 512, 50), 96), (mixer(1, 200, 64, 264, 520, 45), 64),
+                               (mixer(2, 16, 8, 16, 1060, 30), None)]),
 }
 
 
