@@ -35,6 +35,27 @@ CONFIGS = {
 }
 
 
+def random_config(seed):
+    """a configuration drawn from everything the design allows: widths in whole 64s (so that the fused step takes it) or not, heads, ranks,
+    windows and feed-forwards per layer, shared latents in any order"""
+    r = np.random.default_rng(1000 + seed)
+    pick = lambda *v: int(r.choice(v))  # noqa: E731
+    width = pick(64, 128, 192, 320, 448, 576, 1024, 1088) if seed % 3 else pick(40, 100, 152, 260)
+    layers, owners = [], []
+    for i in range(pick(2, 3, 4)):
+        donor = pick(*owners) if owners and r.random() < 0.5 else None
+        d = layers[donor][0] if donor is not None else None
+        rot = d["rot_dim"] if d else pick(2, 8, 12, 16, 32)
+        rank = d["kv_rank"] if d else pick(24, 32, 60, 64, 128, 144, 256, 320)
+        base = d["rot"]["base"] if d else float(pick(100, 10000, 1000000))
+        m = mixer(pick(1, 2, 3, 4, 6, 8), pick(8, 16, 24, 32, 64, 100), rot, pick(8, 16, 40, 48, 64, 96), rank, pick(3, 17, 31, 32, 33, 64, 65, 128, 500), base=base,
+                  kv_from=donor)
+        if donor is None:
+            owners.append(i)
+        layers.append((m, pick(24, 64, 160, 320, 1000, 1408) if r.random() < 0.8 else None))
+    return config(width, pick(48, 97, 256, 448, 1000), layers, eps=float(r.choice([1e-6, 1e-5, 1e-3])), cap=float(r.choice([5.0, 15.0, 30.0])))
+
+
 def random_tensors(cfg, seed=0, peak=3.0):
     """bf16 weights: matrices N(0, 1 / inputs), the query projections `peak` times that (one score stands out per query), norm weights
     around 1, biases and sinks of order 1"""

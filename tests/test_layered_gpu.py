@@ -13,7 +13,7 @@ import numpy as np
 import pytest
 import torch
 
-from layered_models import CONFIGS, error, random_tensors, random_tokens, save_checkpoint
+from layered_models import CONFIGS, error, random_config, random_tensors, random_tokens, save_checkpoint
 from oracle import layered_oracle as O
 
 pytestmark = pytest.mark.gpu
@@ -395,6 +395,37 @@ def test_sparsity_masks_the_projections(tmp_path_factory):
     dense = model.step_pass(StepBatch(eng.cache, dev[0], dev[1], dev[2], 40))
     assert 0.4 < sum(kept) / len(kept) < 0.8
     assert float(error(got, plain.double().cpu())) < 0.12 < float(error(dense, plain.double().cpu()))
+
+
+@pytest.mark.parametrize("seed", range(12))
+def test_random_configurations(seed, tmp_path):
+    """the whole path on configurations of all kinds: a batch of prompts, then decoding together and alone, 32-bit and bf16"""
+    from teal_amd.gpt_fast import registry
+    cfg = random_config(seed)
+    t = random_tensors(cfg, seed, peak=2.0)
+    path = save_checkpoint(tmp_path / "m", cfg, t)
+    n = 105
+    toks = random_tokens(cfg, n, seed)
+    want = O.forward(cfg, t, toks)
+    for dtype in (F32, BF16):
+        model = registry.load_model(path, DEV, dtype)
+        eng = engine(model)
+        assert (eng.fused is not None) == (dtype == BF16 and cfg["width"] % 64 == 0)
+        first = {"a": 70, "b": 1, "c": 34}
+        errs = [error(eng.step([(r, toks[:k], range(k)) for r, k in first.items()]), torch.cat([want[:k] for k in first.values()]))]
+        poison(eng)
+        live = dict(first)
+        for k in range(35):
+            if k == 12:
+                for r in ("b", "c"):
+                    eng.release(r)
+                    live.pop(r)
+                poison(eng)
+            got = eng.step([(r, [toks[p]], [0]) for r, p in live.items()])
+            errs.append(error(got, want[list(live.values())]))
+            live = {r: p + 1 for r, p in live.items()}
+        e = torch.cat(errs)
+        assert close(e, dtype), (cfg, dtype, int(e.argmax()), float(e.max()))
 
 
 # ---- generation ------------------------------------------------------------------------------------------------------------
