@@ -36,7 +36,7 @@ def rotate_pairs(x, positions, dims, base):
 
 
 def window_keys(p, size):
-    """Positions a query at p sees: itself and the size - 1 before it (size None: all before it)."""
+    """Positions a query at p attends to: the `size` most recent ones, its own included (size None: all of them)."""
     lo = 0 if size is None else max(0, p - int(size) + 1)
     return range(lo, p + 1)
 

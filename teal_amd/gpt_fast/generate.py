@@ -521,13 +521,14 @@ def main_layered(args, device: str) -> Dict:
     if fused:
         decoder = EngineDecoder(model, thresholds or [dict.fromkeys(("q", "g", "kv", "o", "gate", "up", "down"), KEEP_ALL)] * len(model.layers),
                                 args.compile, args.temperature, args.top_k)
+    prefill = model.prefill(graph=args.compile and not args.eager_prefill)
     tps, seqs = [], []
     for i in range(-1 if args.compile else 0, args.num_samples):
         torch.cuda.synchronize()
         t0 = time.perf_counter()
         if fused:
             prompt = torch.tensor(prompts[0], dtype=torch.int, device=device)
-            out = [generate(model, prompt, args.max_new_tokens, decoder, temperature=args.temperature, top_k=args.top_k).tolist()]
+            out = [generate(model, prompt, args.max_new_tokens, decoder, temperature=args.temperature, top_k=args.top_k, prefill=prefill).tolist()]
         else:
             new = generate_batch(model, [Request(p, args.max_new_tokens) for p in prompts], args.temperature, args.top_k, max_batch=args.max_batch,
                                  seed=1234 + i * len(prompts), graphs=args.compile)

@@ -13,6 +13,7 @@ The residual stream is fp32 throughout.  dtype fp16 / bf16 (matrix products and 
 """
 from __future__ import annotations
 
+import collections
 import json
 from dataclasses import dataclass, field
 from pathlib import Path
@@ -22,6 +23,7 @@ import numpy as np
 import torch
 import torch.nn as nn
 
+from .. import runtime
 from ..kernels import layered as K
 from ..monkeypatch import to_column_major
 from .paged import PAGE_SHIFT, PagedCache
@@ -57,7 +59,7 @@ class LatentAttentionArgs:
     kv_rank: int
     scale: float
     rope_base: float
-    window: Optional[int] = None     # a query sees itself and the window - 1 positions before it; None: all before it
+    window: Optional[int] = None     # a query attends to the most recent `window` positions, its own included; None: to all
     kv_from: Optional[int] = None    # reads the latents another layer caches
     sink: bool = True
     gate: bool = True
@@ -170,7 +172,10 @@ def named_config(name: str, n_layer: Optional[int] = None) -> Dict[str, Any]:
 # the two passes' shared metadata
 # ------------------------------------------------------------------------------------------------
 class PromptBatch:
-    """A ragged batch of prompt portions: per entry a slot, its first position and its tokens, packed back to back."""
+    """A ragged batch of prompt portions: per entry a slot, its first position and its tokens, packed back to back.
+
+    Everything a pass reads from it on the device lies in one buffer (`dev`, contents `flat`); two batches with the same `shape` differ
+    in the buffer's contents only, so a captured pass serves all of them."""
 
     def __init__(self, cache: PagedCache, entries, device):
         """entries: [(slot, start, tokens)]; the cache already has room for them and `sync` has run"""
@@ -189,14 +194,19 @@ class PromptBatch:
             q0 += n
             k0 += len(span)
         self.n_tokens, self.n_keys = q0, k0
-        flat = np.concatenate([np.concatenate(x) for x in (toks, pos, row)] + krow + [np.asarray(self.spans).ravel()]).astype(np.int32)
-        dev = torch.from_numpy(flat).to(device)
-        self.tokens, self.pos, self.row = dev[:q0], dev[q0:2 * q0], dev[2 * q0:3 * q0]
+        self.flat = np.concatenate([np.concatenate(x) for x in (toks, pos, row)] + krow + [np.asarray(self.spans).ravel()]).astype(np.int32)
+        dev = torch.from_numpy(self.flat).to(device)
+        self.dev, self.tokens, self.pos, self.row = dev, dev[:q0], dev[q0:2 * q0], dev[2 * q0:3 * q0]
         self.key_row = dev[3 * q0:3 * q0 + k0]
         self.seqs = dev[3 * q0 + k0:].view(-1, 5)
         self.device = device
         self._tiles: Dict[int, torch.Tensor] = {}
         self.packed: Dict[int, Any] = {}  # owner layer -> (latents, rotated key parts) of every key row of the batch
+
+    @property
+    def shape(self) -> tuple:
+        """(tokens, first position) of every entry"""
+        return tuple((n, start) for _, n, start, _, _ in self.spans)
 
     @property
     def longest(self) -> int:
@@ -298,6 +308,9 @@ class LatentAttention(nn.Module):
             y[:, self.nv:].zero_()
         return y
 
+    def prompt_tile(self, b: PromptBatch) -> int:
+        return K.latent_prompt_tile(self.a.dim, self.a.rot_dim, self.a.vdim, b.longest, self.uk.dtype)
+
     def prompt(self, h: torch.Tensor, b: PromptBatch) -> torch.Tensor:
         a, pool = self.a, b.cache.pools[self.owner]
         own = a.kv_from is None
@@ -308,7 +321,7 @@ class LatentAttention(nn.Module):
             b.packed[self.index] = K.latent_gather(pool, b.key_row, a.kv_rank, a.rot_dim)
         c, kr = b.packed[self.owner]
         k, vt = torch.matmul(c, self.uk.T), torch.matmul(self.uv, c.T)
-        tile = K.latent_prompt_tile(a.dim, a.rot_dim, a.vdim, b.longest, h.dtype)
+        tile = self.prompt_tile(b)
         y = K.latent_prompt_attention(proj, k, kr, vt, self.sink, self._gate(proj), self._y(b.n_tokens, h), b.seqs, b.tiles(tile), tile, a.heads, a.dim,
                                       a.rot_dim, a.vdim, self.window, a.scale)
         return self.wo(y)
@@ -393,6 +406,42 @@ class LayeredBlock(nn.Module):
         self.norm1, self.norm1b = _weight(cfg.dim), _weight(cfg.dim) if post else None
         self.norm2 = _weight(cfg.dim) if self.mlp is not None else None
         self.norm2b = _weight(cfg.dim) if self.mlp is not None and post else None
+
+
+class GraphedPrompt:
+    """prompt passes replayed from a hipGraph per shape of the batch: a pass of a short prompt is hundreds of launches of a few
+    microseconds.  A shape's first use runs eagerly (the warm-up a capture needs), its second is captured."""
+
+    MAX_TOKENS, MAX_GRAPHS = 256, 8  # longer prompts keep the GPU busy by themselves; least recently used graphs go first
+
+    def __init__(self, model: "LayeredTransformer"):
+        self.model = model
+        self._seen: set = set()
+        self._graphs: "collections.OrderedDict[tuple, tuple]" = collections.OrderedDict()
+
+    def __call__(self, b: PromptBatch, want: Sequence[int]) -> Optional[torch.Tensor]:
+        key = (b.shape, tuple(want), b.cache.version, id(b.cache))
+        if b.n_tokens > self.MAX_TOKENS or not len(want) or (key not in self._graphs and key not in self._seen):
+            if len(self._seen) >= 1024:
+                self._seen.clear()
+            self._seen.add(key)
+            return self.model.prompt_pass(b, want)
+        if key not in self._graphs:
+            rows = torch.tensor(list(want), dtype=torch.int32).to(b.device)
+            for ly in self.model.layers:
+                b.tiles(ly.mix.prompt_tile(b))  # (host-built: before the capture)
+            torch.cuda.synchronize()
+            while len(self._graphs) >= self.MAX_GRAPHS:
+                self._graphs.popitem(last=False)
+            g = torch.cuda.CUDAGraph()
+            with runtime.graph_capture(g):
+                logits = self.model.prompt_pass(b, rows)
+            self._graphs[key] = (g, b, rows, logits)
+        self._graphs.move_to_end(key)
+        g, static, _, logits = self._graphs[key]
+        static.dev.copy_(torch.from_numpy(b.flat))
+        g.replay()
+        return logits.clone()
 
 
 class LayeredTransformer(nn.Module):
@@ -508,10 +557,10 @@ class LayeredTransformer(nn.Module):
         return K.softcap(self.output(h), cfg.vocab_size, cfg.logit_softcap)
 
     @torch.no_grad()
-    def prompt_pass(self, b: PromptBatch, want: Sequence[int], hook=None) -> Optional[torch.Tensor]:
-        """logits (fp32) of the packed rows `want`; the cache rows of every token are written"""
-        w = torch.tensor(list(want), dtype=torch.int32).to(b.tokens.device) if len(want) else None
-        return self._run(b, lambda m, h: m.prompt(h, b), w, len(want), hook)
+    def prompt_pass(self, b: PromptBatch, want, hook=None) -> Optional[torch.Tensor]:
+        """logits (fp32) of the packed rows `want` (a sequence, or int32 on the device); the cache rows of every token are written"""
+        w = want if torch.is_tensor(want) else torch.tensor(list(want), dtype=torch.int32).to(b.tokens.device) if len(want) else None
+        return self._run(b, lambda m, h: m.prompt(h, b), w, 0 if w is None else w.numel(), hook)
 
     @torch.no_grad()
     def step_pass(self, b: StepBatch, hook=None) -> torch.Tensor:
@@ -533,6 +582,17 @@ class LayeredTransformer(nn.Module):
         toks = idx.cpu().numpy()
         b = PromptBatch(self.cache, [(i, start, toks[i]) for i in range(B)], idx.device)
         return self.prompt_pass(b, range(B * S)).view(B, S, -1)
+
+    def prefill(self, graph: bool = True):
+        """generate()'s `prefill` callable: the prompt of slot 0 -> logits [1, 1, vocab] of its last token"""
+        run = GraphedPrompt(self) if graph else self.prompt_pass
+
+        @torch.no_grad()
+        def call(prompt: torch.Tensor) -> torch.Tensor:
+            b = PromptBatch(self.cache, [(0, 0, prompt.view(-1).cpu().numpy())], prompt.device)
+            return run(b, [b.n_tokens - 1]).view(1, 1, -1)
+
+        return call
 
 
 # ------------------------------------------------------------------------------------------------

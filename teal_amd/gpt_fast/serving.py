@@ -15,13 +15,13 @@ import torch
 
 from .. import runtime
 from ..kernels import layered as K
-from .layered import LayeredTransformer, PromptBatch, StepBatch
+from .layered import GraphedPrompt, LayeredTransformer, PromptBatch, StepBatch
 from .layered_engine import LayeredEngine
 
 
 class BatchEngine:
-    """max_tokens: tokens the live requests are expected to hold together (the cache grows past it); graphs: replay a decode step from
-    a hipGraph per batch size (captured at its second use; the first is the eager warm-up)."""
+    """max_tokens: tokens the live requests are expected to hold together (the cache grows past it); graphs: replay decode steps (per
+    batch size) and short prompts (per shape of the batch) from hipGraphs, captured at their second use."""
 
     MAX_GRAPHS = 16
 
@@ -33,6 +33,7 @@ class BatchEngine:
         self.graphs = graphs
         # one running request, 16-bit: the fused step (same cache, same attention kernels)
         self.fused = LayeredEngine(model, cache=self.cache, max_seq=8) if LayeredEngine.supports(model, need_caches=False) is None else None
+        self.prompt = GraphedPrompt(model) if graphs else model.prompt_pass
         self._graphs: Dict[tuple, tuple] = {}
         self._seen: set = set()
 
@@ -51,6 +52,8 @@ class BatchEngine:
         if key not in self._graphs:
             dev = torch.from_numpy(flat).to(self.device)
             if key not in self._seen:
+                if len(self._seen) >= 1024:
+                    self._seen.clear()
                 self._seen.add(key)
                 return self._decode(dev, max_pos)
             torch.cuda.synchronize()
@@ -97,7 +100,8 @@ class BatchEngine:
             # (a copy: the next step overwrites the buffer of the fused step and of a graph)
             out = None if not want else logits.clone() if len(want) == len(batch) else logits[torch.tensor(want, device=self.device)]
         else:
-            out = self.model.prompt_pass(PromptBatch(self.cache, batch, self.device), want, hook)
+            b = PromptBatch(self.cache, batch, self.device)
+            out = self.prompt(b, want) if hook is None else self.model.prompt_pass(b, want, hook)
         for s, _, _ in batch:
             self.cache.trim(s)
         return out

@@ -40,7 +40,7 @@ def random_config(seed):
     windows and feed-forwards per layer, shared latents in any order"""
     r = np.random.default_rng(1000 + seed)
     pick = lambda *v: int(r.choice(v))  # noqa: E731
-    width = pick(64, 128, 192, 320, 448, 576, 1024, 1088) if seed % 3 else pick(40, 100, 152, 260)
+    width = pick(64, 128, 256, 320, 448, 576, 1024, 1088) if seed % 3 else pick(40, 100, 152, 260)
     layers, owners = [], []
     for i in range(pick(2, 3, 4)):
         donor = pick(*owners) if owners and r.random() < 0.5 else None
@@ -52,8 +52,8 @@ def random_config(seed):
                   kv_from=donor)
         if donor is None:
             owners.append(i)
-        layers.append((m, pick(24, 64, 160, 320, 1000, 1408) if r.random() < 0.8 else None))
-    return config(width, pick(48, 97, 256, 448, 1000), layers, eps=float(r.choice([1e-6, 1e-5, 1e-3])), cap=float(r.choice([5.0, 15.0, 30.0])))
+        layers.append((m, pick(24, 64, 160, 352, 1000, 1408) if r.random() < 0.8 else None))
+    return config(width, pick(48, 97, 256, 424, 1000), layers, eps=float(r.choice([1e-6, 1e-5, 1e-3])), cap=float(r.choice([5.0, 15.0, 30.0])))
 
 
 def random_tensors(cfg, seed=0, peak=3.0):

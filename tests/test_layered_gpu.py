@@ -362,6 +362,30 @@ def test_graph_replays_equal_eager_steps(name, dtype, batch, tmp_path_factory):
     assert b._graphs
 
 
+@pytest.mark.parametrize("name,dtype", [("even", BF16), ("ragged", F32), ("heads", BF16)])
+def test_graphed_prompts_equal_eager_ones(name, dtype, tmp_path_factory):
+    """the same shapes again and again with other tokens and on other pages: every replay against the oracle"""
+    cfg, t, model = setup(name, dtype, tmp_path_factory)
+    eng = engine(model, max_tokens=1024, max_requests=4, graphs=True)
+    toks, want = expected(name, cfg, t, 160, 3)
+    other, want2 = expected(name, cfg, t, 33, 2)
+    eng.step([("keep", toks[:90], [])])  # (occupies the first pages)
+    for rep in range(5):
+        got = eng.step([("x", toks[:20], [19]), ("y", other[:33], [0, 32])])
+        assert close(error(got, torch.cat([want[19:20], want2[[0, 32]]])), dtype), rep
+        got = eng.step([("x", toks[20:40], [19])])  # a portion
+        assert close(error(got, want[39:40]), dtype), rep
+        eng.release("x"), eng.release("y")
+        got = eng.step([("x", other[:20], [19]), ("y", toks[:33], [0, 32])])
+        assert close(error(got, torch.cat([want2[19:20], want[[0, 32]]])), dtype), rep
+        eng.release("y"), eng.release("x")
+        poison(eng)
+        if rep == 2:
+            eng.release("keep")
+    assert len(eng.prompt._graphs) == 2
+    assert close(error(eng.step([("long", toks, [0, 159])]), want[[0, 159]]), dtype)
+
+
 def test_sparsity_masks_the_projections(tmp_path_factory):
     """thresholds of the fused step = the unfused step on masked activations"""
     from teal_amd.gpt_fast.layered import StepBatch
