@@ -519,7 +519,7 @@ class LayeredTransformer(nn.Module):
         return PagedCache(widths, w.dtype, w.device, max_tokens, max_requests, None if None in windows else max(windows))
 
     def setup_caches(self, max_batch_size: int, max_seq_length: int):
-        """model.Transformer's contract: room for max_batch_size sequences of max_seq_length positions, slots 0 .. max_batch_size - 1"""
+        """model.Transformer's interface: room for max_batch_size sequences of max_seq_length positions, slots 0 .. max_batch_size - 1"""
         if self.max_seq_length >= max_seq_length and self.max_batch_size >= max_batch_size:
             return
         self.max_seq_length, self.max_batch_size = pad_to(max_seq_length, 8), max_batch_size
@@ -569,7 +569,7 @@ class LayeredTransformer(nn.Module):
 
     @torch.no_grad()
     def forward(self, idx: torch.Tensor, input_pos: Optional[torch.Tensor] = None) -> torch.Tensor:
-        """model.Transformer's contract: idx [B, S] at positions input_pos [S] of slots 0 .. B - 1 -> logits [B, S, vocab].  S = 1 keeps
+        """model.Transformer's interface: idx [B, S] at positions input_pos [S] of slots 0 .. B - 1 -> logits [B, S, vocab].  S = 1 keeps
         everything on the device (capturable into a hipGraph)."""
         assert self.cache is not None, "Caches must be initialized first"
         B, S = idx.shape

@@ -497,7 +497,7 @@ def test_generate_entry_point_and_command_line(tmp_path_factory):
         G.main(G.build_parser().parse_args(["--synthetic", "7B", "--precision", "fp32"]))
 
 
-def test_module_contract(tmp_path_factory):
+def test_module_interface(tmp_path_factory):
     """forward(idx, input_pos) as model.Transformer's: prompt of a batch, then a captured single-token step"""
     from teal_amd.gpt_fast.generate import GraphedDecoder
     cfg, t, model = setup("even", F32, tmp_path_factory)
