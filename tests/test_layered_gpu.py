@@ -244,6 +244,21 @@ def test_whole_prompts(name, dtype, tmp_path_factory):
         eng.release(n)
 
 
+@pytest.mark.parametrize("name", list(CONFIGS))
+def test_residual_after_every_layer(name, tmp_path_factory):
+    """32-bit: the residual stream layer by layer, of a prompt and of a decoded token"""
+    cfg, t, model = setup(name, F32, tmp_path_factory)
+    toks, want = random_tokens(cfg, 50, 6), []
+    O.forward(cfg, t, toks, layers_out=want)
+    eng, got, step = engine(model), [], []
+    eng.step([("a", toks[:49], [48])], hook=lambda i, x: got.append(x.double().cpu()))
+    eng.step([("a", toks[49:], [0])], hook=lambda i, x: step.append(x.double().cpu()))
+    assert len(got) == len(step) == len(want) == len(cfg["layers"])
+    for i, w in enumerate(want):
+        assert (got[i] - w[:49]).abs().max() < 1e-4 * w.abs().max(), i
+        assert (step[i] - w[49:]).abs().max() < 1e-4 * w.abs().max(), i
+
+
 @pytest.mark.parametrize("name,dtype", ALL)
 def test_token_by_token_equals_the_prompt(name, dtype, tmp_path_factory):
     """decoding from the second token on, through several pages and windows, over poisoned memory"""
@@ -305,6 +320,43 @@ def test_unequal_batch_and_reused_pages(name, dtype, tmp_path_factory):
         for r in ["e", *live]:
             eng.release(r)
         assert eng.cache.pages_in_use == 0
+
+
+@pytest.mark.parametrize("name,dtype", ALL)
+def test_wide_batches(name, dtype, tmp_path_factory):
+    """batches past eight (a workgroup then serves four tokens per weight read), not a multiple of four, and one past the tiles' rows"""
+    cfg, t, model = setup(name, dtype, tmp_path_factory)
+    toks, want = expected(name, cfg, t, 160, 3)
+    eng = engine(model, max_tokens=4096, max_requests=32)
+    for B in (10, 23):
+        at = {r: 1 + 5 * r for r in range(B)}
+        eng.step([(r, toks[:p], []) for r, p in at.items()])
+        for _ in range(3):
+            poison(eng)
+            got = eng.step([(r, toks[p:p + 1], [0]) for r, p in at.items()])
+            assert close(error(got, want[list(at.values())]), dtype), B
+            at = {r: p + 1 for r, p in at.items()}
+        for r in at:
+            eng.release(r)
+
+
+@pytest.mark.parametrize("dtype", [F32, BF16])
+def test_long_decoding_far_keys(dtype, tmp_path):
+    """hundreds of decoded tokens over many pages, most of them given back on the way; windows of several pages"""
+    from layered_models import config, mixer
+    from teal_amd.gpt_fast import registry
+    cfg = config(64, 120, [(mixer(2, 24, 8, 24, 40, 300), 80), (mixer(3, 16, 8, 16, 40, 190, kv_from=0), None), (mixer(1, 32, 8, 32, 64, 10), 40)])
+    t = random_tensors(cfg, 2)
+    model = registry.load_model(save_checkpoint(tmp_path / "m", cfg, t), DEV, dtype)
+    toks = random_tokens(cfg, 620, 5)
+    want = O.forward(cfg, t, toks)
+    eng = engine(model, max_tokens=64, max_requests=1)
+    got = [eng.step([("a", toks[:40], [39])])]
+    for p in range(40, 620):
+        if p % 50 == 0:
+            poison(eng)
+        got.append(eng.step([("a", toks[p:p + 1], [0])]))
+    assert close(error(torch.cat(got), want[39:]), dtype) and eng.cache.pages_in_use <= 6
 
 
 def test_bad_steps_are_refused(tmp_path_factory):
